@@ -64,23 +64,32 @@ __global__ void silu_mul_bf16x8_kernel(const uint16_t* __restrict__ gate, const 
   *reinterpret_cast<uint4*>(out + t * width + j) = uint4{ow[0], ow[1], ow[2], ow[3]};
 }
 
-// out[i] = parts[0][i] + parts[1][i] + ..., added in that order: the sum of the float32 partial
+// What a sum of partial products passes through on its way out: nothing, or max(z, 0)^2 (the activation of a feed-forward
+// without a gate).
+constexpr int kSumPlain = 0, kSumSquaredRelu = 1;
+__device__ __forceinline__ float sum_act(float z, int act) {
+  if (act != kSumSquaredRelu) return z;
+  const float r = fmaxf(z, 0.f);
+  return r * r;
+}
+
+// out[i] = act(parts[0][i] + parts[1][i] + ...), added in that order: the sum of the float32 partial
 // products that a matrix product with K split over workgroups leaves behind.
 template <typename TOut>
 __global__ void sum_partials_kernel(const float* __restrict__ parts, int n_parts, int64_t stride,
-                                    TOut* __restrict__ out, int64_t count) {
+                                    TOut* __restrict__ out, int64_t count, int act) {
   const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= count) return;
   float v = parts[i];
   for (int sp = 1; sp < n_parts; ++sp) v += parts[sp * stride + i];
-  out[i] = from_float<TOut>(v);
+  out[i] = from_float<TOut>(sum_act(v, act));
 }
 
 // Four elements a thread, eight parts in flight at a time (loads without a condition: past the last part the
 // last one is fetched again and not added).  count, stride % 4 == 0 and 16-byte aligned pointers.
 template <typename TOut>
 __global__ __launch_bounds__(256) void sum_partials_x4_kernel(const float* __restrict__ parts, int n_parts, int64_t stride,
-                                                              TOut* __restrict__ out, int64_t groups) {
+                                                              TOut* __restrict__ out, int64_t groups, int act) {
   const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= groups) return;
   const float* p = parts + 4 * i;
@@ -98,6 +107,7 @@ __global__ __launch_bounds__(256) void sum_partials_x4_kernel(const float* __res
       acc.w += in ? e[u].w : 0.f;
     }
   }
+  acc = float4{sum_act(acc.x, act), sum_act(acc.y, act), sum_act(acc.z, act), sum_act(acc.w, act)};
   if constexpr (sizeof(TOut) == 4) {
     *reinterpret_cast<float4*>(out + 4 * i) = acc;
   } else {
@@ -155,9 +165,9 @@ extern "C" int arle_silu_mul(const void* gate, const void* up, long long in_stri
   return arle_act_mul(gate, up, in_stride, out, dtype, tokens, width, block, kActSilu, stream);
 }
 
-// parts [n_parts][count] float32 (stride elements apart) -> out [count] float32 or bfloat16.
+// parts [n_parts][count] float32 (stride elements apart) -> out [count] float32 or bfloat16.  act: a kSum code.
 extern "C" int arle_sum_partials(const float* parts, int n_parts, long long stride, void* out, int out_dtype,
-                                 long long count, void* stream) {
+                                 long long count, int act, void* stream) {
   if (count == 0) return 0;
   if (n_parts < 1) return static_cast<int>(hipErrorInvalidValue);
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -166,16 +176,16 @@ extern "C" int arle_sum_partials(const float* parts, int n_parts, long long stri
     const int64_t groups = count / 4;
     const unsigned blocks = static_cast<unsigned>((groups + 255) / 256);
     if (out_dtype == kF32)
-      sum_partials_x4_kernel<float><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<float*>(out), groups);
+      sum_partials_x4_kernel<float><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<float*>(out), groups, act);
     else
-      sum_partials_x4_kernel<bf16><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<bf16*>(out), groups);
+      sum_partials_x4_kernel<bf16><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<bf16*>(out), groups, act);
     return launch_status();
   }
   const unsigned blocks = static_cast<unsigned>((count + 255) / 256);
   if (out_dtype == kF32)
-    sum_partials_kernel<float><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<float*>(out), count);
+    sum_partials_kernel<float><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<float*>(out), count, act);
   else
-    sum_partials_kernel<bf16><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<bf16*>(out), count);
+    sum_partials_kernel<bf16><<<blocks, 256, 0, s>>>(parts, n_parts, stride, static_cast<bf16*>(out), count, act);
   return launch_status();
 }
 

@@ -1,11 +1,14 @@
 // A mixture of experts: the router, and the experts' products over the tokens that chose them.
 //
-//   z = W_r h (32-bit sums),  s = sigmoid(z) or softmax(z) over all router outputs;  the `top` experts with the largest
-//   s + correction are chosen (ties: the lower index), where the experts form `groups` equal groups of neighbours among
-//   the `keep` groups with the largest such number in them only (the others count as minus infinity);  weight of a
-//   chosen expert = s / (sum of the chosen s + 1e-20) * scale, or without the division s * scale.
-//   expert e: down_e (silu(gate_e h) * (up_e h)).  Router outputs past the experts that have tensors stand for experts
-//   that hand back their input (`moe_identity` writes their rows).
+//   z = W_r h + bias (32-bit sums; bias optional),  s = sigmoid(z), softmax(z) over all router outputs, or z itself;  the
+//   `top` experts with the largest s + correction are chosen (ties: the lower index), where the experts form `groups`
+//   equal groups of neighbours among the `keep` groups with the largest such number in them only (the others count as
+//   minus infinity);  weight of a chosen expert = s / (sum of the chosen s + 1e-20) * scale, or without the division
+//   s * scale; where s is z itself, the softmax over the chosen z * scale.
+//   expert e: down_e (silu(gate_e h) * (up_e h)), or without a gate down_e (max(up_e h, 0)^2).  Router outputs past the
+//   experts that have tensors stand for experts that hand back their input (`moe_identity` writes their rows).  The
+//   router's kernel also makes the one number a token that a shared expert's output is multiplied by, sigmoid(w_s h),
+//   where the caller has one.
 //
 // `moe_route`: one workgroup a token.  `moe_expert`: a workgroup takes one expert, 64 consecutive rows of the step and 64
 // output columns; it lists the rows of its 64 that chose the expert (in row order) and multiplies only those, so no
@@ -43,7 +46,7 @@ constexpr int kRouteThreads = 256;
 // (eight consecutive entries a lane and step where the width allows, one otherwise: an order that depends on the
 // width alone); then the first wave picks the `top` experts one after the other.
 struct RouteRule {
-  int softmax;     // 0: s = sigmoid(z); 1: s = softmax(z)
+  int softmax;     // 0: s = sigmoid(z); 1: s = softmax(z); 2: s = z, and the weights are the softmax over the chosen z
   int groups;      // equal groups of neighbouring experts (1: no groups)
   int keep;        // groups among which the choice is made
   int normalize;   // 1: the chosen scores are divided by their sum
@@ -52,9 +55,12 @@ struct RouteRule {
 
 template <typename T, typename TW, bool VEC>
 __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __restrict__ x, long long x_stride,
-                                                                  const TW* __restrict__ w, const void* __restrict__ correction,
-                                                                  int c_dtype, int* __restrict__ ids, float* __restrict__ weights,
-                                                                  int width, int experts, int top, const RouteRule rule) {
+                                                                  const TW* __restrict__ w, const void* __restrict__ bias,
+                                                                  int b_dtype, const void* __restrict__ correction,
+                                                                  int c_dtype, const TW* __restrict__ shared_w,
+                                                                  float* __restrict__ shared_gate, int* __restrict__ ids,
+                                                                  float* __restrict__ weights, int width, int experts,
+                                                                  int top, const RouteRule rule) {
   extern __shared__ float route_lds[];   // [width] the row, then [experts] the scores, [experts] the choice numbers, [groups]
   float* xs = route_lds;
   float* score = route_lds + width;
@@ -65,8 +71,8 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
   const T* row = x + t * x_stride;
   for (int i = threadIdx.x; i < width; i += kRouteThreads) xs[i] = to_float(row[i]);
   __syncthreads();
-  for (int e = wave; e < experts; e += kRouteThreads / kWave) {
-    const TW* we = w + static_cast<int64_t>(e) * width;
+  for (int e = wave; e < experts + (shared_w ? 1 : 0); e += kRouteThreads / kWave) {
+    const TW* we = e < experts ? w + static_cast<int64_t>(e) * width : shared_w;
     float dot = 0.f;
     if (VEC) {
       for (int i = 8 * lane; i < width; i += 8 * kWave) {
@@ -78,7 +84,13 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
       for (int i = lane; i < width; i += kWave) dot = fmaf(xs[i], to_float(we[i]), dot);
     }
     dot = wave_sum(dot);
-    if (lane == 0) score[e] = rule.softmax ? dot : 1.0f / (1.0f + expf(-dot));
+    if (lane != 0) continue;
+    if (e == experts) {
+      shared_gate[t] = 1.0f / (1.0f + expf(-dot));
+      continue;
+    }
+    if (bias) dot += load_as_float(bias, b_dtype, e);
+    score[e] = rule.softmax ? dot : 1.0f / (1.0f + expf(-dot));
   }
   __syncthreads();
   // From here on the first wave works alone; the others only keep the barriers' count.
@@ -89,7 +101,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
       const int e = lane + j * kWave;
       s[j] = e < experts ? score[e] : (rule.softmax ? -INFINITY : 0.f);
     }
-    if (rule.softmax) {   // over all router outputs, in 32 bits: the largest logit taken off, one sum in a fixed order
+    if (rule.softmax == 1) {   // over all router outputs, in 32 bits: the largest logit taken off, one sum in a fixed order
       float top_z = -INFINITY;
 #pragma unroll
       for (int j = 0; j < kMaxExpertsPerLane; ++j) top_z = fmaxf(top_z, s[j]);
@@ -158,12 +170,13 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
   if (wave != 0) return;
   float sum = 0.f, mine = 0.f;   // lane k keeps the k-th chosen score (top <= 64)
   int mine_id = 0;
+  unsigned taken = 0;            // bit j: this lane's expert lane + 64 j has been chosen
   for (int k = 0; k < top; ++k) {
     Best b{-INFINITY, 0x7fffffff};
 #pragma unroll
     for (int j = 0; j < kMaxExpertsPerLane; ++j) {
       const int e = lane + j * kWave;
-      if (e < experts && s[j] >= 0.f && (choice[j] > b.v || (choice[j] == b.v && e < b.i))) {
+      if (e < experts && !(taken >> j & 1u) && (choice[j] > b.v || (choice[j] == b.v && e < b.i))) {
         b.v = choice[j];
         b.i = e;
       }
@@ -174,8 +187,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
     for (int j = 0; j < kMaxExpertsPerLane; ++j) {
       if (b.i == lane + j * kWave) {
         sv = s[j];
-        choice[j] = -INFINITY;
-        s[j] = -1.0f;   // taken: a score is never negative, so this marks it whatever its choice number was
+        taken |= 1u << j;
       }
     }
     sv = __shfl(sv, b.i % kWave, kWave);
@@ -184,6 +196,16 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
       mine = sv;
       mine_id = b.i;
     }
+  }
+  if (rule.softmax == 2) {   // the softmax over the chosen
+    const float top_z = wave_max(lane < top ? mine : -INFINITY);
+    const float e = lane < top ? expf(mine - top_z) : 0.f;
+    const float total = wave_sum(e);
+    if (lane < top) {
+      ids[t * top + lane] = mine_id;
+      weights[t * top + lane] = e / total * rule.scale;
+    }
+    return;
   }
   if (lane < top) {
     ids[t * top + lane] = mine_id;
@@ -213,13 +235,23 @@ __global__ __launch_bounds__(256) void moe_identity_kernel(const T* __restrict__
 constexpr int kEM = 64, kEN = 64, kEK = 16;
 constexpr int kExpertThreads = 256;
 
-// GATE_UP: w [experts, 2 N, K] (gate rows, then up rows), rows of x are tokens, out[(t top + k), n] = silu(g) u of
-// type T.  Else: w [experts, N, K], rows of x are t top + k, out float32 [(t top + k), n].
-template <typename T, bool GATE_UP>
+// Which of an expert's products a launch makes.
+//   kGateUp: w [experts, 2 N, K] (gate rows, then up rows), rows of x are tokens, out[(t top + k), n] = silu(g) u of type T
+//   kUp:     w [experts, N, K], rows of x are tokens, out[(t top + k), n] = max(u, 0)^2 of type T
+//   kDown:   w [experts, N, K], rows of x are t top + k, out float32 [(t top + k), n]
+constexpr int kDown = 0, kGateUp = 1, kUp = 2;
+
+__device__ __forceinline__ float squared_relu(float u) {
+  const float r = fmaxf(u, 0.f);
+  return r * r;
+}
+
+template <typename T, int MODE>
 __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __restrict__ x, long long x_stride,
                                                                     const T* __restrict__ w, const int* __restrict__ ids,
                                                                     void* __restrict__ out, int tokens, int top, int N,
                                                                     int K) {
+  constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
   __shared__ int list_t[kEM], list_k[kEM];
   __shared__ int count;
   __shared__ float as[kEK][kEM + 4];
@@ -255,7 +287,7 @@ __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __r
       const int gk = k0 + c, gn = n0 + r;
       float av = 0.f;
       if (r < rows && gk < K) {
-        const int64_t src = GATE_UP ? list_t[r] : static_cast<int64_t>(list_t[r]) * top + list_k[r];
+        const int64_t src = TOKENS ? list_t[r] : static_cast<int64_t>(list_t[r]) * top + list_k[r];
         av = to_float(x[src * x_stride + gk]);
       }
       as[c][r] = av;
@@ -304,6 +336,8 @@ __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __r
       if (GATE_UP) {
         const float g = acc[i][j];
         static_cast<T*>(out)[dst + n] = from_float<T>(g / (1.0f + expf(-g)) * acc_u[i][j]);
+      } else if (MODE == kUp) {
+        static_cast<T*>(out)[dst + n] = from_float<T>(squared_relu(acc[i][j]));
       } else {
         static_cast<float*>(out)[dst + n] = acc[i][j];
       }
@@ -326,10 +360,11 @@ constexpr int kMoeChunk = 256;     // rows of the step a workgroup looks through
 constexpr int kMoeCols = 128;      // weight rows of a tile (gate|up: 64 + 64)
 constexpr int kMoeLdsRow = 40;     // bfloat16 a weight row of 32 takes in LDS (80 bytes: no two lanes of a read on one bank)
 
-template <bool GATE_UP>
+template <int MODE>
 __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __restrict__ x, long long x_stride,
                                                               const bf16* __restrict__ w, const int* __restrict__ ids,
                                                               void* __restrict__ out, int tokens, int top, int N, int K) {
+  constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
   __shared__ int list_src[kMoeChunk], list_dst[kMoeChunk];
   __shared__ int wave_count[4];
   __shared__ __attribute__((aligned(16))) bf16 wt[kMoeCols * kMoeLdsRow];
@@ -348,7 +383,7 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
     for (int i = 0; i < wave; ++i) before += wave_count[i];
     if (slot >= 0) {
       const int rank = before + __popcll(chose & ((1ull << lane) - 1ull));
-      list_src[rank] = GATE_UP ? t : t * top + slot;
+      list_src[rank] = TOKENS ? t : t * top + slot;
       list_dst[rank] = t * top + slot;
     }
     __syncthreads();
@@ -412,7 +447,11 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
           const int col = n0 + 16 * j + n;
-          if (col < N) static_cast<float*>(out)[dst + col] = acc[j][i];
+          if (col >= N) continue;
+          if (MODE == kUp)
+            static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(acc[j][i]));
+          else
+            static_cast<float*>(out)[dst + col] = acc[j][i];
         }
       }
     }
@@ -433,11 +472,12 @@ __global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __rest
 constexpr int kBigCols = 256;       // weight rows of a tile
 constexpr int kBigRows = 64;        // listed rows of a group of four waves
 
-template <bool GATE_UP, int RG, int BK>
+template <int MODE, int RG, int BK>
 __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* __restrict__ x, long long x_stride,
                                                                     const bf16* __restrict__ w, const int* __restrict__ ids,
                                                                     void* __restrict__ out, int tokens, int top, int N,
                                                                     int K) {
+  constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
   constexpr int kThreads = 256 * RG, kWaves = 4 * RG, kRows = kBigRows * RG;
   constexpr int kLdsRow = BK + 8;                 // bfloat16 a row of BK takes in LDS (no two lanes of a read on one bank)
   constexpr int kLanesRow = BK / 8;               // lanes that copy one row of a tile, a piece of 8 each (whole lines)
@@ -463,7 +503,7 @@ __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* 
     for (int i = 0; i < wave; ++i) before += wave_count[i];
     if (slot >= 0) {
       const int rank = before + __popcll(chose & ((1ull << lane) - 1ull));
-      list_src[rank] = GATE_UP ? t : t * top + slot;
+      list_src[rank] = TOKENS ? t : t * top + slot;
       list_dst[rank] = t * top + slot;
     }
     __syncthreads();
@@ -569,7 +609,11 @@ __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* 
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
             const int col = n0 + cw * 64 + 16 * j + n;
-            if (col < N) static_cast<float*>(out)[dst + col] = acc[i][j][c];
+            if (col >= N) continue;
+            if (MODE == kUp)
+              static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(acc[i][j][c]));
+            else
+              static_cast<float*>(out)[dst + col] = acc[i][j][c];
           }
         }
       }
@@ -582,13 +626,15 @@ __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* 
 
 using namespace arle;
 
-// x [T, width] of x_dtype, w [experts, width] of w_dtype, correction [experts] or null; ids int32 [T, top], weights
-// float32 [T, top].
+// x [T, width] of x_dtype, w [experts, width] of w_dtype, bias and correction [experts] or null; shared_w [width] of
+// w_dtype with shared_gate float32 [T], or null; ids int32 [T, top], weights float32 [T, top].
 extern "C" int arle_moe_route(const void* x, long long x_stride, int x_dtype, const void* w, int w_dtype,
-                              const void* correction, int c_dtype, int* ids, float* weights, int tokens, int width,
-                              int experts, int top, float scale, int softmax, int groups, int keep, int normalize,
+                              const void* bias, int b_dtype, const void* correction, int c_dtype, const void* shared_w,
+                              float* shared_gate, int* ids, float* weights, int tokens, int width, int experts, int top,
+                              float scale, int softmax, int groups, int keep, int normalize,
                               void* stream) {
   if (tokens == 0) return 0;
+  if (softmax < 0 || softmax > 2 || (shared_w && !shared_gate)) return static_cast<int>(hipErrorInvalidValue);
   if (experts < 1 || experts > kWave * kMaxExpertsPerLane || top < 1 || top > experts || top > kWave || groups < 1 ||
       experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups))
     return static_cast<int>(hipErrorInvalidValue);
@@ -596,7 +642,7 @@ extern "C" int arle_moe_route(const void* x, long long x_stride, int x_dtype, co
   const RouteRule rule{softmax, groups, keep, normalize, scale};
   const size_t lds = static_cast<size_t>(width + 2 * experts + groups) * sizeof(float);
   if (lds > 60 * 1024) return static_cast<int>(hipErrorInvalidValue);
-  const bool vec = width % 8 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
+  const bool vec = width % 8 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 && reinterpret_cast<uintptr_t>(shared_w) % 16 == 0;
 #define ARLE_ROUTE_V(TX, TWT, V)                                                                                   \
   do {                                                                                                             \
     static bool raised = false;                                                                                    \
@@ -607,8 +653,9 @@ extern "C" int arle_moe_route(const void* x, long long x_stride, int x_dtype, co
       raised = true;                                                                                               \
     }                                                                                                              \
     moe_route_kernel<TX, TWT, V><<<tokens, kRouteThreads, lds, s>>>(static_cast<const TX*>(x), x_stride,           \
-                                                                    static_cast<const TWT*>(w), correction, c_dtype, \
-                                                                    ids, weights, width, experts, top, rule);       \
+                                                                    static_cast<const TWT*>(w), bias, b_dtype,      \
+                                                                    correction, c_dtype, static_cast<const TWT*>(shared_w), \
+                                                                    shared_gate, ids, weights, width, experts, top, rule); \
   } while (0)
 #define ARLE_ROUTE(TX, TWT)                          \
   do {                                               \
@@ -639,51 +686,67 @@ extern "C" int arle_moe_identity(const void* x, long long x_stride, int dtype, c
   return launch_status();
 }
 
-// gate_up != 0: x [T, K], w [experts, 2 N, K], out [T * top, N] of `dtype`.  Else: x [T * top, K], w [experts, N, K],
-// out float32 [T * top, N].
+// mode: kGateUp, kUp or kDown (see above); out [T * top, N] of `dtype`, or of float32 for kDown.
 extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w, const int* ids, void* out, int dtype,
-                               int gate_up, int tokens, int experts, int top, int N, int K, void* stream) {
+                               int mode, int tokens, int experts, int top, int N, int K, void* stream) {
   if (tokens == 0) return 0;
-  if (experts < 1 || experts > 65535 || top < 1 || N < 1 || K < 1 || (N + kEN - 1) / kEN > 65535)
+  if (mode < 0 || mode > 2 || experts < 1 || experts > 65535 || top < 1 || N < 1 || K < 1 || (N + kEN - 1) / kEN > 65535)
     return static_cast<int>(hipErrorInvalidValue);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == kBF16 && K % 8 == 0 && x_stride % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(w) % 16 == 0) {
     if (tokens > 64) {      // rows enough that an expert's list fills tiles of 64
-      const int bcols = gate_up ? kBigCols / 2 : kBigCols;
+      const int bcols = mode == kGateUp ? kBigCols / 2 : kBigCols;
       const bf16* xb = static_cast<const bf16*>(x);
       const bf16* wb = static_cast<const bf16*>(w);
 #define ARLE_TILES(GU, RGS)                                                                                      \
   moe_expert_tiles_kernel<GU, RGS, 64><<<dim3((tokens + 256 * RGS - 1) / (256 * RGS), (N + bcols - 1) / bcols, experts), \
                                          256 * RGS, 0, s>>>(xb, x_stride, wb, ids, out, tokens, top, N, K)
+#define ARLE_TILES_MODE(RGS)              \
+  do {                                    \
+    if (mode == kGateUp)                  \
+      ARLE_TILES(kGateUp, RGS);           \
+    else if (mode == kUp)                 \
+      ARLE_TILES(kUp, RGS);               \
+    else                                  \
+      ARLE_TILES(kDown, RGS);             \
+  } while (0)
       // two groups of 64 rows a weight tile once the step has rows for them: a tile's fetch is what the launch waits
       // for (all sixteen launches of a 2,048-token prefill at the Qwen3-4B widths: one group 6,508 us, two 5,219 us,
       // four, which leaves a wave 128 registers, 5,456 us)
       if (tokens > 256) {
-        if (gate_up) ARLE_TILES(true, 2); else ARLE_TILES(false, 2);
+        ARLE_TILES_MODE(2);
       } else {
-        if (gate_up) ARLE_TILES(true, 1); else ARLE_TILES(false, 1);
+        ARLE_TILES_MODE(1);
       }
+#undef ARLE_TILES_MODE
 #undef ARLE_TILES
       return launch_status();
     }
-    const int cols = gate_up ? kMoeCols / 2 : kMoeCols;
+    const int cols = mode == kGateUp ? kMoeCols / 2 : kMoeCols;
     const dim3 mgrid((tokens + kMoeChunk - 1) / kMoeChunk, (N + cols - 1) / cols, experts);
-    if (gate_up)
-      moe_expert_mfma_kernel<true><<<mgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), ids, out, tokens, top, N, K);
-    else
-      moe_expert_mfma_kernel<false><<<mgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), ids, out, tokens, top, N, K);
+#define ARLE_MFMA(MODE)                                                                                           \
+  moe_expert_mfma_kernel<MODE><<<mgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), \
+                                                     ids, out, tokens, top, N, K)
+    if (mode == kGateUp) ARLE_MFMA(kGateUp); else if (mode == kUp) ARLE_MFMA(kUp); else ARLE_MFMA(kDown);
+#undef ARLE_MFMA
     return launch_status();
   }
   const dim3 grid((tokens + kEM - 1) / kEM, (N + kEN - 1) / kEN, experts);
 #define ARLE_EXPERT(TT, GU)                                                                                         \
   moe_expert_kernel<TT, GU><<<grid, kExpertThreads, 0, s>>>(static_cast<const TT*>(x), x_stride,                    \
                                                             static_cast<const TT*>(w), ids, out, tokens, top, N, K)
-  if (dtype == kF32) {
-    if (gate_up) ARLE_EXPERT(float, true); else ARLE_EXPERT(float, false);
-  } else {
-    if (gate_up) ARLE_EXPERT(bf16, true); else ARLE_EXPERT(bf16, false);
-  }
+#define ARLE_EXPERT_MODE(TT)              \
+  do {                                    \
+    if (mode == kGateUp)                  \
+      ARLE_EXPERT(TT, kGateUp);           \
+    else if (mode == kUp)                 \
+      ARLE_EXPERT(TT, kUp);               \
+    else                                  \
+      ARLE_EXPERT(TT, kDown);             \
+  } while (0)
+  if (dtype == kF32) ARLE_EXPERT_MODE(float); else ARLE_EXPERT_MODE(bf16);
+#undef ARLE_EXPERT_MODE
 #undef ARLE_EXPERT
   return launch_status();
 }

@@ -7,24 +7,14 @@
 //
 // m is one number of the model (1 where it has none).
 //
-// An addend is a float32 tensor [T, W], or parts that are added in ascending order: the float32 partial products of
-// a matrix product whose K was split (part p of row t at p * part_stride + t * row_stride), or the outputs of the
-// experts that a token chose, [T, n, W] with a weight per (token, part).  The sums, the statistics, the weight and
-// the residual are 32-bit.  A row's arithmetic depends on nothing but the row.
-#include "common.h"
+// An addend (addend.h) is a float32 tensor, a stack of partial sums, or weighted outputs of experts.  The sums, the
+// statistics, the weight and the residual are 32-bit.  A row's arithmetic depends on nothing but the row.
+#include "addend.h"
 
 namespace arle {
 
 constexpr int kPostThreads = 256;
 constexpr int kPostWaves = kPostThreads / kWave;
-
-struct Addend {
-  const float* p;         // null: no addend
-  int parts;              // parts added in order (>= 1)
-  long long part_stride;  // elements between parts of one row
-  long long row_stride;   // elements between rows
-  const float* weights;   // [T, parts] factors, or null
-};
 
 // Four consecutive entries of an addend's row: its parts added in ascending order (weighted where it has weights).
 // Every load is typed and stands under no condition on data, so the parts' loads are in flight together.
@@ -37,13 +27,13 @@ __device__ __forceinline__ float4 addend_at(const Addend& a, int64_t row, int i)
   };
   float4 sum = get(0);
   if (a.weights) {
-    const float f = a.weights[row * a.parts];
+    const float f = a.weights[row * a.w_row];
     sum.x *= f; sum.y *= f; sum.z *= f; sum.w *= f;
   }
   for (int p = 1; p < a.parts; ++p) {
     const float4 v = get(p);
     if (a.weights) {
-      const float f = a.weights[row * a.parts + p];
+      const float f = a.weights[row * a.w_row + p * a.w_part];
       sum.x = fmaf(f, v.x, sum.x); sum.y = fmaf(f, v.y, sum.y); sum.z = fmaf(f, v.z, sum.z); sum.w = fmaf(f, v.w, sum.w);
     } else {
       sum.x += v.x; sum.y += v.y; sum.z += v.z; sum.w += v.w;
@@ -132,14 +122,15 @@ using namespace arle;
 // residual float32 [rows, width], updated in place.  Addends are float32.  act: [rows, width] of act_dtype, or null.
 // center != 0: the layer norm; bias: [width] of the weight's type, or null; mult: the factor on what is added.
 extern "C" int arle_norm_add(float* residual, const float* a, int a_parts, long long a_part_stride,
-                             long long a_row_stride, const float* a_weights, const float* b, int b_parts,
-                             long long b_part_stride, long long b_row_stride, const float* b_weights,
+                             long long a_row_stride, const float* a_weights, int a_w_row, int a_w_part, const float* b,
+                             int b_parts, long long b_part_stride, long long b_row_stride, const float* b_weights,
+                             int b_w_row, int b_w_part,
                              const void* w, int w_dtype, int one_plus, int center, const void* bias, float mult,
                              void* act, int act_dtype, int rows, int width, float eps, void* stream) {
   if (rows == 0) return 0;
   if (!a || a_parts < 1 || (b && b_parts < 1) || width < 1 || width > 16384) return static_cast<int>(hipErrorInvalidValue);
-  const Addend A{a, a_parts, a_part_stride, a_row_stride, a_weights};
-  const Addend B{b, b_parts, b_part_stride, b_row_stride, b_weights};
+  const Addend A{a, a_parts, a_part_stride, a_row_stride, a_weights, a_w_row, a_w_part};
+  const Addend B{b, b_parts, b_part_stride, b_row_stride, b_weights, b_w_row, b_w_part};
   hipStream_t s = static_cast<hipStream_t>(stream);
   const size_t lds = static_cast<size_t>(width) * sizeof(float);
   auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };

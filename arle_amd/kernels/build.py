@@ -45,10 +45,12 @@ SOURCES = {
     "hyper": "hyper.hip",
     "rotary_store": "rotary_store.hip",
     "gated_delta": "gated_delta.hip",
+    "group_norm": "group_norm.hip",
+    "retention": "retention.hip",
     "host": "host/runtime.cpp",
 }
 HEADERS = ("common.h", "attention_static.h", "attention_args.h", "attention_stream.h", "attention_portions.h",
-           "attention_portions_dma.h")
+           "attention_portions_dma.h", "addend.h")
 HOST_LIBS = ("host",)   # plain C++: page pool, block tables, step packing
 HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-shared"]
 

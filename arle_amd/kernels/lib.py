@@ -23,7 +23,7 @@ SIGNATURES = {
     "arle_silu_mul": ("elementwise", [_p, _p, _ll, _p, _i, _i, _i, _i, _p]),
     "arle_rmsnorm": ("norm", [_p, _i, _ll, _p, _i, _p, _i, _p, _i, _i, _f, _p]),
     "arle_add_rmsnorm": ("norm", [_p, _p, _i, _ll, _i, _p, _i, _p, _i, _p, _i, _i, _f, _p]),
-    "arle_sum_partials": ("elementwise", [_p, _i, _ll, _p, _i, _ll, _p]),
+    "arle_sum_partials": ("elementwise", [_p, _i, _ll, _p, _i, _ll, _i, _p]),
     "arle_gemm_rows_rounds": ("gemm_rows", [_p, _ll, _p, _ll, _i, _p, _ll, _i, _i, _i, _i, _i, _p]),
     "arle_gemm_rows": ("gemm_rows", [_p, _ll, _p, _ll, _i, _p, _ll, _ll, _i, _i, _i, _i, _i, _i, _i, _i, _p]),
     "arle_gemm_rows_geometry": ("gemm_rows", [_i]),
@@ -75,13 +75,20 @@ SIGNATURES = {
     "arle_wide_norm_store": ("attention_softcap", [_p, _ll, _p, _ll, _p, _ll, _p, _ll, _i, _p, _p, _i, _p, _i, _f, _p, _p,
                                                    _p, _i, _p, _p, _i, _i, _i, _i, _i, _i, _p, _p, _i, _i, _p]),
     "arle_tanh_cap": ("elementwise", [_p, _ll, _f, _p]),
-    "arle_norm_add": ("post_norm", [_p, _p, _i, _ll, _ll, _p, _p, _i, _ll, _ll, _p, _p, _i, _i, _i, _p, _f, _p, _i, _i, _i, _f,
-                                    _p]),
+    "arle_norm_add": ("post_norm", [_p, _p, _i, _ll, _ll, _p, _i, _i, _p, _i, _ll, _ll, _p, _i, _i, _p, _i, _i, _i, _p, _f, _p,
+                                    _i, _i, _i, _f, _p]),
+    "arle_group_norm": ("group_norm", [_p, _i, _ll, _p, *3 * [_p, _i, _ll, _ll, _p, _i, _i], _p, _i, _p, _i, _p, _i, _i, _i, _f,
+                                       _p]),
+    "arle_retention_prep": ("retention", [_p, _ll, _p, _ll, _p, _p, _i, _p, _i, _i, _i, _p]),
+    "arle_retention_scan": ("retention", [_p, _ll, _p, _ll, _p, _ll, _p, _p, _p, _p, _i, _p, _i, _i, _i, _p]),
+    "arle_retention_output": ("retention", [_p, _p, _ll, _f, _p, _i, _i, _i, _i, _p]),
+    "arle_retention_decode": ("retention", [_p, _i, _ll, _ll, _p, _p, _p, _i, _p, _p, _p, _p, _f, _p, _i, _i, _i, _i, _i, _p]),
+    "arle_retention_chunks": ("retention", [_p, _ll, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _p, _f, _p, _i, _i, _i, _i, _p]),
     "arle_latent_prep": ("latent", [_p, _ll, _p, _ll, _p, _ll, _i, _p, _i, _f, _p, _p, _i, _p, _p, _p, _i, _p, _p, _i, _i,
                                     _i, _i, _i, _i, _i, _p]),
     "arle_head_proj": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _i, _p]),
     "arle_head_proj_mfma": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _p]),
-    "arle_moe_route": ("moe", [_p, _ll, _i, _p, _i, _p, _i, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p]),
+    "arle_moe_route": ("moe", [_p, _ll, _i, _p, _i, _p, _i, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p]),
     "arle_moe_identity": ("moe", [_p, _ll, _i, _p, _p, _i, _i, _i, _i, _p]),
     "arle_moe_expert": ("moe", [_p, _ll, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
     "arle_gate_mul": ("elementwise", [_p, _ll, _p, _ll, _p, _i, _i, _i, _i, _p]),

@@ -991,15 +991,19 @@ def gemm_tiles(x, tiles, n: int, out_dtype=torch.bfloat16, epilogue: int = EPI_N
     return out
 
 
-def sum_partials(parts: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
-    """[S, ...] float32 -> [...]: the stack added in order."""
+SUM_ACTS = {None: 0, "squared_relu": 1}      # what a sum of partial products passes through: nothing, or max(z, 0)^2
+
+
+def sum_partials(parts: torch.Tensor, out_dtype: torch.dtype, act: str | None = None) -> torch.Tensor:
+    """[S, ...] float32 -> [...]: the stack added in order, then `act` (one of SUM_ACTS)."""
     _gpu(parts)
     _need(parts.dtype == torch.float32 and parts.dim() >= 2 and parts.is_contiguous() and parts.shape[0] >= 1,
           "sum_partials takes a contiguous float32 stack")
     _need(out_dtype in _CODES, "sum_partials writes bfloat16 or float32")
+    _need(act in SUM_ACTS, "unknown activation")
     out = torch.empty(parts.shape[1:], dtype=out_dtype, device=parts.device)
     lib.call("arle_sum_partials", parts.data_ptr(), parts.shape[0], out.numel(), out.data_ptr(), _CODES[out_dtype],
-             out.numel(), _stream())
+             out.numel(), SUM_ACTS[act], _stream())
     return out
 
 
@@ -1798,22 +1802,40 @@ def wide_norm_store(q, k, v, *, num_q_heads: int, num_kv_heads: int, key_dim: in
 NORM_ADD_MAX_WIDTH = 16384
 
 
+class Scaled:
+    """An addend with one factor a row: `delta` (float32 [T, W] or a stack [S, T, W] of partial sums) times `factor`
+    (float32 [T])."""
+
+    def __init__(self, delta: torch.Tensor, factor: torch.Tensor):
+        self.delta, self.factor = delta, factor
+
+
+def _addend_tensors(term) -> tuple:
+    if isinstance(term, Scaled):
+        return (term.delta, term.factor)
+    return term if isinstance(term, tuple) else (term,)
+
+
 def _addend_args(term, rows: int, width: int):
-    """(pointer, parts, part stride, row stride, weights pointer) of one float32 addend of `norm_add`: a tensor [T, W];
-    a stack [S, T, W] of partial sums; or (outputs [T, n, W], weights [T, n])."""
+    """(pointer, parts, part stride, row stride, factors' pointer, their stride a row and a part) of one float32 addend:
+    a tensor [T, W]; a stack [S, T, W] of partial sums; (outputs [T, n, W], weights [T, n]); or a `Scaled` one."""
     if term is None:
-        return (0, 0, 0, 0, 0)
+        return (0, 0, 0, 0, 0, 0, 0)
+    if isinstance(term, Scaled):
+        _need(term.factor.shape == (rows,) and term.factor.dtype == torch.float32 and term.factor.is_contiguous(),
+              "an addend's factor must be contiguous float32 [T]")
+        return _addend_args(term.delta, rows, width)[:4] + (term.factor.data_ptr(), 1, 0)
     if isinstance(term, tuple):
         outs, weights = term
         _need(outs.dim() == 3 and outs.shape[0] == rows and outs.shape[2] == width and outs.is_contiguous()
               and outs.dtype == torch.float32, "weighted outputs must be contiguous float32 [T, n, W]")
         _need(weights.shape == outs.shape[:2] and weights.dtype == torch.float32 and weights.is_contiguous(),
               "their weights must be contiguous float32 [T, n]")
-        return (outs.data_ptr(), outs.shape[1], width, outs.shape[1] * width, weights.data_ptr())
+        return (outs.data_ptr(), outs.shape[1], width, outs.shape[1] * width, weights.data_ptr(), outs.shape[1], 1)
     _need(term.dim() in (2, 3) and tuple(term.shape[-2:]) == (rows, width) and term.is_contiguous()
           and term.dtype == torch.float32 and term.shape[0] >= 1,
           "an addend must match the residual (float32 [T, W] or a stack [S, T, W])")
-    return (term.data_ptr(), term.shape[0] if term.dim() == 3 else 1, rows * width, width, 0)
+    return (term.data_ptr(), term.shape[0] if term.dim() == 3 else 1, rows * width, width, 0, 0, 0)
 
 
 def norm_add(residual: torch.Tensor, terms, weight: torch.Tensor, eps: float, *, one_plus: bool = False,
@@ -1826,7 +1848,7 @@ def norm_add(residual: torch.Tensor, terms, weight: torch.Tensor, eps: float, *,
     _need(1 <= len(terms) <= 2, "norm_add takes one or two addends")
     # what a sublayer leaves for the residual is 32-bit sums; an output that was rounded on its way is widened first
     terms = [t.float() if torch.is_tensor(t) and t.dtype == torch.bfloat16 else t for t in terms]
-    _gpu(residual, weight, *[x for t in terms for x in (t if isinstance(t, tuple) else (t,))])
+    _gpu(residual, weight, *[x for t in terms for x in _addend_tensors(t)])
     _need(residual.dtype == torch.float32 and residual.dim() == 2 and residual.is_contiguous(),
           "residual must be contiguous float32 [T, W]")
     rows, width = residual.shape
@@ -1841,6 +1863,40 @@ def norm_add(residual: torch.Tensor, terms, weight: torch.Tensor, eps: float, *,
     lib.call("arle_norm_add", residual.data_ptr(), *args, weight.data_ptr(), _code(weight), 1 if one_plus else 0,
              1 if center else 0, _ptr(bias), float(mult), _ptr(act), _code(act) if act is not None else 0, rows, width, float(eps), _stream())
     return act
+
+
+GROUP_NORM_MAX_WIDTH = 16384
+GROUP_NORM_MAX_TERMS = 3
+
+
+def group_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out_dtype: torch.dtype, *, terms=(),
+               rows: torch.Tensor | None = None):
+    """x [., W] + the sum of up to three `terms` (see `_addend_args`; x is then the float32 residual and takes the sum in
+    place, unless `rows` is given), each of `groups` equal groups of consecutive entries divided by its own
+    sqrt(mean(x^2) + eps), times weight [W].  rows: which rows of x (and of the terms) are normed, e.g. the rows of a
+    table."""
+    terms = list(terms)
+    _need(len(terms) <= GROUP_NORM_MAX_TERMS, f"group_norm adds at most {GROUP_NORM_MAX_TERMS} terms")
+    terms = [t.float() if torch.is_tensor(t) and t.dtype == torch.bfloat16 else t for t in terms]
+    _gpu(x, weight, rows, *[y for t in terms for y in _addend_tensors(t)])
+    _rows(x, "x")
+    width = x.shape[1]
+    _need(x.dtype in _CODES and 0 < width <= GROUP_NORM_MAX_WIDTH, f"group_norm takes widths up to {GROUP_NORM_MAX_WIDTH}")
+    _need(groups >= 1 and width % groups == 0, "the groups must divide the width evenly")
+    _need(weight.shape == (width,) and weight.is_contiguous() and weight.dtype in _CODES, "norm weight must be [width]")
+    _need(not terms or (x.dtype == torch.float32 and x.is_contiguous()), "terms are added to a contiguous float32 residual")
+    n_rows = x.shape[0]
+    if rows is not None:
+        _i32(rows, "rows")
+        n_rows = rows.numel()
+    out = torch.empty((n_rows, width), dtype=out_dtype, device=x.device)
+    args = []
+    for i in range(GROUP_NORM_MAX_TERMS):
+        args += _addend_args(terms[i] if i < len(terms) else None, x.shape[0], width)
+    lib.call("arle_group_norm", x.data_ptr(), _code(x), x.stride(0), x.data_ptr() if terms and rows is None else 0, *args,
+             weight.data_ptr(), _code(weight), out.data_ptr(), _code(out), _ptr(rows), n_rows, width, int(groups), float(eps),
+             _stream())
+    return out
 
 
 def tanh_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
@@ -1930,17 +1986,21 @@ def head_proj_mfma(x, wnk, out, *, heads: int, in_head: int, out_head: int):
 
 MOE_MAX_EXPERTS = 1024
 MOE_MAX_TOP = 64
+MOE_SCORES = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
+MOE_DOWN, MOE_GATE_UP, MOE_UP = 0, 1, 2      # which of an expert's products `moe_expert` makes
 
 
 def moe_route(x, router, correction, *, top: int, scale: float, score: str = "sigmoid", groups: int = 1,
-              keep_groups: int = 1, normalize: bool = True):
+              keep_groups: int = 1, normalize: bool = True, bias=None, shared_gate=None):
     """(ids int32 [T, top], weights float32 [T, top]) of a router: z = router x in 32-bit sums, s = sigmoid(z) or
     (score "softmax") softmax(z) over all rows of the router, the `top` largest s + correction chosen (ties: the lower
     index) among the experts of the `keep_groups` best of `groups` equal groups of neighbours (a group's number: the
     largest s + correction in it), weights s / (sum + 1e-20) * scale, or s * scale without `normalize`, in the order
-    they were chosen."""
-    _need(score in ("sigmoid", "softmax"), "a router's scores are sigmoid or softmax")
-    _gpu(x, router, correction)
+    they were chosen.  score "softmax_chosen": s = z, and the weights are the softmax over the chosen z, times scale.
+    bias [experts]: added to z.  shared_gate: a weight [1, width] of the router's type; the answer is then (ids, weights,
+    sigmoid(shared_gate x) float32 [T])."""
+    _need(score in MOE_SCORES, f"a router's scores are one of {', '.join(MOE_SCORES)}")
+    _gpu(x, router, correction, bias, shared_gate)
     _rows(x, "x")
     experts, width = router.shape
     _need(router.dim() == 2 and router.is_contiguous() and router.dtype in _CODES and x.shape[1] == width and x.dtype in _CODES,
@@ -1952,13 +2012,20 @@ def moe_route(x, router, correction, *, top: int, scale: float, score: str = "si
     if correction is not None:
         _need(correction.shape == (experts,) and correction.is_contiguous() and correction.dtype in _CODES,
               "correction must be [experts]")
+    if bias is not None:
+        _need(bias.shape == (experts,) and bias.is_contiguous() and bias.dtype in _CODES, "bias must be [experts]")
+    gate = None
+    if shared_gate is not None:
+        _need(shared_gate.shape == (1, width) and shared_gate.is_contiguous() and shared_gate.dtype == router.dtype,
+              "the shared expert's gate must be [1, width] of the router's type")
+        gate = torch.empty((x.shape[0],), dtype=torch.float32, device=x.device)
     ids = torch.empty((x.shape[0], top), dtype=torch.int32, device=x.device)
     weights = torch.empty((x.shape[0], top), dtype=torch.float32, device=x.device)
-    lib.call("arle_moe_route", x.data_ptr(), x.stride(0), _code(x), router.data_ptr(), _code(router), _ptr(correction),
-             _code(correction) if correction is not None else 0, ids.data_ptr(), weights.data_ptr(), x.shape[0], width,
-             experts, int(top), float(scale), 1 if score == "softmax" else 0, int(groups), int(keep_groups),
-             1 if normalize else 0, _stream())
-    return ids, weights
+    lib.call("arle_moe_route", x.data_ptr(), x.stride(0), _code(x), router.data_ptr(), _code(router), _ptr(bias),
+             _code(bias) if bias is not None else 0, _ptr(correction), _code(correction) if correction is not None else 0,
+             _ptr(shared_gate), _ptr(gate), ids.data_ptr(), weights.data_ptr(), x.shape[0], width, experts, int(top),
+             float(scale), MOE_SCORES[score], int(groups), int(keep_groups), 1 if normalize else 0, _stream())
+    return (ids, weights) if gate is None else (ids, weights, gate)
 
 
 def moe_identity(x, ids, outs, first: int):
@@ -1976,22 +2043,24 @@ def moe_identity(x, ids, outs, first: int):
     return outs
 
 
-def moe_expert(x, w, ids, *, gate_up: bool):
-    """The chosen experts' products.  gate_up: x [T, K], w [experts, 2N, K] (gate rows, then up rows) ->
-    silu(gate) * up as [T * top, N] of x's type, row t * top + k for token t's k-th choice.  Else: x [T * top, K],
-    w [experts, N, K] -> float32 [T * top, N]."""
+def moe_expert(x, w, ids, which: int):
+    """The chosen experts' products.  MOE_GATE_UP: x [T, K], w [experts, 2N, K] (gate rows, then up rows) ->
+    silu(gate) * up as [T * top, N] of x's type, row t * top + k for token t's k-th choice.  MOE_UP: the same for
+    w [experts, N, K] without a gate -> max(up, 0)^2.  MOE_DOWN: x [T * top, K], w [experts, N, K] -> float32
+    [T * top, N]."""
+    _need(which in (MOE_DOWN, MOE_GATE_UP, MOE_UP), "unknown expert product")
     _gpu(x, w, ids)
     _rows(x, "x")
     _need(ids.dtype == torch.int32 and ids.dim() == 2 and ids.is_contiguous(), "ids must be contiguous int32 [T, top]")
     tokens, top = ids.shape
     _need(w.dim() == 3 and w.is_contiguous() and w.dtype == x.dtype and x.dtype in _CODES and w.shape[2] == x.shape[1],
           "w must be contiguous [experts, N, K] of x's type")
-    _need(x.shape[0] == (tokens if gate_up else tokens * top), "x has a row a token (gate|up) or a row a choice (down)")
-    _need(not gate_up or w.shape[1] % 2 == 0, "gate|up has an even number of rows")
-    N = w.shape[1] // 2 if gate_up else w.shape[1]
-    out = torch.empty((tokens * top, N), dtype=x.dtype if gate_up else torch.float32, device=x.device)
+    _need(x.shape[0] == (tokens * top if which == MOE_DOWN else tokens), "x has a row a token (up) or a row a choice (down)")
+    _need(which != MOE_GATE_UP or w.shape[1] % 2 == 0, "gate|up has an even number of rows")
+    N = w.shape[1] // 2 if which == MOE_GATE_UP else w.shape[1]
+    out = torch.empty((tokens * top, N), dtype=torch.float32 if which == MOE_DOWN else x.dtype, device=x.device)
     lib.call("arle_moe_expert", x.data_ptr(), x.stride(0), w.data_ptr(), ids.data_ptr(), out.data_ptr(), _code(x),
-             1 if gate_up else 0, tokens, w.shape[0], top, N, x.shape[1], _stream())
+             int(which), tokens, w.shape[0], top, N, x.shape[1], _stream())
     return out
 
 
@@ -2246,4 +2315,99 @@ def gated_delta_output(o, gate, weight, eps: float, *, heads: int, value_dim: in
     out = torch.empty((tokens, width), dtype=gate.dtype, device=o.device)
     lib.call("arle_gated_delta_output", o.data_ptr(), gate.data_ptr(), gate.stride(0), _code(gate), weight.data_ptr(),
              _code(weight), float(eps), out.data_ptr(), tokens, heads, value_dim, int(act), _stream())
+    return out
+
+
+# ------------------------------------------------------------- retention
+
+RETENTION_MAX_KEY_DIM = 256
+RETENTION_CHUNK = 64
+_RETENTION_DECODE_MAX_DV = 1024
+_RETENTION_CHUNK_MAX_DV = 256
+_RETENTION_WORK_BYTES = 4 << 30     # most memory for the states in front of the chunks
+
+
+def _retention_check(y, s_state, seg_row0, seg_slot, positions, cos, sin, rotary_dims, heads, key_dim, value_dim):
+    H, D, Dv = heads, key_dim, value_dim
+    _gpu(y, s_state, seg_row0, seg_slot, positions, cos, sin)
+    _need(y.dim() in (2, 3) and y.shape[-1] == 2 * H * (D + Dv) and y.dtype == torch.float32 and y.is_contiguous(),
+          "y must be contiguous float32 [T, q | k | v | gate] (or a stack of partial sums of it)")
+    _need(0 < D <= RETENTION_MAX_KEY_DIM and 0 < Dv and 0 < H <= _GRID_Y_MAX, f"key sizes up to {RETENTION_MAX_KEY_DIM}")
+    _need(s_state.dim() == 4 and tuple(s_state.shape[1:]) == (H, D, Dv) and s_state.dtype == torch.float32
+          and s_state.is_contiguous(), "the state is float32 [slots, heads, D, Dv]")
+    _need(0 <= rotary_dims <= D and rotary_dims % 2 == 0, "rotary dims must be even and at most the key's size")
+    if rotary_dims:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _need(t is not None and t.dtype == torch.float32 and t.dim() == 2 and t.shape[1] == rotary_dims // 2
+                  and t.is_contiguous(), f"{name} must be contiguous float32 [positions, rotary_dims / 2]")
+    _i32(positions, "positions", y.shape[-2])
+    _i32(seg_slot, "seg_slot")
+    _i32(seg_row0, "seg_row0", seg_slot.numel() + 1)
+
+
+def retention_decode_supported(value_dim: int) -> bool:
+    """Whether `retention_decode` takes heads of this value size."""
+    return value_dim % 4 == 0 and value_dim <= _RETENTION_DECODE_MAX_DV
+
+
+def retention_chunks_supported(tokens: int, segments: int, heads: int, key_dim: int, value_dim: int, rotary_dims: int) -> bool:
+    """Whether the form over chunks on the matrix cores takes these sizes."""
+    work = (tokens // RETENTION_CHUNK + segments) * heads * key_dim * value_dim * 4
+    return (key_dim % 4 == 0 and value_dim % 4 == 0 and value_dim <= _RETENTION_CHUNK_MAX_DV and rotary_dims % 8 == 0
+            and work <= _RETENTION_WORK_BYTES)
+
+
+def retention_rows(y, decay, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, positions, cos, sin, rotary_dims: int,
+                   heads: int, key_dim: int, value_dim: int):
+    """Retention over the rows of every segment, row by row (see csrc/retention.hip): y float32 [T, q | k | v | gate]
+    (q and k are turned in place), decay float32 [heads].  Returns [T, heads * Dv] of `out_dtype`, gated and normed."""
+    _retention_check(y, s_state, seg_row0, seg_slot, positions, cos, sin, rotary_dims, heads, key_dim, value_dim)
+    _need(y.dim() == 2, "the rows' form takes whole sums")
+    _need(decay.shape == (heads,) and decay.dtype == torch.float32 and decay.is_contiguous() and decay.is_cuda, "decay must be float32 [heads]")
+    T, H, D, Dv = y.shape[0], heads, key_dim, value_dim
+    q, k, v, g = y[:, :H * D], y[:, H * D:2 * H * D], y[:, 2 * H * D:2 * H * D + H * Dv], y[:, 2 * H * D + H * Dv:]
+    lib.call("arle_retention_prep", q.data_ptr(), y.stride(0), k.data_ptr(), y.stride(0), _ptr(cos) if rotary_dims else 0,
+             _ptr(sin) if rotary_dims else 0, int(rotary_dims), positions.data_ptr(), T, H, D, _stream())
+    o = torch.empty((T, H * Dv), dtype=torch.float32, device=y.device)
+    lib.call("arle_retention_scan", q.data_ptr(), y.stride(0), k.data_ptr(), y.stride(0), v.data_ptr(), y.stride(0),
+             decay.data_ptr(), s_state.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(), seg_slot.numel(), o.data_ptr(),
+             H, D, Dv, _stream())
+    out = torch.empty((T, H * Dv), dtype=out_dtype, device=y.device)
+    lib.call("arle_retention_output", o.data_ptr(), g.data_ptr(), y.stride(0), float(eps), out.data_ptr(), _code(out), T, H,
+             Dv, _stream())
+    return out
+
+
+def retention_decode(y, decay, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, positions, cos, sin, rotary_dims: int,
+                     heads: int, key_dim: int, value_dim: int):
+    """`retention_rows` for steps of one row a segment, in one kernel; y may be the stack of the product's partial sums."""
+    _retention_check(y, s_state, seg_row0, seg_slot, positions, cos, sin, rotary_dims, heads, key_dim, value_dim)
+    _need(y.shape[-2] == seg_slot.numel(), "one row a segment")
+    _need(retention_decode_supported(value_dim), f"value sizes that are multiples of 4 up to {_RETENTION_DECODE_MAX_DV}")
+    _need(decay.shape == (heads,) and decay.dtype == torch.float32 and decay.is_contiguous() and decay.is_cuda, "decay must be float32 [heads]")
+    T, width = y.shape[-2], y.shape[-1]
+    out = torch.empty((T, heads * value_dim), dtype=out_dtype, device=y.device)
+    lib.call("arle_retention_decode", y.data_ptr(), y.shape[0] if y.dim() == 3 else 1, T * width, width, decay.data_ptr(),
+             _ptr(cos) if rotary_dims else 0, _ptr(sin) if rotary_dims else 0, int(rotary_dims), positions.data_ptr(),
+             seg_row0.data_ptr(), seg_slot.data_ptr(), s_state.data_ptr(), float(eps), out.data_ptr(), _code(out),
+             seg_slot.numel(), heads, key_dim, value_dim, _stream())
+    return out
+
+
+def retention_chunks(y, powers, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, positions, cos, sin, rotary_dims: int,
+                     heads: int, key_dim: int, value_dim: int):
+    """`retention_rows` over chunks of 64 rows on the matrix cores (float32 products); powers float32 [heads, 65]: the
+    decays to the powers 0 .. 64."""
+    _retention_check(y, s_state, seg_row0, seg_slot, positions, cos, sin, rotary_dims, heads, key_dim, value_dim)
+    T, segments, H, D, Dv = y.shape[0], seg_slot.numel(), heads, key_dim, value_dim
+    _need(y.dim() == 2 and retention_chunks_supported(T, segments, H, D, Dv, rotary_dims), "sizes outside the chunks' form")
+    _need(powers.shape == (H, RETENTION_CHUNK + 1) and powers.dtype == torch.float32 and powers.is_contiguous() and powers.is_cuda,
+          "powers must be float32 [heads, 65]")
+    items = T // RETENTION_CHUNK + segments      # no fewer than the chunks of all segments together
+    work = torch.empty((items, H, Dv, D), dtype=torch.float32, device=y.device)
+    out = torch.empty((T, H * Dv), dtype=out_dtype, device=y.device)
+    lib.call("arle_retention_chunks", y.data_ptr(), y.stride(0), _ptr(cos) if rotary_dims else 0,
+             _ptr(sin) if rotary_dims else 0, int(rotary_dims), positions.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(),
+             powers.data_ptr(), s_state.data_ptr(), segments, items, work.data_ptr(), float(eps), out.data_ptr(), _code(out),
+             H, D, Dv, _stream())
     return out

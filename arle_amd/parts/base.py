@@ -16,10 +16,12 @@ Interfaces (T = tokens of the packed step, H = hidden size, A = activation dtype
                 be sized from its description alone, the class method `declare_cache(params)` with the same answer;
                 `reader_cache_need()` / `declare_reader_cache(params)`: what it keeps in an entry that reads another
                 entry's cache); `forward(x A[T,H], batch: StepBatch, cache_view) -> delta`.
-* feed_forward  `forward(x A[T,H]) -> delta`.
+* feed_forward  `forward(x A[T,H]) -> delta`, or a list of addends (tensor or stack, (outputs f32[T,n,H], weights
+                f32[T,n]), `ops.Scaled`) for a block whose norm adds them.
 * block         `forward(residual f32[T,H], delta | None, batch, cache_view) -> (residual, delta)`;
                 the returned delta is what the next block (or the final norm) still has to add: a tensor, a stack,
-                or a `Pending` list of (tensor or stack, bias or None) for norms that add several terms in one pass.
+                or a `Pending` list of (tensor, stack or another addend of `ops.group_norm`, bias or None) for norms
+                that add several terms in one pass.
 * embedding     `forward(token_ids i32[T]) -> f32[T,H]`.
 * head          `forward(x A[R,H]) -> f32[R,V]`.
 """
@@ -76,7 +78,7 @@ class Runtime:
 
 
 class Pending(list):
-    """What a block leaves for the next norm to add into the residual: [(tensor or float32 stack, bias or None), ...]."""
+    """What a block leaves for the next norm to add into the residual: [(addend, bias or None), ...]."""
 
 
 class Part:

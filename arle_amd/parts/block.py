@@ -86,9 +86,10 @@ class PostNormBlock:
 @register("block", "parallel")
 class ParallelBlock:
     """h += mixer(norm_a(h)) + ffn(norm_b(h)): both read the same residual.  norm roles: "mixer_in", "ffn_in" (the
-    second only with a feed-forward).  The two outputs go on, unadded, to the next block's norms (or the final one),
-    which add them in the pass that computes their statistics; the two norms of this block come out of one pass too.
-    A mixer or feed-forward may hand back (delta, bias): the bias of its last projection, added with the delta."""
+    second only with a feed-forward; without it the feed-forward reads the mixer's norm too).  The two outputs go on,
+    unadded, to the next block's norms (or the final one), which add them in the pass that computes their statistics; the
+    two norms of this block come out of one pass too.  A mixer or feed-forward may hand back (delta, bias), the bias of
+    its last projection, added with the delta, or a list of addends (a mixture of experts)."""
 
     norm_roles = ("mixer_in", "ffn_in")
 
@@ -105,10 +106,12 @@ class ParallelBlock:
         if self.norm_ffn is not None:
             a, b = self.norm_mixer.add_norm(residual, delta, also=self.norm_ffn)
         else:
-            a = self.norm_mixer.add_norm(residual, delta)
+            a = b = self.norm_mixer.add_norm(residual, delta)
         left = Pending()
         for out in (self.mixer.forward(a, batch, cache_view),
-                    self.feed_forward.forward(b) if self.norm_ffn is not None else None):
-            if out is not None:
+                    self.feed_forward.forward(b) if self.feed_forward is not None else None):
+            if isinstance(out, list):
+                left.extend((term, None) for term in out)
+            elif out is not None:
                 left.append(out if isinstance(out, tuple) else (out, None))
         return residual, left

@@ -14,7 +14,8 @@ from .linear import Linear
 
 @register("embedding", "token_table")
 class TokenEmbedding(Part):
-    """params: vocab_size, hidden_size, scale (a factor on every row, in 32 bits; default 1)."""
+    """params: vocab_size, hidden_size, scale (a factor on every row, in 32 bits; default 1), norm (PartSpec of a norm
+    that the rows pass on their way into the residual, in 32 bits; default none)."""
 
     graph_safe = True  # launches depend on shapes only, never on the values of a step
 
@@ -22,12 +23,21 @@ class TokenEmbedding(Part):
     def declare_weights(cls, params):
         return {"table": WeightDecl((params["vocab_size"], params["hidden_size"]))}
 
+    @classmethod
+    def children(cls, params):
+        return {"norm": ("norm", params["norm"])} if params.get("norm") is not None else {}
+
     def __init__(self, params, tensors, rt, children=None):
         super().__init__(params, tensors, rt, children)
         self.table = tensors["table"]
         self.scale = float(params.get("scale", 1.0))
+        self.norm = (children or {}).get("norm")
+        if self.norm is not None and self.scale != 1.0:
+            raise ValueError("a normed embedding has no scale of its own")
 
     def forward(self, token_ids):
+        if self.norm is not None:       # the rows are picked and normed in one pass
+            return self.norm.forward(self.table, rows=token_ids, out_dtype=torch.float32)
         return ops.embed_gather(self.table, token_ids, scale=self.scale)
 
 

@@ -1,4 +1,5 @@
-"""Dense feed-forwards.  SwiGLU: down(silu(gate(x)) * up(x)), no biases; PolyNorm (below): one projection up
+"""Dense feed-forwards.  SwiGLU: down(silu(gate(x)) * up(x)), no biases; the squared relu (below):
+down(max(up(x), 0)^2), no biases; PolyNorm (below): one projection up
 with a bias, a polynomial of row-normalised powers, one projection down with a bias.
 
 infer/src/model/qwen3/prefill.rs:291-337.  gate and up are kept as one [2I, H] matrix
@@ -64,6 +65,36 @@ class SwiGLU(Part):
             gu = self.gate_up(x)
             act = ops.act_mul(gu[:, : self.inter], gu[:, self.inter:], self.act)
         return self.down(act, out_dtype=torch.float32 if self.float32_out else None, partials_ok=True)
+
+
+@register("feed_forward", "squared_relu")
+class SquaredReLU(Part):
+    """down(max(up x, 0)^2), no biases.  params: hidden_size, intermediate_size.  The activation rides on the pass that
+    adds the first product's partial sums; the down projection hands on its 32-bit sums."""
+
+    graph_safe = True  # launches depend on shapes only, never on the values of a step
+
+    @classmethod
+    def declare_weights(cls, params):
+        h, i = params["hidden_size"], params["intermediate_size"]
+        return {"up": WeightDecl((i, h)), "down": WeightDecl((h, i))}
+
+    def __init__(self, params, tensors, rt, children=None):
+        super().__init__(params, tensors, rt, children)
+        self.up = Linear(tensors["up"], rt.weight_tiles)
+        self.down = Linear(tensors["down"], rt.weight_tiles)
+
+    def products(self):
+        if self.up.weight.dtype != torch.bfloat16:
+            return []
+        return [("up", self.up.out_features, self.up.in_features, False, "norm"),
+                ("down", self.down.out_features, self.down.in_features, False, "norm")]
+
+    def forward(self, x):
+        """x [T, H] -> float32 [T, H], or a float32 stack [S, T, H] to be added in order (see Linear)."""
+        u = self.up(x, out_dtype=torch.float32, partials_ok=True)
+        act = ops.sum_partials(u if u.dim() == 3 else u.unsqueeze(0), self.rt.act_dtype, act="squared_relu")
+        return self.down(act, out_dtype=torch.float32, partials_ok=True)
 
 
 @register("feed_forward", "polynorm")

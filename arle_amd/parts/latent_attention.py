@@ -3,7 +3,8 @@
 Per token, with h the mixer's input, H heads, per head D unrotated and R rotated query/key entries, value size Dv,
 latent size C:
 
-    q = W_q h, head by head [D unrotated | R rotated];     W_dkv h = [C entries | R entries]
+    q = W_q h, or through a latent of their own W_uq (rms_norm(W_dq h) * w_q), head by head [D unrotated | R rotated]
+    W_dkv h = [C entries | R entries]
     c = rms_norm(first C entries) * w_c;                    k_rot = rotate(last R entries)        (one for all heads)
     k_h = W_uk,h c,  v_h = W_uv,h c
     s_ij,h = scale (q_h,i . k_h,j + rotate(q_rot,h,i) . k_rot,j)    for 0 <= i - j < window  (None: every j <= i)
@@ -30,7 +31,7 @@ from .softcap_attention import softcap_attention
 
 @register("mixer", "latent_attention")
 class LatentAttention(Part):
-    """params: hidden_size, heads, dim, rot_dim, value_dim, rank, eps, scale, window (int | None), sink (bool),
+    """params: hidden_size, heads, dim, rot_dim, value_dim, rank, q_rank (int | None: the size of the queries' own latent), eps, scale, window (int | None), sink (bool),
     gate (bool: a sigmoid gate on the heads' outputs, a projection of the mixer's input), position (PartSpec of the
     rotation over the rot_dim part)."""
 
@@ -40,8 +41,13 @@ class LatentAttention(Part):
     def declare_weights(cls, params):
         h, H = params["hidden_size"], params["heads"]
         D, R, Dv, C = params["dim"], params["rot_dim"], params["value_dim"], params["rank"]
-        decl = {"q": WeightDecl((H * (D + R), h)), "dkv": WeightDecl((C + R, h)), "c_norm": WeightDecl((C,), init="ones"),
-                "uk": WeightDecl((H * D, C)), "uv": WeightDecl((H * Dv, C)), "o": WeightDecl((h, H * Dv))}
+        Cq = params.get("q_rank")
+        if Cq:
+            decl = {"dq": WeightDecl((Cq, h)), "q_norm": WeightDecl((Cq,), init="ones"), "uq": WeightDecl((H * (D + R), Cq))}
+        else:
+            decl = {"q": WeightDecl((H * (D + R), h))}
+        decl |= {"dkv": WeightDecl((C + R, h)), "c_norm": WeightDecl((C,), init="ones"),
+                 "uk": WeightDecl((H * D, C)), "uv": WeightDecl((H * Dv, C)), "o": WeightDecl((h, H * Dv))}
         if params.get("sink"):
             decl["sink"] = WeightDecl((H,), init="normal")
         if params.get("gate"):
@@ -74,15 +80,19 @@ class LatentAttention(Part):
         self.scale = float(params["scale"])
         self.window = int(params.get("window") or 0)
         self.position = children["position"]
-        wq, wd = tensors["q"], tensors["dkv"]
+        self.q_rank = int(params.get("q_rank") or 0)
+        wq, wd = tensors["dq" if self.q_rank else "q"], tensors["dkv"]
         self.gated = bool(params.get("gate"))
         fused = [wq, wd] + ([tensors["g"]] if self.gated else [])
         if len({t.dtype for t in fused} | {tensors["uk"].dtype, tensors["uv"].dtype}) != 1:
             raise ValueError("the projections of a latent attention must be stored in one type")
         self.q_width = self.H * (self.D + self.R)
+        self.first_width = self.q_rank or self.q_width      # columns of the first product in front of the keys' latent
         self.dkv_width = self.C + self.R
         self.proj = Linear(torch.cat(fused, dim=0).contiguous(), rt.weight_tiles)
         self.c_norm = tensors["c_norm"]
+        self.q_norm = tensors.get("q_norm")
+        self.uq = Linear(tensors["uq"], rt.weight_tiles) if self.q_rank else None
         # a matrix a head, stored [inner, outer]: q'_h = q_h W_uk,h (W_uk,h is [D, C] as it lies), out_h = lat_h W_uv,h^T
         # (the matrix-core form of the product reads the other layout, [outer, inner]; only the one that runs is kept)
         uk, uv = tensors["uk"].view(self.H, self.D, self.C), tensors["uv"].view(self.H, self.Dv, self.C)
@@ -98,7 +108,8 @@ class LatentAttention(Part):
     def products(self):
         if self.proj.weight.dtype != torch.bfloat16:
             return []
-        return [("q_dkv_g" if self.gated else "q_dkv", self.proj.out_features, self.proj.in_features, False, None),
+        queries = [("uq", self.uq.out_features, self.uq.in_features, False, None)] if self.uq is not None else []
+        return [("q_dkv_g" if self.gated else "q_dkv", self.proj.out_features, self.proj.in_features, False, None), *queries,
                 ("o", self.o.out_features, self.o.in_features, False, "norm")]
 
     def _per_head(self, x, which, out, *, in_head, out_head):
@@ -119,7 +130,8 @@ class LatentAttention(Part):
         self.position.ensure_positions(batch.max_position + 1)
         cos, sin, rot = self.position.fused_rotary()
         y = self.proj(x)
-        q, dkv = y[:, :self.q_width], y[:, self.q_width:self.q_width + self.dkv_width]
+        first, dkv = y[:, :self.first_width], y[:, self.first_width:self.first_width + self.dkv_width]
+        q = self.uq(ops.rmsnorm(first, self.q_norm, self.eps, x.dtype)) if self.uq is not None else first
         q_full = torch.empty((x.shape[0], H * (C + R)), dtype=x.dtype, device=x.device)
         ops.latent_prep(q, dkv, q_full, heads=H, dim=D, rot_dim=R, rank=C, c_weight=self.c_norm, eps=self.eps, cos=cos,
                         sin=sin, rotary_dims=rot, positions=batch.positions, slot_of_token=batch.slot_of_token,
@@ -132,5 +144,5 @@ class LatentAttention(Part):
         heads_out = torch.empty((x.shape[0], H * Dv), dtype=x.dtype, device=x.device)
         self._per_head(latent, "uv", heads_out, in_head=C, out_head=Dv)
         if self.gated:
-            heads_out = ops.gate_mul(y[:, self.q_width + self.dkv_width:], heads_out, ops.ACT_SIGMOID)
+            heads_out = ops.gate_mul(y[:, self.first_width + self.dkv_width:], heads_out, ops.ACT_SIGMOID)
         return self.o(heads_out, out_dtype=torch.float32, partials_ok=True)   # into the 32-bit residual unrounded

@@ -1,5 +1,5 @@
 """Norms over the model width.  RMSNorm: x / sqrt(mean(x^2) + eps) * w with the plain weight w (not 1 + w);
-LayerNorm with or without a bias of its own.
+GroupRMSNorm: the same in equal groups of neighbouring entries, each by its own root mean square; LayerNorm with or without a bias of its own.
 
 crates/cuda-kernels/csrc/misc/norm.cu:8,59,221-359; the residual add fused in as at :462-.
 The weight keeps the type the checkpoint stores it in (bfloat16 or float32).
@@ -106,3 +106,37 @@ class LayerNorm(Part):
         return ops.add_layernorm(residual, terms, self.weight, self.eps, self.rt.act_dtype,
                                  weight_b=also.weight if also is not None else None, rows=rows, bias=self.bias,
                                  bias_b=also.bias if also is not None else None)
+
+
+@register("norm", "group_rmsnorm")
+class GroupRMSNorm(Part):
+    """The row in `groups` equal consecutive parts, each divided by its own sqrt(mean(part^2) + eps), the whole times w.
+    params: width, groups (default 1: the plain RMS norm), eps.
+
+    `add_norm` takes what the block before has left to add as one delta or as a `Pending` list of up to three (tensor,
+    stack of partial sums, weighted outputs of experts, or an addend with a factor a row), without biases.  `forward`
+    can also norm picked rows of a table (`rows`) into another type (`out_dtype`): an embedding that is normed."""
+
+    graph_safe = True  # launches depend on shapes only, never on the values of a step
+
+    @classmethod
+    def declare_weights(cls, params):
+        return {"weight": WeightDecl((params["width"],), init="ones")}
+
+    def __init__(self, params, tensors, rt, children=None):
+        super().__init__(params, tensors, rt, children)
+        self.weight = tensors["weight"]
+        self.width, self.groups = int(params["width"]), int(params.get("groups") or 1)
+        if self.groups < 1 or self.width % self.groups:
+            raise ValueError(f"{self.groups} groups do not divide a width of {self.width} evenly")
+        self.eps = float(params["eps"])
+
+    def forward(self, x, rows=None, out_dtype=None):
+        return ops.group_norm(x, self.weight, self.groups, self.eps, out_dtype or self.rt.act_dtype, rows=rows)
+
+    def add_norm(self, residual, delta, rows=None):
+        terms = delta if isinstance(delta, list) else ([] if delta is None else [(delta, None)])
+        if any(bias is not None for _, bias in terms):
+            raise ValueError("a group norm adds terms without biases")
+        return ops.group_norm(residual, self.weight, self.groups, self.eps, self.rt.act_dtype,
+                              terms=[term for term, _ in terms], rows=rows)
