@@ -7,6 +7,7 @@
     python bench.py --workload sovutar [--shape 4b|8b] [--layers L]  (the Sovutar design beside Qwen3 at equal sizes)
     python bench.py --workload tazitar [--shape 4b|8b] [--layers L]  (the Tazitar design beside Qwen3 at equal sizes)
     python bench.py --workload retudra [--shape 4b|8b] [--layers L]  (the Retudra design beside Sovutar and Qwen3 at equal sizes)
+    python bench.py --workload nafezen [--shape 4b|8b] [--layers L]  (the Nafezen design beside Retudra and Qwen3 at equal sizes)
 
 A step is one decode step of `batch` requests, each holding a `prompt`-token random prompt
 (prefilled by the engine itself before the clock starts) and growing by one token per step.
@@ -120,7 +121,8 @@ def classify_step(names, layers: int) -> list:
 def profiled_steps(torch, fns) -> list:
     """The kernels of every call in `fns`, run one after the other inside ONE profiler session (a second session
     in a process has crashed the profiler here): a list, one entry a call, of (name, microseconds) in launch
-    order.  A step begins with the embedding kernel, which is how the session's kernels are cut into calls."""
+    order.  A step begins with the embedding kernel (the gather, or the grouped norm that reads bfloat16 rows: the table's;
+    all later ones read the float32 residual), which is how the session's kernels are cut into calls."""
     from torch.profiler import ProfilerActivity, profile
 
     torch.cuda.synchronize()
@@ -134,7 +136,7 @@ def profiled_steps(torch, fns) -> list:
     steps, early = [], []
     for e in evs:
         item = (e.name, e.time_range.end - e.time_range.start)
-        if "embed_gather" in e.name:
+        if "embed_gather" in e.name or ("group_norm" in e.name and e.name.split("<")[1].startswith(("arle::bf16", "bf16"))):
             steps.append(early + [item])     # what ran before the first step's embedding is counted with it
             early = []
         elif steps:
@@ -978,6 +980,82 @@ def retudra_bench(args) -> int:
                         {"sovutar": lambda tokens, batch, context: sovutar_work(sov, q, tokens, batch, context)})
 
 
+# ---- the Nafezen design beside Retudra and Qwen3 at equal sizes ------------------------------------------
+# The widths and head counts of Qwen3-4B / 8B; layers alternate between the retention (its states as large as those of
+# Retudra's delta rule) and the latent attention (Retudra's sizes, with a latent of 768 for the queries); the first
+# layer's feed-forward is dense, the others have sixteen squared-relu experts, four choices a token, and a shared one;
+# norms in four groups.
+def nafezen_config(shape: str, layers: int) -> dict:
+    q, span, ff = SOVUTAR_SHAPES[shape]
+    H, D = q["num_attention_heads"], q["head_dim"]
+    ret = {"heads": H, "dim": D, "vdim": D, "decay": [1.0 - 2.0 ** -(3.0 + 5.0 * h / H) for h in range(H)],
+           "rot": {"base": 1000000.0, "dims": D}}
+    lat = {"heads": H, "dim": D, "rot_dim": 64, "vdim": D, "kv_rank": 192, "q_rank": 768, "scale": (D + 64) ** -0.5,
+           "rot": {"base": 1000000.0, "dims": 64}}
+    kinds = [("retention", ret), ("latent_attention", lat)]
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": 16, "top": 4}, "shared": {"ff": ff}}
+    out = [{"type": kinds[i % 2][0], "mixer": json.loads(json.dumps(kinds[i % 2][1])),
+            "mlp": {"kind": "dense", "ff": q["intermediate_size"]} if i == 0 else json.loads(json.dumps(moe))}
+           for i in range(layers)]
+    return {"architecture": "Nafezen", "vocab": q["vocab_size"], "width": q["hidden_size"], "norm": {"eps": 1e-6, "groups": 4},
+            "layers": out}
+
+
+def nafezen_work(raw: dict, tokens: int, batch: int, context: int) -> dict:
+    """Ideal work of the design's kernels, per step: kernel family -> (bytes, flops)."""
+    W, L = raw["width"], len(raw["layers"])
+    of = lambda kind: [l for l in raw["layers"] if l["type"] == kind]
+    n_ret, n_lat = len(of("retention")), len(of("latent_attention"))
+    moes = [l["mlp"] for l in raw["layers"] if l["mlp"] and l["mlp"]["kind"] == "moe"]
+    decode = tokens == batch
+    work = {}
+    top = moes[0]["router"]["top"] if moes else 0
+    # a layer's norm: the residual in and out, its normed copy, and what the layer before left (the mixer's and the
+    # feed-forward's 32-bit outputs; behind a mixture the chosen experts' and the shared one's)
+    work["group_norm"] = (tokens * W * (2 + 4 * 2 + (L + 1) * (4 + 4 + 2) + (L - len(moes)) * 8 + len(moes) * (top + 2) * 4), 0)
+    if n_lat:
+        m = of("latent_attention")[0]["mixer"]
+        LH, LD, R, LDv, C, Cq = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["q_rank"]
+        keys = context if decode else tokens / 2
+        work["attn_softcap_mfma_kernel"] = (n_lat * batch * keys * (2 * C + R) * 2 if decode else 0,
+                                            n_lat * tokens * keys * LH * 2 * (2 * C + R))
+        work["rmsnorm"] = (n_lat * tokens * Cq * 4, 0)
+        work["latent_down"] = (n_lat * tokens * ((Cq + C + R) * 4 + (Cq + 2 * C + R) * 2), 0)
+        work["latent_prep_kernel"] = (n_lat * tokens * (LH * R * 2 + (C + R) + 2 * C + R) * 2, 0)
+        work["head_proj"] = (n_lat * (tokens * LH * (LD + 2 * C + LDv) * 2 + LH * C * (LD + LDv) * 2),
+                             n_lat * tokens * LH * C * (LD + LDv) * 2)
+    if n_ret:
+        r = of("retention")[0]["mixer"]
+        H, D, Dv = r["heads"], r["dim"], r["vdim"]
+        state = H * D * Dv
+        rows = H * (2 * D + 2 * Dv) * 4 + H * Dv * 2      # q, k, v and the gate in 32 bits, the output in 16
+        work["retention_decode_kernel"] = (n_ret * (batch * state * 8 + tokens * rows), n_ret * tokens * state * 4)
+        work["retention_chunk_sum"] = (n_ret * tokens * H * (D + Dv) * 4, n_ret * tokens * state * 2)
+        work["retention_chunk_carry"] = (n_ret * batch * state * 8, 0)
+        work["retention_chunk_out"] = (n_ret * tokens * rows, n_ret * tokens * state * 2)
+    if moes:
+        E, F = moes[0]["router"]["experts"], moes[0]["expert"]["ff"]
+        active = min(E, batch * top) if decode else E
+        n = len(moes)
+        work["moe_route_kernel"] = (n * (tokens + E + 1) * W * 2, 0)
+        work["moe_expert"] = (n * (active * 2 * W * F * 2 + tokens * top * (W * 2 + F * 4 + W * 4)), n * tokens * top * 2 * 2 * W * F)
+    return work
+
+
+def nafezen_bench(args) -> int:
+    """Prefill and decode throughput of the Nafezen design, of Retudra (the closest design: a recurrent state beside a
+    latent attention, a mixture of experts) and of Qwen3 at the same widths and depth."""
+    from arle_amd.config import NafezenConfig, Qwen3Config, RetudraConfig
+
+    layers = args.layers if args.layers != FULL_LAYERS else 8
+    q = dict(SOVUTAR_SHAPES[args.shape][0], num_hidden_layers=layers)
+    raw, ret = nafezen_config(args.shape, layers), retudra_config(args.shape, layers)
+    models = {"nafezen": ("Nafezen", NafezenConfig.from_dict(raw)), "retudra": ("Retudra", RetudraConfig.from_dict(ret)),
+              "qwen3": ("Qwen3ForCausalLM", Qwen3Config.from_dict(q))}
+    return design_bench(args, "nafezen", models, q, layers, lambda tokens, batch, context: nafezen_work(raw, tokens, batch, context),
+                        {"retudra": lambda tokens, batch, context: retudra_work(ret, q, tokens, batch, context)})
+
+
 def tazitar_bench(args) -> int:
     """Prefill and decode throughput of the Tazitar design and of Qwen3 at the same widths and depth."""
     from arle_amd.config import Qwen3Config, TazitarConfig
@@ -1138,10 +1216,10 @@ def main() -> int:
                          "and write the table that ARLE_AMD_PRODUCT_TABLE / ops.load_product_table reads; WIDTHS: 4b, 8b, "
                          "32b or hidden,q_width,kv_width,intermediate[,vocabulary]")
     ap.add_argument("--out", default=None, help="--tune-products: the table's file (default: product_table_<widths>.json)")
-    ap.add_argument("--workload", default="qwen3-4b", choices=["qwen3-4b", "qwen3-8b-mixed", "qwen3-32b-decode", "gufasun", "sovutar", "tazitar", "retudra"],
+    ap.add_argument("--workload", default="qwen3-4b", choices=["qwen3-4b", "qwen3-8b-mixed", "qwen3-32b-decode", "gufasun", "sovutar", "tazitar", "retudra", "nafezen"],
                     help="qwen3-4b is the default run; the next two are further workloads at larger shapes; gufasun: "
                          "the Gufasun design beside Qwen3 at equal widths and depth (--shape, --layers, --batch, --prompt-len)")
-    ap.add_argument("--shape", default="4b", choices=["4b", "8b"], help="--workload gufasun / sovutar / tazitar / retudra: whose widths")
+    ap.add_argument("--shape", default="4b", choices=["4b", "8b"], help="--workload gufasun / sovutar / tazitar / retudra / nafezen: whose widths")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path (asked for --gpus {args.gpus})")
@@ -1169,6 +1247,8 @@ def main() -> int:
         return tazitar_bench(args)
     if args.workload == "retudra":
         return retudra_bench(args)
+    if args.workload == "nafezen":
+        return nafezen_bench(args)
     if args.workload == "qwen3-4b" and args.batch is None:
         args.batch = 8
     if args.workload != "qwen3-4b":

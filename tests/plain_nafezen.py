@@ -103,8 +103,8 @@ def squared_relu_ff(h, up, down):
     return mm(torch.relu(mm(h, up)) ** 2, down)
 
 
-# every call of `route` leaves here, a token, how far its choice was from another one: the chosen logit that is
-# smallest less the largest that was not chosen (infinity where every expert is chosen)
+# every call of `route` leaves here, a token, how far its choice was from another one: the smallest chosen logit less
+# the largest that was not chosen, over the root mean square of the token's logits (infinity where all are chosen)
 route_margins: list = []
 
 
@@ -112,7 +112,8 @@ def route(h, top, router, bias):
     """-> (chosen [T, top] indices, weights [T, top]): the largest logits, and the softmax over just those."""
     z = mm(h, router) + (bias if bias is not None else 0.0)
     ordered = torch.sort(z, dim=-1, descending=True).values
-    route_margins.append(ordered[:, top - 1] - ordered[:, top] if top < z.shape[1]
+    size = torch.sqrt((z * z).mean(-1))
+    route_margins.append((ordered[:, top - 1] - ordered[:, top]) / size if top < z.shape[1]
                          else torch.full((h.shape[0],), float("inf"), dtype=F))
     best = torch.topk(z, top, dim=-1)
     return best.indices, torch.softmax(best.values, dim=-1)

@@ -1,0 +1,611 @@
+"""Nafezen on the GPU against the plain implementation (`plain_nafezen.py`): every mechanism alone as the part or the
+operation the engine runs, in cuts of every size, and whole models through `Engine.step`, the scheduler and
+`LLM.generate`.
+
+Tolerances.  float32: 5e-5 of the largest plain logit for whole models, 5e-5 of the largest plain output for a mechanism
+alone (the plain side is float64; the engine adds in 32 bits).  bfloat16: 3e-2 of the largest plain logit for whole
+models, 2.5e-2 of the largest plain output for a mechanism alone.
+"""
+import pytest
+import torch
+
+import plain_nafezen as plain
+import replay
+from arle_amd import LLM
+from arle_amd.cache import CacheManager
+from arle_amd.config import NafezenConfig
+from arle_amd.engine import Engine, StepEntry
+from arle_amd.engine.batch import build_step_batch
+from arle_amd.kernels import ops
+from arle_amd.models.nafezen import nafezen_spec
+from arle_amd.parts.base import Runtime, build_part, expected_tensors
+from arle_amd.parts.position import rope_table
+from arle_amd.parts.spec import PartSpec
+from tiny import random_tokens, read_folder
+from tiny_nafezen import ARCH, TINY, dense, latent, layer, make_model_dir, moe, retention, rot
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+F32, BF16 = torch.float32, torch.bfloat16
+TOL = {F32: 5e-5, BF16: 2.5e-2}
+EPS = 1e-5
+
+
+def rnd(shape, seed, std=1.0):
+    g = torch.Generator().manual_seed(seed)
+    return (torch.randn(shape, generator=g) * std).to(BF16).float()     # values that bfloat16 holds exactly
+
+
+def close(got, want, dtype, what, tol=None):
+    got, want = got.double().cpu(), want.double()
+    assert torch.isfinite(got).all(), what
+    err = float((got - want).abs().max()) / float(want.abs().max())
+    assert err <= (tol or TOL[dtype]), f"{what}: {err:.3e}"
+
+
+def one_layer(kind, mixer, mlp=None, width=40, groups=1):
+    """(config dictionary, ModelSpec) of a model of one layer."""
+    raw = {"architecture": ARCH, "vocab": 50, "width": width, "norm": {"eps": EPS, "groups": groups},
+           "layers": [layer(kind, mixer, mlp)]}
+    return raw, nafezen_spec(NafezenConfig.from_dict(raw))
+
+
+def random_part(role, spec, dtype, seed, std=0.3, fills=None):
+    """A part of `spec` with random tensors; returns (part, {checkpoint name: float32 CPU tensor})."""
+    tensors = {}
+    for i, (name, decl) in enumerate(sorted(expected_tensors(role, spec).items())):
+        t = rnd(tuple(decl.shape), seed + i, std)
+        if decl.init == "ones":
+            t = 1 + rnd(tuple(decl.shape), seed + i, 0.3)
+        for suffix, fill in (fills or {}).items():
+            if name.endswith(suffix):
+                t = fill(t, seed + i)
+        tensors[name] = t
+    rt = Runtime(device=torch.device(DEV), act_dtype=dtype)
+    held = {k: v.to(DEV, dtype) for k, v in tensors.items()}
+    return build_part(role, spec, held.__getitem__, rt), tensors
+
+
+def run_mixer(part, x, cuts, *, page=4, dtype=F32):
+    """Feed x [T, W] of one request to a mixer in portions of the given sizes (repeating), through a cache in which
+    another request's pages and slot lie between, every page starts as NaN and the other request's state is rubbish.
+    Returns the concatenated outputs."""
+    T = x.shape[0]
+    part.prepare(T + page)
+    cache = CacheManager([part.cache_need()], page_size=page, num_pages=2 * (-(-T // page)) + 4, max_slots=3,
+                         max_request_tokens=T + page, device=torch.device(DEV), dtype=dtype)
+    cache.admit("other")
+    cache.append([("other", page + 1)])
+    for group in cache.page_buffers:
+        for t in group.values():
+            t.fill_(float("nan"))
+    cache.admit("r")
+    state = getattr(cache.view(0), "state", None)
+    if state is not None:
+        state[cache.slot_of["other"]] = float("nan")
+    outs, at, k = [], 0, 0
+    xd = x.to(DEV, dtype)
+    while at < T:
+        n = min(cuts[k % len(cuts)], T - at)
+        k += 1
+        before = cache.length("r")
+        cache.append([("r", n)])
+        cache.sync_tables()
+        batch = build_step_batch([StepEntry("r", [0] * n, [])], cache.slot_of.__getitem__, lambda _r, b=before: b, 10, DEV)
+        y = part.forward(xd[at:at + n].contiguous(), batch, cache.view(0))
+        outs.append((y.float().sum(0) if y.dim() == 3 else y.float()).cpu())
+        at += n
+    cache.check()
+    return torch.cat(outs)
+
+
+CUTS = [(1000,), (1,), (2,), (5, 2, 7, 3, 1, 16, 2)]
+
+
+def mixer_case(kind, mixer, dtype, seed, T, *, page=4, loud=(), std=0.3, cuts=CUTS, tol=None, limits=None):
+    """A mixer alone against its plain function, in every cutting; in float32 the cuttings agree bit for bit.
+    loud: positions whose input dwarfs the others', so that a key seen or hidden by mistake shows.
+    limits(x, w, want) -> a bound for every row beside the tolerance."""
+    raw, spec = one_layer(kind, mixer)
+    part, tensors = random_part("mixer", spec.layers[0].mixer, dtype, seed, std)
+    x = rnd((T, raw["width"]), seed + 100)
+    for p in loud:
+        if 0 <= p < T:
+            x[p] *= 6.0
+    w = lambda name: tensors["l0.mix." + name].double()
+    want = plain.MIXERS[kind](x.double(), mixer, w, EPS)
+    bound = torch.full((T,), tol or TOL[dtype], dtype=torch.float64)
+    if limits is not None:
+        bound = torch.maximum(bound, limits(x.double(), w, want))
+    first = None
+    for c in cuts:
+        got = run_mixer(part, x, c, page=page, dtype=dtype)
+        assert torch.isfinite(got).all()
+        err = (got.double() - want).abs().max(1).values / want.abs().max()
+        worst = int((err / bound).argmax())
+        assert err[worst] <= bound[worst], f"{kind} {dtype} cut {c}: row {worst} is off by {float(err[worst]):.3e}"
+        if dtype == F32:
+            first = got if first is None else first
+            assert torch.equal(got, first), f"{kind}: cut {c} differs in bits from the whole prompt"
+
+
+def product_jitter(kind, mixer, dtype):
+    """What moving every entry of every product by up to half a unit in the last place does to a row, eight times: the
+    read-out's norm magnifies rounding where the terms of o nearly cancel (most at a request's first rows)."""
+    unit = 2.0 ** -24 if dtype == F32 else 2.0 ** -9
+
+    def limits(x, w, want):
+        found = torch.zeros(x.shape[0], dtype=torch.float64)
+        for trial in range(3):
+            g = torch.Generator().manual_seed(50 + trial)
+            plain.after_product = lambda y: y * (1 + (torch.rand(y.shape, generator=g, dtype=torch.float64) - 0.5) * 2 * unit)
+            try:
+                moved = plain.MIXERS[kind](x, mixer, w, EPS)
+            finally:
+                plain.after_product = None
+            found = torch.maximum(found, 8.0 * (moved - want).abs().max(1).values / want.abs().max())
+        return found
+
+    return limits
+
+
+# ----------------------------------------------------------------------------------- the grouped norm
+
+@pytest.mark.parametrize("width,groups,rows", [(72, 3, 5), (1001, 7, 3), (4096, 1, 2), (42, 7, 4), (80, 20, 3), (2560, 4, 600),
+                                               (5120, 8, 3), (6144, 2, 520), (16384, 64, 2), (16384, 16384, 2), (320, 320, 3),
+                                               (2048, 16, 513), (1, 1, 2)])
+def test_the_grouped_norm_adds_what_is_left_and_norms_every_group_by_itself(width, groups, rows):
+    res = rnd((rows, width), 1, 2.0) * (1 + torch.arange(width) * groups // width).float()     # groups of different sizes
+    w = 1 + rnd((width,), 2, 0.3)
+    y, stack = rnd((rows, width), 3, 3.0), rnd((5, rows, width), 4)
+    outs, coefs, shared, factor = rnd((rows, 3, width), 5), rnd((rows, 3), 6), rnd((2, rows, width), 7), rnd((rows,), 8)
+    d = lambda t: t.to(DEV)
+    weighted = (outs * coefs[:, :, None]).sum(1)
+    scaled = shared.sum(0) * factor[:, None]
+    cases = [([], torch.zeros(rows, width)), ([d(y)], y), ([d(stack)], stack.sum(0)),
+             ([d(stack), (d(outs), d(coefs))], stack.sum(0) + weighted),
+             ([d(y), (d(outs), d(coefs)), ops.Scaled(d(shared), d(factor))], y + weighted + scaled),
+             ([ops.Scaled(d(y), d(factor))], y * factor[:, None])]
+    for terms, total in cases:
+        want_x = res.double() + total.double()
+        want = plain.group_norm(want_x, w.double(), groups, EPS)
+        for dtype in (F32, BF16):
+            r32 = d(res).clone()
+            got = ops.group_norm(r32, d(w).to(dtype), groups, EPS, dtype, terms=terms)
+            close(r32, want_x, F32, "the residual")
+            close(got, plain.group_norm(want_x, w.to(dtype).double(), groups, EPS), dtype, f"{len(terms)} terms {dtype}",
+                  tol=1e-2 if dtype == BF16 else 1e-5)
+        # picked rows (the last norm): read with what is left to add, not written back
+        picks = torch.tensor([rows - 1, 0], dtype=torch.int32, device=DEV)
+        r32 = d(res).clone()
+        got = ops.group_norm(r32, d(w), groups, EPS, F32, terms=terms, rows=picks)
+        close(got, want[[rows - 1, 0]], F32, "picked rows", tol=1e-5)
+        assert torch.equal(r32.cpu(), res)
+    if groups > 1 and groups < width:
+        assert float((plain.group_norm(want_x, w.double(), 1, EPS) - want).abs().max()) > 0.05 * float(want.abs().max())
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("width,groups", [(72, 3), (42, 7), (2560, 4)])
+def test_the_embedding_is_normed_on_its_way_into_the_residual(dtype, width, groups):
+    norm = PartSpec("group_rmsnorm", {"width": width, "groups": groups, "eps": EPS}, {"weight": "n"})
+    spec = PartSpec("token_table", {"vocab_size": 33, "hidden_size": width, "norm": norm}, {"table": "t"})
+    part, tensors = random_part("embedding", spec, dtype, 5, 1.0)
+    tokens = [32, 0, 7, 7, 31]
+    got = part.forward(torch.tensor(tokens, dtype=torch.int32, device=DEV))
+    assert got.dtype == F32
+    close(got, plain.group_norm(tensors["t"].double()[tokens], tensors["n"].double() if dtype == F32 else
+                                tensors["n"].to(BF16).double(), groups, EPS), F32, "normed embedding", tol=1e-5)
+
+
+# ----------------------------------------------------------------------------------- the latent attention
+
+LATENTS = [
+    (latent(4, 16, 8, 12, 24, 20, scale=0.3, rot=rot(500.0, 8)), 4, 50),
+    (latent(1, 10, 6, 14, 18, 9, scale=0.4, rot=rot(50.0, 4)), 8, 40),          # one head; only part of the rotated part turns
+    (latent(4, 32, 32, 48, 64, 48, scale=0.12, rot=rot(250000.0, 32)), 16, 130),
+    (latent(6, 64, 32, 48, 112, 72, scale=0.1, rot=rot(100000.0, 32)), 16, 90),
+    (latent(3, 8, 2, 8, 6, 33, scale=0.5, rot=rot(10.0, 2)), 4, 30),
+    (latent(2, 16, 64, 32, 320, 16, scale=0.15, rot=rot(1000.0, 64)), 16, 60),   # keys wider than the matrix cores' kernel takes
+]
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("case", range(len(LATENTS)))
+def test_the_latent_attention_makes_its_queries_through_a_latent_too(dtype, case):
+    mixer, page, T = LATENTS[case]
+    mixer_case("latent_attention", mixer, dtype, 40 + 20 * case, T, page=page, loud=(0, page - 1, page, T // 2), std=0.2,
+               tol=4e-2 if dtype == BF16 else None)
+
+
+def far_key_inputs(tensors, mixer, T, W, target):
+    """Inputs in which the latent at `target` lies along what the last row's first head asks for: its score stands out
+    among T, and its value decides the last row's output."""
+    w = lambda name: tensors["l0.mix." + name].double()
+    x = rnd((T, W), 3, 0.5)
+    cq = plain.unit_rms(x[T - 1].double() @ w("dq").T, EPS) * w("dq.norm")
+    q = (cq @ w("uq").T)[:mixer["dim"]]
+    asked = (w("uk")[:mixer["dim"]].T @ q) / w("dkv.norm")
+    along = torch.linalg.lstsq(w("dkv")[:mixer["kv_rank"]], asked[:, None]).solution[:, 0]
+    x[target] = (along / along.pow(2).mean().sqrt()).to(BF16).float()
+    return x
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+def test_a_far_latent_is_found(dtype):
+    T, W = 400, 48
+    mixer = latent(2, 16, 8, 16, 24, 20, scale=1.0, rot=rot(1e6, 8))
+    raw, spec = one_layer("latent_attention", mixer, width=W)
+    part, tensors = random_part("mixer", spec.layers[0].mixer, dtype, 77, 0.25)
+    w = lambda name: tensors["l0.mix." + name].double()
+    for target in (0, 63, 64, T - 17, T - 16):      # the first token, and both sides of pages' borders
+        x = far_key_inputs(tensors, mixer, T, W, target)
+        other = x.clone()
+        other[target] = rnd((W,), 4, 0.5)
+        want = plain.latent_attention(x.double(), mixer, w, EPS)
+        without = plain.latent_attention(other.double(), mixer, w, EPS)
+        assert float((want[-1] - without[-1]).abs().max()) > 0.2 * float(want[-1].abs().max()), "the test's own inputs must make it matter"
+        for c in ((1000,), (7, 1)):
+            close(run_mixer(part, x, c, page=16, dtype=dtype)[-1], want[-1], dtype, f"far key at {target}, cut {c}",
+                  tol=4e-2 if dtype == BF16 else None)
+
+
+# ----------------------------------------------------------------------------------- retention
+
+RETENTIONS = [
+    (retention(3, 16, 24, (0.5, 0.9, 0.99), rot(10000.0, 12)), 50),          # a rotation the chunks' form refuses
+    (retention(1, 10, 6, (0.9375,)), 70),                                    # sizes it refuses, no rotation
+    (retention(2, 64, 128, (1.0, 0.0), rot(250000.0, 32)), 200),
+    (retention(4, 32, 64, (0.98, 0.998, 0.9, 0.6), rot(1000.0, 32)), 193),
+    (retention(2, 128, 36, (0.99, 0.8), rot(800.0, 64)), 130),
+    (retention(1, 40, 20, (0.95,), rot(800.0, 8)), 150),
+    (retention(2, 132, 200, (0.97, 0.5), rot(100.0, 132)), 90),              # a rotation of 132 entries: row by row
+    (retention(1, 256, 256, (0.999,), rot(1e6, 256)), 140),
+    (retention(3, 20, 4, (0.9, 0.99, 0.3)), 129),
+]
+RET_CUTS = CUTS + [(64, 1), (63, 65, 2), (17, 1, 1, 33), (128, 3)]
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("case", range(len(RETENTIONS)))
+def test_retention_equals_the_plain_recurrence_in_every_cut(dtype, case):
+    mixer, T = RETENTIONS[case]
+    # loud rows at a chunk's borders and at the start: their terms are heard as far as the decay reaches
+    mixer_case("retention", mixer, dtype, 200 + 20 * case, T, loud=(0, 63, 64), std=0.25, cuts=RET_CUTS,
+               tol=2e-4 if dtype == F32 else None, limits=product_jitter("retention", mixer, dtype))
+
+
+OP_CASES = [
+    # (heads, key size, value size, rotated entries, decays, segments: (rows now, position of the first))
+    (2, 64, 128, 64, (0.96, 0.999), [(64, 0)]),
+    (3, 32, 64, 32, (1.0, 0.0, 0.7), [(1, 0), (65, 17), (1, 900), (128, 0), (2, 5)]),
+    (1, 128, 256, 32, (0.9,), [(200, 3), (63, 64)]),
+    (2, 256, 40, 0, (0.99, 0.5), [(31, 0), (97, 128)]),
+    (2, 24, 20, 8, (0.95, 0.8), [(129, 0), (16, 1), (17, 40)]),
+    (5, 4, 4, 0, (0.9, 0.8, 0.7, 0.6, 0.5), [(70, 0)]),
+]
+
+
+@pytest.mark.parametrize("case", range(len(OP_CASES)))
+@pytest.mark.parametrize("form", ["rows", "chunks", "decode"])
+def test_the_three_forms_of_retention_agree_with_float64_from_a_state_on(case, form):
+    """Segments of several requests with states of their own in slots out of order, 32-bit in and out."""
+    H, D, Dv, rotated, decays, segments = OP_CASES[case]
+    if form == "decode":
+        segments = [(1, start) for _, start in segments]
+    N, T = 2 * H * (D + Dv), sum(n for n, _ in segments)
+    y = rnd((T, N), 7 + case)
+    slots = [2 * i + 1 for i in reversed(range(len(segments)))]
+    state = rnd((2 * len(segments) + 1, H, D, Dv), 9 + case, 0.5)
+    cos, sin = rope_table(rotated, 10000.0, 1200) if rotated else (None, None)
+    pos = torch.cat([torch.arange(start, start + n) for n, start in segments]).to(torch.int32)
+    row0 = torch.tensor([0] + [n for n, _ in segments]).cumsum(0).to(torch.int32)
+    # float64, one row after the other
+    want, after = torch.zeros(T, H * Dv, dtype=torch.float64), state.double().clone()
+    for s, (n, start) in enumerate(segments):
+        for t in range(int(row0[s]), int(row0[s]) + n):
+            r = y[t].double()
+            p = pos[t:t + 1].long()
+            q = plain.rotate_half(r[:H * D].view(1, H, D), p, rotated, 10000.0)[0]
+            k = plain.rotate_half(r[H * D:2 * H * D].view(1, H, D), p, rotated, 10000.0)[0] * D ** -0.5
+            v = r[2 * H * D:2 * H * D + H * Dv].view(H, Dv)
+            S = after[slots[s]] * torch.tensor(decays, dtype=torch.float64)[:, None, None] + k[:, :, None] * v[:, None, :]
+            after[slots[s]] = S
+            o = plain.unit_rms(torch.einsum("hde,hd->he", S, q), EPS).reshape(-1)
+            want[t] = o * plain.silu(r[2 * H * D + H * Dv:])
+    d = lambda t: t.to(DEV) if t is not None else None
+    powers = torch.tensor(decays, dtype=torch.float64)[:, None] ** torch.arange(65, dtype=torch.float64)
+    common = dict(positions=d(pos), cos=d(cos), sin=d(sin), rotary_dims=rotated, heads=H, key_dim=D, value_dim=Dv)
+    for out_dtype in (F32, BF16):
+        held = d(state).clone()
+        where = (held, d(row0), torch.tensor(slots, dtype=torch.int32, device=DEV), EPS, out_dtype)
+        if form == "chunks":
+            assert ops.retention_chunks_supported(T, len(segments), H, D, Dv, rotated)
+            got = ops.retention_chunks(d(y), d(powers.float()), *where, **common)
+        elif form == "rows":
+            got = ops.retention_rows(d(y).clone(), d(torch.tensor(decays)), *where, **common)
+        else:
+            stack = torch.stack([d(y) * 0.5, d(y) * 0.25, d(y) * 0.25])      # partial sums of the product, exact halves
+            got = ops.retention_decode(stack, d(torch.tensor(decays)), *where, **common)
+        close(got, want, out_dtype, f"{form} {out_dtype}", tol=1e-2 if out_dtype == BF16 else 1e-4)
+        close(held, after, F32, "the states", tol=1e-5)
+        untouched = [s for s in range(state.shape[0]) if s not in slots]
+        assert torch.equal(held.cpu()[untouched], state[untouched]), "other slots keep theirs"
+
+
+def test_retention_over_long_decoding():
+    mixer = retention(2, 32, 16, (0.999, 0.9), rot(1000.0, 32))
+    raw, spec = one_layer("retention", mixer)
+    x = rnd((460, raw["width"]), 91)
+    for dtype in (F32, BF16):
+        part, tensors = random_part("mixer", spec.layers[0].mixer, dtype, 90, 0.25)
+        w = lambda name: tensors["l0.mix." + name].double()
+        want = plain.retention(x.double(), mixer, w, EPS)
+        got = run_mixer(part, x, (60,) + (1,) * 400, dtype=dtype)
+        close(got[60:], want[60:], dtype, "400 rows decoded one by one", tol=2e-4 if dtype == F32 else 3e-2)
+
+
+# ----------------------------------------------------------------------------------- the feed-forwards
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("width,ff,rows", [(40, 24, 5), (42, 30, 3), (96, 128, 80), (256, 1024, 300), (2048, 512, 9)])
+def test_the_squared_relu_feed_forward(dtype, width, ff, rows):
+    spec = PartSpec("squared_relu", {"hidden_size": width, "intermediate_size": ff}, {"up": "u", "down": "d"})
+    part, tensors = random_part("feed_forward", spec, dtype, 5, width ** -0.5)
+    x = rnd((rows, width), 6)
+    y = part.forward(x.to(DEV, dtype))
+    assert y.dtype == F32
+    y = y.sum(0) if y.dim() == 3 else y
+    close(y, plain.squared_relu_ff(x.double(), tensors["u"].double(), tensors["d"].double()), dtype, "squared relu")
+
+
+ROUTERS = [
+    # (experts, top, width, ff, shared)
+    (6, 2, 72, 40, 56), (5, 3, 40, 24, 24), (4, 1, 42, 30, None), (7, 7, 96, 48, 64), (9, 3, 80, 40, 72), (2, 2, 64, 16, 8),
+    (70, 6, 128, 64, 128), (1, 1, 48, 32, 10), (3, 2, 42, 18, 10),
+]
+
+
+def weighed(terms):
+    """The sum of what a mixture of experts leaves to be added."""
+    total = 0.0
+    for t in terms:
+        if isinstance(t, ops.Scaled):
+            y = t.delta.double().sum(0) if t.delta.dim() == 3 else t.delta.double()
+            total = total + y * t.factor.double()[:, None]
+        elif isinstance(t, tuple):
+            total = total + (t[0].double() * t[1].double()[:, :, None]).sum(1)
+        else:
+            total = total + (t.double().sum(0) if t.dim() == 3 else t.double())
+    return total
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("case", range(len(ROUTERS)))
+def test_the_router_weighs_the_chosen_by_their_own_softmax_and_the_shared_expert_is_gated(dtype, case):
+    experts, top, width, ff, shared = ROUTERS[case]
+    mlp = moe(experts, top, ff, shared)
+    raw, spec = one_layer("retention", retention(1, 8, 8, (0.5,)), mlp, width=width)
+    fills = {".router.b": lambda t, s: rnd(t.shape, s, 1.0)}
+    part, tensors = random_part("feed_forward", spec.layers[0].feed_forward, dtype, 300 + 7 * case, width ** -0.5 * 1.5, fills)
+    w = lambda name: tensors["l0.mlp." + name].double()
+    for rows in (1, 9, 70, 300):
+        x = rnd((rows, width), 7 + rows)
+        chosen, weights = plain.route(x.double(), top, w("router"), w("router.b"))
+        dev = lambda name: tensors["l0.mlp." + name].to(DEV, dtype)
+        found = ops.moe_route(x.to(DEV, dtype), dev("router"), None, top=top, scale=1.0, score="softmax_chosen",
+                              bias=dev("router.b"), shared_gate=dev("shared.sg") if shared else None)
+        z = x.double() @ w("router").T + w("router.b")
+        gaps = (z[:, :, None] - z[:, None, :]).abs() + 10.0 * torch.eye(experts)
+        clear = gaps.flatten(1).min(1).values > 1e-5      # (the router's sums are 32-bit in both modes, from the same inputs)
+        assert clear.sum() >= rows // 2 or rows == 1
+        assert torch.equal(found[0].cpu().long()[clear], chosen[clear]), "the chosen experts, in the order they were chosen"
+        close(found[1].cpu()[clear], weights[clear], F32, "their weights")
+        if shared:
+            close(found[2], torch.sigmoid(x.double() @ w("shared.sg").T)[:, 0], F32, "the shared expert's gate")
+        if bool(clear.all()):
+            close(weighed(part.forward(x.to(DEV, dtype))), plain.mixture(x.double(), mlp, w), dtype, f"the mixture at {rows} rows")
+
+
+def test_logits_far_apart_and_all_negative_are_chosen_by_their_size():
+    """Logits whose exponentials vanish beside the largest are still ordered, and negative ones are no less chosen."""
+    width, experts = 16, 8
+    bias = torch.tensor([-500.0, -20.0, -900.0, -300.0, -250.0, -700.0, -400.0, -600.0])
+    x = rnd((5, width), 2, 0.1)
+    router = rnd((experts, width), 3, 0.1)
+    ids, weights = ops.moe_route(x.to(DEV), router.to(DEV), None, top=4, scale=1.0, score="softmax_chosen", bias=bias.to(DEV))
+    assert ids.cpu().tolist() == [[1, 4, 3, 6]] * 5
+    assert torch.allclose(weights.cpu().sum(1), torch.ones(5)) and bool((weights[:, 0] > 0.999).all())
+
+
+def test_the_products_of_ungated_experts_next_to_each_other():
+    """Experts whose rows are next to each other in a portion, and a tile's border in rows and columns."""
+    for tokens, E, top, N, K in ((300, 3, 1, 200, 64), (64, 5, 2, 130, 40), (65, 2, 2, 16, 24), (600, 4, 3, 257, 128)):
+        x, up, down = rnd((tokens, K), 1), rnd((E, N, K), 2, K ** -0.5), rnd((E, K, N), 3, N ** -0.5)
+        ids = torch.stack([torch.randperm(E, generator=torch.Generator().manual_seed(t))[:top] for t in range(tokens)]).to(torch.int32)
+        for dtype in (F32, BF16):
+            act = ops.moe_expert(x.to(DEV, dtype), up.to(DEV, dtype), ids.to(DEV), ops.MOE_UP)
+            want = torch.relu(torch.einsum("tk,tjnk->tjn", x.double(), up.double()[ids.long()])) ** 2
+            close(act.view(tokens, top, N), want, dtype, f"up {tokens} {dtype}", tol=1e-2 if dtype == BF16 else None)
+            outs = ops.moe_expert(act, down.to(DEV, dtype), ids.to(DEV), ops.MOE_DOWN)
+            want = torch.einsum("tjn,tjkn->tjk", act.double().cpu().view(tokens, top, N), down.double()[ids.long()])
+            close(outs.view(tokens, top, K), want, F32, f"down {tokens} {dtype}", tol=1e-5)
+
+
+# ----------------------------------------------------------------------------------- whole models
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    base = tmp_path_factory.mktemp("nafezen")
+    return {name: make_model_dir(base, name) for name in TINY}
+
+
+def requests_for(cfg, lengths, seed):
+    return {f"r{i}": random_tokens(n, cfg["vocab"], seed + i) for i, n in enumerate(lengths)}
+
+
+def engine_for(folder, name, dtype, tokens, slots=4, **kw):
+    return Engine.from_folder(folder, dtype=dtype, page_size=TINY[name][1], max_tokens=tokens, max_slots=slots, **kw)
+
+
+def references(cfg, weights, reqs):
+    return {rid: plain.forward(cfg, weights, toks) for rid, toks in reqs.items()}
+
+
+OWN_MARGIN, EARLIER_MARGIN = 0.08, 0.04
+
+
+def close_calls(cfg, weights, reqs):
+    """{request: bool [T]}: rows that bfloat16 is not held to, because a router's choice there, or at an earlier row
+    of the request that this one attends to or carries in its state, was a close call in the plain implementation (the
+    last chosen and the first unchosen logit less than a twelfth of the logits' root mean square apart, a twenty-fifth at
+    an earlier row).  Rounding moves the hidden state by about a hundredth, which decides such a call the other way, and
+    another expert is another function.  float32 is held to every row."""
+    out = {}
+    for rid, toks in reqs.items():
+        plain.route_margins.clear()
+        plain.forward(cfg, weights, toks)
+        own = torch.stack(plain.route_margins).min(0).values
+        earlier = torch.cat([torch.full((1,), float("inf"), dtype=own.dtype), torch.cummin(own, 0).values[:-1]])
+        out[rid] = (own < OWN_MARGIN) | (earlier < EARLIER_MARGIN)
+    return out
+
+
+MODEL_TOL = {"float32": 5e-5, "bfloat16": 3e-2}
+UNIT = {"float32": 2.0 ** -24, "bfloat16": 2.0 ** -9}     # half a unit in the last place
+
+
+def row_limits(cfg, weights, reqs, ref, dtype, floor=None):
+    """What rounding may do to each row: the norm on a retention's read-out magnifies the rounding of what lies in front
+    where terms nearly cancel, most at a request's first rows.  A row's limit is eight times what the plain logits of
+    that row change by when every matrix entry, or every entry of every matrix product, moves by up to half a unit in
+    the last place of the type, and no less than the usual tolerance."""
+    limits = {rid: torch.full((len(toks),), floor or MODEL_TOL[dtype], dtype=torch.float64) for rid, toks in reqs.items()}
+    jitter = lambda t, g: t * (1 + (torch.rand(t.shape, generator=g, dtype=torch.float64) - 0.5) * 2.0 * UNIT[dtype])
+    for trial in range(3):
+        g = torch.Generator().manual_seed(1000 + trial)
+        moved = weights
+        if trial == 0:
+            moved = {k: (jitter(v.double(), g) if v.dim() == 2 else v) for k, v in weights.items()}
+        else:
+            plain.after_product = lambda y: jitter(y, g)
+        try:
+            for rid, toks in reqs.items():
+                err = (plain.forward(cfg, moved, toks) - ref[rid]).abs().max(1).values / ref[rid].abs().max()
+                limits[rid] = torch.maximum(limits[rid], 8.0 * err)
+        finally:
+            plain.after_product = None
+    return limits
+
+
+def check(got, ref, limits, dtype, what, floor=None, exempt=None):
+    """Every row within its limit, and the median row within the usual tolerance.  exempt {request: bool [T]}: rows
+    that only have to be finite (bfloat16 behind a router's close call)."""
+    errors = []
+    for rid, want in ref.items():
+        scale = float(want.abs().max())
+        for p in range(want.shape[0]):
+            row = got[(rid, p)].double()
+            assert torch.isfinite(row).all(), f"{what}: non-finite logits at {rid}:{p}"
+            err = float((row - want[p]).abs().max()) / scale
+            if exempt is not None and dtype == "bfloat16" and bool(exempt[rid][p]):
+                continue
+            errors.append(err)
+            assert err <= float(limits[rid][p]), f"{what}: row {rid}:{p} is off by {err:.3e}, its limit is {float(limits[rid][p]):.3e}"
+    assert sorted(errors)[len(errors) // 2] <= (floor or MODEL_TOL[dtype]), f"{what}: the median row is off by more than the tolerance"
+
+
+CASES = [(name, dtype) for name in TINY for dtype in ("float32", "bfloat16")]
+
+
+@pytest.mark.parametrize("name,dtype", CASES)
+def test_whole_prompts_decoding_and_portions_equal_the_plain_logits(folders, name, dtype):
+    cfg, weights = read_folder(folders[name])
+    reqs = requests_for(cfg, (1, 2, 23, 61, 130), 100)
+    ref = references(cfg, weights, reqs)
+    eng = engine_for(folders[name], name, dtype, 160)
+    limits = row_limits(cfg, weights, reqs, ref, dtype)
+    exempt = close_calls(cfg, weights, reqs)
+    assert sum(int((~e).sum()) for e in exempt.values()) >= 20, "too few rows are left for bfloat16 to be held to"
+    for how, make in (("whole", replay.whole), ("decode", lambda r, t: replay.prefill_then_decode(r, t, tail=80)),
+                      ("portions", replay.portions), ("pairs", lambda r, t: replay.portions(r, t, sizes=(2,))),
+                      ("chunk borders", lambda r, t: replay.portions(r, t, sizes=(63, 2, 64))),
+                      ("single tokens", lambda r, t: replay.portions(r, t, sizes=(1,)))):
+        got = {}
+        for rid, toks in reqs.items():
+            got.update(replay.run_steps(eng, make(rid, toks)))
+        check(got, ref, limits, dtype, f"nafezen {name} {dtype} {how}", exempt=exempt)
+        assert eng.cache.free_tokens() == eng.cache.pool_tokens()
+
+
+@pytest.mark.parametrize("name,dtype", CASES)
+def test_mixed_batches_with_pages_and_slots_used_again(folders, name, dtype):
+    cfg, weights = read_folder(folders[name])
+    reqs = requests_for(cfg, (40, 7, 75, 2, 33, 58, 19, 90), 210)
+    ref = references(cfg, weights, reqs)
+    # three slots and a pool that just holds the three longest live requests: every slot and page is used again
+    eng = engine_for(folders[name], name, dtype, 90 + 75 + 58 + 3 * TINY[name][1], slots=3)
+    alone = engine_for(folders[name], name, dtype, 128, slots=1)
+    limits = row_limits(cfg, weights, reqs, ref, dtype)
+    exempt = close_calls(cfg, weights, reqs)
+    for seed, portion in ((1, 17), (2, 40)):
+        steps = replay.mixed(reqs, max_live=3, seed=seed, decode_tail=12, max_portion=portion)
+        got = replay.run_steps(eng, steps)
+        check(got, ref, limits, dtype, f"nafezen {name} {dtype} mixed {seed}", exempt=exempt)
+        assert eng.cache.free_slot_count == 3 and eng.cache.free_tokens() == eng.cache.pool_tokens()
+    if dtype == "float32":      # in 32 bits a row is the same bits in a batch and alone
+        for rid in ("r0", "r3", "r5"):
+            solo = replay.run_steps(alone, replay.whole(rid, reqs[rid]))
+            for key, row in solo.items():
+                assert torch.equal(row, got[key]), f"{key} differs between the batch and the request alone"
+
+
+def test_a_long_prompt_and_long_decoding_stay_with_the_plain_logits(folders):
+    # (R chooses every expert, so bfloat16 has no close calls there)
+    for name, dtype in (("P", "float32"), ("R", "float32"), ("R", "bfloat16")):
+        cfg, weights = read_folder(folders[name])
+        toks = random_tokens(700, cfg["vocab"], 31)
+        ref = {"a": plain.forward(cfg, weights, toks)}
+        eng = engine_for(folders[name], name, dtype, 720)
+        got = replay.run_steps(eng, replay.prefill_then_decode("a", toks, tail=300))
+        floor = 1e-4 if dtype == "float32" else None      # a thousand steps of a 32-bit recurrence
+        check(got, ref, row_limits(cfg, weights, {"a": toks}, ref, dtype, floor), dtype, f"long {name} {dtype}", floor,
+              exempt=close_calls(cfg, weights, {"a": toks}))
+
+
+@pytest.mark.parametrize("name", ["P", "R"])
+def test_captured_steps_give_the_bits_of_eager_ones(folders, name):
+    cfg, _ = read_folder(folders[name])
+    reqs = requests_for(cfg, (54, 54, 71), 300)
+    steps = []
+    for rid, toks in reqs.items():      # equal portions, then decoding: shapes repeat and are captured
+        steps += [{"entries": [(rid, toks[i:i + 24], list(range(len(toks[i:i + 24]))))], "end": []} for i in range(0, 48, 24)]
+    live = list(reqs)
+    for i in range(48, 54):
+        steps.append({"entries": [(rid, reqs[rid][i:i + 1], [0]) for rid in live], "end": live if i == 53 else []})
+    out = {}
+    for graphs in (False, True):
+        eng = engine_for(folders[name], name, "bfloat16", 240, cuda_graph=graphs)
+        out[graphs] = replay.run_steps(eng, steps)
+        assert (eng.graph_replays > 0) == graphs
+    assert all(torch.equal(out[True][k], out[False][k]) for k in out[False])
+
+
+def _plain_greedy(cfg, weights, prompt, n):
+    toks = list(prompt)
+    for _ in range(n):
+        toks.append(int(plain.forward(cfg, weights, toks)[-1].argmax()))
+    return toks[len(prompt):]
+
+
+@pytest.mark.parametrize("name", ["P", "Q"])
+def test_greedy_generation_through_the_scheduler_equals_the_plain_implementation(folders, name):
+    cfg, weights = read_folder(folders[name])
+    prompts = [random_tokens(n, cfg["vocab"], 400 + n) for n in (3, 12, 29, 18, 7)]
+    want = [_plain_greedy(cfg, weights, p, 24) for p in prompts]
+    # two slots for five requests, portions of at most eight tokens: slots and pages are used again
+    llm = LLM(folders[name], dtype="float32", page_size=TINY[name][1], kv_cache_tokens=160, max_seq_len=64, num_slots=2,
+              chunked_prefill_size=8)
+    outs = llm.generate(prompts, max_tokens=24)
+    assert [o.response_token_ids for o in outs] == want
+    assert all(o.finish_reason == "length" for o in outs)
