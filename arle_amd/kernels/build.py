@@ -46,6 +46,7 @@ SOURCES = {
     "rotary_store": "rotary_store.hip",
     "gated_delta": "gated_delta.hip",
     "group_norm": "group_norm.hip",
+    "latent_attention": "latent_attention.hip",
     "retention": "retention.hip",
     "host": "host/runtime.cpp",
 }

@@ -86,6 +86,8 @@ SIGNATURES = {
     "arle_retention_chunks": ("retention", [_p, _ll, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _p, _f, _p, _i, _i, _i, _i, _p]),
     "arle_latent_prep": ("latent", [_p, _ll, _p, _ll, _p, _ll, _i, _p, _i, _f, _p, _p, _i, _p, _p, _p, _i, _p, _p, _i, _i,
                                     _i, _i, _i, _i, _i, _p]),
+    "arle_latent_attn": ("latent_attention", [_p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _p, _i, _i, _i, _p, _p,
+                                              _p]),
     "arle_head_proj": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _i, _p]),
     "arle_head_proj_mfma": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _p]),
     "arle_moe_route": ("moe", [_p, _ll, _i, _p, _i, _p, _i, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p]),

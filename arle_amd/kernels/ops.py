@@ -1943,6 +1943,54 @@ def latent_prep(q, dkv, q_full, *, heads: int, dim: int, rot_dim: int, rank: int
              int(page_size), 1 if halves else 0, _stream())
 
 
+LATENT_ATTN_MAX_RANK = 256
+LATENT_ATTN_MAX_ROT = 64
+_LATENT_ATTN_ROWS = 128            # rows (token, head) of a workgroup on portions
+_LATENT_ATTN_WORKGROUPS = 512      # workgroups wanted for decoded rows
+_LATENT_ATTN_MAX_SPLITS = 32
+
+
+def latent_attn_supported(dtype, rank: int, rot_dim: int, page_size: int) -> bool:
+    """Whether the matrix-core attention over latents takes this shape."""
+    return (dtype == torch.bfloat16 and 0 < rank <= LATENT_ATTN_MAX_RANK and rank % 32 == 0 and rot_dim % 16 == 0
+            and 0 <= rot_dim <= LATENT_ATTN_MAX_ROT and page_size >= 16 and page_size & (page_size - 1) == 0)
+
+
+def latent_attn(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, seg_start, *, max_qlen: int, heads: int, rank: int,
+                rot_dim: int, page_size: int, scale: float, window: int = 0, sink=None):
+    """Attention of `heads` query heads over one key/value head with keys [c | k_rot] and values c (see
+    csrc/latent_attention.hip): q bfloat16 [T, heads * (rank + rot_dim)], out [T, heads * rank], both contiguous; pages as
+    `latent_prep` writes them.  window > 0: a row sees its last so many keys; sink [heads]: a term exp(sink_h) in the
+    softmax's denominator."""
+    _gpu(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, seg_start, sink)
+    tokens, D = q.shape[0], rank + rot_dim
+    _need(latent_attn_supported(q.dtype, rank, rot_dim, page_size), "shape outside the latent attention's")
+    _need(q.shape == (tokens, heads * D) and q.is_contiguous() and q.data_ptr() % 16 == 0, "q must be contiguous [T, heads * (rank + rot)]")
+    _need(out.shape == (tokens, heads * rank) and out.is_contiguous() and out.dtype == q.dtype and out.data_ptr() % 16 == 0,
+          "out must be contiguous [T, heads * rank] of q's type")
+    _need(0 < heads <= _GRID_Y_MAX and window >= 0 and tokens * heads < 2 ** 31, "head count or window out of range")
+    _check_kv_pages(k_pages, v_pages, 1, page_size, D, rank, q.dtype)
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous(),
+          "block_table must be contiguous int32 [slots, pages]")
+    if sink is not None:
+        _need(sink.shape == (heads,) and sink.is_contiguous() and sink.dtype in _CODES, "sink must be [heads]")
+    segments = seg_slot.numel()
+    _i32(seg_slot, "seg_slot")
+    _i32(seg_start, "seg_start", segments)
+    _i32(seg_row0, "seg_row0", segments + 1)
+    splits, items, part_o, part_ml = 0, tokens * heads // _LATENT_ATTN_ROWS + segments, None, None
+    if max_qlen == 1 and segments == tokens:
+        splits = max(1, min(_LATENT_ATTN_MAX_SPLITS, _LATENT_ATTN_WORKGROUPS // (segments * ((heads + 31) // 32))))
+        if splits > 1:
+            part_o = torch.empty((segments, splits, heads, rank), dtype=torch.float32, device=q.device)
+            part_ml = torch.empty((segments, splits, heads, 2), dtype=torch.float32, device=q.device)
+    lib.call("arle_latent_attn", q.data_ptr(), out.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(),
+             block_table.shape[1], seg_row0.data_ptr(), seg_slot.data_ptr(), seg_start.data_ptr(), segments, heads, D, rank,
+             int(page_size), float(scale), int(window), _ptr(sink), _code(sink) if sink is not None else 0, items, splits,
+             _ptr(part_o), _ptr(part_ml), _stream())
+    return out
+
+
 def head_proj(x, wt, out, *, heads: int, in_head: int, out_head: int):
     """out[t, h * out_head + n] = sum_k x[t, h * in_head + k] wt[h, k, n] for wt [heads, K, N]: a matrix of its own
     for every head, one fixed-order chain over k an output."""

@@ -139,8 +139,13 @@ class LatentAttention(Part):
                         page_size=cache.page_size, halves=self.position.kind != "rope_interleaved")
         self._per_head(q, "uk", q_full, in_head=D + R, out_head=C + R)
         latent = torch.empty((x.shape[0], H * C), dtype=x.dtype, device=x.device)
-        softcap_attention(q_full, latent, cache, batch, num_q_heads=H, num_kv_heads=1, key_dim=C + R, value_dim=C,
-                          scale=self.scale, softcap=0.0, r1=None, r2=None, window=self.window, sink=self.sink)
+        if ops.latent_attn_supported(x.dtype, C, R, cache.page_size):
+            ops.latent_attn(q_full, latent, cache.pages["k"], cache.pages["v"], cache.block_table, batch.seg_row0,
+                            batch.seg_slot, batch.seg_start, max_qlen=batch.max_qlen, heads=H, rank=C, rot_dim=R,
+                            page_size=cache.page_size, scale=self.scale, window=self.window, sink=self.sink)
+        else:
+            softcap_attention(q_full, latent, cache, batch, num_q_heads=H, num_kv_heads=1, key_dim=C + R, value_dim=C,
+                              scale=self.scale, softcap=0.0, r1=None, r2=None, window=self.window, sink=self.sink)
         heads_out = torch.empty((x.shape[0], H * Dv), dtype=x.dtype, device=x.device)
         self._per_head(latent, "uv", heads_out, in_head=C, out_head=Dv)
         if self.gated:

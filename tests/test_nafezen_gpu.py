@@ -250,6 +250,70 @@ def test_a_far_latent_is_found(dtype):
                   tol=4e-2 if dtype == BF16 else None)
 
 
+LATENT_OPS = [
+    # (heads, latent, rotated, page, window, sink, segments: (rows now, position of the first))
+    (32, 192, 64, 64, 0, False, [(300, 0), (1, 700), (5, 63)]),
+    (6, 128, 32, 16, 0, False, [(97, 0), (64, 64), (2, 31), (1, 0)]),
+    (40, 64, 16, 16, 0, True, [(33, 500), (1, 15), (1, 16), (17, 0)]),
+    (1, 32, 0, 32, 0, False, [(400, 100), (1, 1)]),
+    (5, 256, 64, 16, 45, True, [(150, 0), (3, 200), (1, 300), (40, 44)]),
+    (16, 96, 32, 128, 130, False, [(140, 129), (1, 128), (64, 0)]),
+    (33, 160, 48, 16, 1, True, [(20, 0), (1, 77)]),
+    (3, 224, 32, 64, 0, True, [(130, 62), (2, 0)]),
+]
+
+
+@pytest.mark.parametrize("single", [False, True])
+@pytest.mark.parametrize("case", range(len(LATENT_OPS)))
+def test_the_attention_over_latents_equals_float64(case, single):
+    """Segments of several requests on pages in a shuffled order; slots behind the last key hold NaN, and pages a window
+    has passed are gone (their entries in the table name no page)."""
+    H, C, R, page, window, has_sink, segments = LATENT_OPS[case]
+    if single:      # decoded rows, each at its request's end; also one with a single key and one at a tile's border
+        segments = [(1, start + n - 1) for n, start in segments] + [(1, 0), (1, 32), (1, 31)]
+    D, S = C + R, len(segments)
+    T = sum(n for n, _ in segments)
+    g = torch.Generator().manual_seed(case)
+    most = max(n + start for n, start in segments)
+    per = -(-most // page)
+    order = torch.randperm(S * per + 2, generator=g).to(torch.int32)
+    table = torch.full((S, per), -1, dtype=torch.int32)
+    k_pages = torch.full((S * per + 2, 1, page, D), float("nan"))
+    v_pages = torch.full((S * per + 2, 1, C, page), float("nan"))
+    q = rnd((T, H, D), 3 + case)
+    q[:, :, 0] += 2.0
+    sink = rnd((H,), 5) if has_sink else None
+    want = torch.zeros(T, H, C, dtype=torch.float64)
+    row0, at, scale = [0], 0, 3.0 / D ** 0.5
+    for s, (n, start) in enumerate(segments):
+        keys = rnd((start + n, D), 100 + 10 * case + s)
+        keys[torch.randint(0, start + n, (3,), generator=g), 0] += 3.0      # keys that stand out
+        first = max(0, start - window + 1) if window else 0
+        for p in range(first // page, -(-(start + n) // page)):
+            pid = int(order[s * per + p])
+            table[s, p] = pid
+            part = keys[p * page:(p + 1) * page]
+            k_pages[pid, 0, :part.shape[0]] = part
+            v_pages[pid, 0, :, :part.shape[0]] = part[:, :C].T
+        for t in range(n):
+            pos = start + t
+            lo = max(0, pos - window + 1) if window else 0
+            seen = keys[lo:pos + 1].double()
+            z = (q[at + t].double() @ seen.T) * scale
+            if has_sink:
+                z = torch.cat([z, sink.double()[:, None]], dim=1)
+            p = torch.softmax(z, dim=1)[:, :seen.shape[0]]
+            want[at + t] = p @ seen[:, :C]
+        at += n
+        row0.append(at)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=DEV)
+    out = torch.full((T, H * C), float("nan"), dtype=BF16, device=DEV)
+    ops.latent_attn(q.reshape(T, H * D).to(DEV, BF16), out, k_pages.to(DEV, BF16), v_pages.to(DEV, BF16), table.to(DEV), i32(row0),
+                    i32(list(range(S))), i32([start for _, start in segments]), max_qlen=max(n for n, _ in segments), heads=H,
+                    rank=C, rot_dim=R, page_size=page, scale=scale, window=window, sink=sink.to(DEV) if has_sink else None)
+    close(out.view(T, H, C), want, BF16, "attention over latents", tol=1.2e-2)
+
+
 # ----------------------------------------------------------------------------------- retention
 
 RETENTIONS = [
