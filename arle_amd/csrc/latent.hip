@@ -10,6 +10,9 @@
 // the key pages and of c (d-major) into the value pages.  The rotation pairs entry 2i with 2i + 1 over the first
 // `rot` entries (or, with `halves`, entry i with i + rot / 2), by a table of cos and sin per position; entries past
 // `rot` pass unchanged.
+// `latent_down`: the same for the keys' side where the queries go through a latent of their own, from the sums of the one
+// product that makes both latents (its partial products added in order): RMS norm of the queries' latent, and norm,
+// rotation and page write of the keys'.
 // `head_proj`: out[t, h, :] = in[t, h, :] . Wt[h] for a matrix of its own per head, Wt[h] stored [K, N]; the sum over
 // k is one chain of fused multiply-adds in ascending k for every output, whatever else the launch holds.
 // Norm, angles and sums are 32-bit.
@@ -40,7 +43,7 @@ __global__ __launch_bounds__(kLatentThreads) void latent_prep_kernel(
     const float v = to_float(x[i]), other = to_float(x[partner]), c = cs[pair], sv = sn[pair];
     return second ? fmaf(v, c, other * sv) : fmaf(v, c, -other * sv);
   };
-  if (blockIdx.y == 0) {
+  if (dkv && blockIdx.y == 0) {
     const T* row = dkv + t * dkv_stride;
     float ss = 0.f;
     for (int i = threadIdx.x; i < C; i += kLatentThreads) {
@@ -62,11 +65,63 @@ __global__ __launch_bounds__(kLatentThreads) void latent_prep_kernel(
     }
     return;
   }
-  const int h = blockIdx.y - 1;
+  const int h = blockIdx.y - (dkv ? 1 : 0);
   const T* src = q + t * q_stride + static_cast<int64_t>(h) * (D + R) + D;
   T* dst = q_full + t * qf_stride + static_cast<int64_t>(h) * (C + R) + C;
   for (int i = threadIdx.x; i < R; i += kLatentThreads) {
     dst[i] = from_float<T>(i < rot ? turned(src, i) : to_float(src[i]));
+  }
+}
+
+// y: `parts` partial sums part_stride apart, rows row_stride apart, columns [Cq | C | R].  grid (tokens, 2): the keys' side,
+// the queries'.
+template <typename TIn, typename T>
+__global__ __launch_bounds__(kLatentThreads) void latent_down_kernel(
+    const TIn* __restrict__ y, int parts, long long part_stride, long long row_stride, T* __restrict__ cq, int Cq,
+    const void* __restrict__ q_weight, const void* __restrict__ c_weight, int w_dtype, float eps,
+    const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, const int* __restrict__ positions,
+    const int* __restrict__ slot_of_token, const int* __restrict__ block_table, int table_stride,
+    T* __restrict__ k_pages, T* __restrict__ v_pages, int R, int C, int page_size, int halves) {
+  extern __shared__ float row[];   // the sums: [C + R] or [Cq]
+  __shared__ float lds[kLatentThreads / kWave];
+  const int64_t t = blockIdx.x;
+  const bool queries = blockIdx.y == 1;
+  const int normed = queries ? Cq : C, width = queries ? Cq : C + R;
+  const TIn* src = y + t * row_stride + (queries ? 0 : Cq);
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < width; i += kLatentThreads) {
+    float v = to_float(src[i]);
+    for (int p = 1; p < parts; ++p) v += to_float(src[p * part_stride + i]);
+    row[i] = v;
+    if (i < normed) ss = fmaf(v, v, ss);
+  }
+  const float inv = 1.0f / sqrtf(block_sum<kLatentThreads / kWave>(ss, lds) / static_cast<float>(normed) + eps);   // (and a barrier)
+  if (queries) {
+    for (int i = threadIdx.x; i < Cq; i += kLatentThreads) cq[t * Cq + i] = from_float<T>(row[i] * inv * load_as_float(q_weight, w_dtype, i));
+    return;
+  }
+  const int pos = positions[t], half = rot / 2;
+  const int64_t page = block_table[static_cast<int64_t>(slot_of_token[t]) * table_stride + pos / page_size];
+  const int in_page = pos % page_size;
+  T* krow = k_pages + (page * page_size + in_page) * (C + R);
+  T* vcol = v_pages + page * C * page_size + in_page;
+  for (int i = threadIdx.x; i < C; i += kLatentThreads) {
+    const T c = from_float<T>(row[i] * inv * load_as_float(c_weight, w_dtype, i));
+    krow[i] = c;
+    vcol[static_cast<int64_t>(i) * page_size] = c;
+  }
+  const float* cs = cos_t + static_cast<int64_t>(pos) * half;
+  const float* sn = sin_t + static_cast<int64_t>(pos) * half;
+  for (int i = threadIdx.x; i < R; i += kLatentThreads) {
+    float v = row[C + i];
+    if (i < rot) {
+      const int partner = halves ? (i < half ? i + half : i - half) : (i ^ 1);
+      const int pair = halves ? (i < half ? i : i - half) : i / 2;
+      const bool second = halves ? i >= half : (i & 1);
+      const float other = row[C + partner];
+      v = second ? fmaf(v, cs[pair], other * sn[pair]) : fmaf(v, cs[pair], -other * sn[pair]);
+    }
+    krow[C + i] = from_float<T>(v);
   }
 }
 
@@ -113,9 +168,38 @@ typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
 typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
 
+// What rides along: the rotation of the R entries behind a head's K inputs into the R entries behind its N outputs (rotate
+// half or interleaved pairs over the first `rot`), by the workgroups of one more column tile.
+struct TurnAlong {
+  const float* cos_t;
+  const float* sin_t;
+  const int* positions;   // null: nothing rides along
+  int R, rot, halves;
+};
+
 __global__ __launch_bounds__(256) void head_proj_mfma_kernel(const bf16* __restrict__ in, long long in_stride, int in_head,
                                                              const bf16* __restrict__ wnk, bf16* __restrict__ out,
-                                                             long long out_stride, int out_head, int rows, int K, int N) {
+                                                             long long out_stride, int out_head, int rows, int K, int N,
+                                                             const TurnAlong turn) {
+  if (turn.positions && blockIdx.z == gridDim.z - 1) {
+    const int half = turn.rot / 2;
+    for (int i = threadIdx.x; i < 64 * turn.R; i += 256) {
+      const int r = blockIdx.x * 64 + i / turn.R, e = i % turn.R;
+      if (r >= rows) break;
+      const bf16* src = in + static_cast<int64_t>(r) * in_stride + static_cast<int64_t>(blockIdx.y) * in_head + K;
+      float v = to_float(src[e]);
+      if (e < turn.rot) {
+        const int partner = turn.halves ? (e < half ? e + half : e - half) : (e ^ 1);
+        const int pair = turn.halves ? (e < half ? e : e - half) : e / 2;
+        const bool second = turn.halves ? e >= half : (e & 1);
+        const int64_t at = static_cast<int64_t>(turn.positions[r]) * half + pair;
+        const float other = to_float(src[partner]), c = turn.cos_t[at], sv = turn.sin_t[at];
+        v = second ? fmaf(v, c, other * sv) : fmaf(v, c, -other * sv);
+      }
+      out[static_cast<int64_t>(r) * out_stride + static_cast<int64_t>(blockIdx.y) * out_head + N + e] = from_float<bf16>(v);
+    }
+    return;
+  }
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, n = lane % 16, g = lane / 16;
   const int h = blockIdx.y, n0 = blockIdx.z * 64;
   const int row0 = blockIdx.x * 64 + wave * 16;
@@ -159,22 +243,27 @@ __global__ __launch_bounds__(256) void head_proj_mfma_kernel(const bf16* __restr
 
 using namespace arle;
 
-// bfloat16; wnk [heads, N, K].
+// bfloat16; wnk [heads, N, K].  positions (or null): the R entries behind a head's K inputs are turned into those behind
+// its N outputs (see TurnAlong).
 extern "C" int arle_head_proj_mfma(const void* in, long long in_stride, int in_head, const void* wnk, void* out,
-                                   long long out_stride, int out_head, int rows, int heads, int K, int N, void* stream) {
+                                   long long out_stride, int out_head, int rows, int heads, int K, int N,
+                                   const float* cos_t, const float* sin_t, const int* positions, int R, int rot, int halves,
+                                   void* stream) {
   if (rows == 0) return 0;
+  if (positions && (R < 1 || rot < 0 || rot > R || rot % 2 || (rot && (!cos_t || !sin_t)))) return static_cast<int>(hipErrorInvalidValue);
   if (heads < 1 || heads > 65535 || K < 8 || K % 8 || in_head % 8 || in_stride % 8 || N < 1 || (N + 63) / 64 > 65535 ||
       reinterpret_cast<uintptr_t>(in) % 16 || reinterpret_cast<uintptr_t>(wnk) % 16)
     return static_cast<int>(hipErrorInvalidValue);
-  const dim3 grid((rows + 63) / 64, heads, (N + 63) / 64);
+  const dim3 grid((rows + 63) / 64, heads, (N + 63) / 64 + (positions ? 1 : 0));
   head_proj_mfma_kernel<<<grid, 256, 0, static_cast<hipStream_t>(stream)>>>(
       static_cast<const bf16*>(in), in_stride, in_head, static_cast<const bf16*>(wnk), static_cast<bf16*>(out), out_stride,
-      out_head, rows, K, N);
+      out_head, rows, K, N, TurnAlong{cos_t, sin_t, positions, R, rot, halves});
   return launch_status();
 }
 
 // q [T, heads*(D+R)], dkv [T, C+R] and q_full [T, heads*(C+R)] of `dtype`, as the pages: k_pages
-// [pages, 1, page_size, C+R], v_pages [pages, 1, C, page_size].  cos, sin: float32 [positions, rot/2].
+// [pages, 1, page_size, C+R], v_pages [pages, 1, C, page_size].  cos, sin: float32 [positions, rot/2].  dkv null: the
+// queries' side alone.
 extern "C" int arle_latent_prep(const void* q, long long q_stride, const void* dkv, long long dkv_stride, void* q_full,
                                 long long qf_stride, int dtype, const void* c_weight, int w_dtype, float eps,
                                 const float* cos_t, const float* sin_t, int rot, const int* positions,
@@ -185,7 +274,7 @@ extern "C" int arle_latent_prep(const void* q, long long q_stride, const void* d
   if (heads < 1 || heads > 65534 || D < 1 || R < 0 || C < 1 || rot < 0 || rot > R || rot % 2 || page_size < 1 ||
       (rot > 0 && (!cos_t || !sin_t)))
     return static_cast<int>(hipErrorInvalidValue);
-  const dim3 grid(tokens, 1 + heads);
+  const dim3 grid(tokens, (dkv ? 1 : 0) + heads);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == kF32) {
     latent_prep_kernel<float><<<grid, kLatentThreads, 0, s>>>(
@@ -198,6 +287,36 @@ extern "C" int arle_latent_prep(const void* q, long long q_stride, const void* d
         qf_stride, c_weight, w_dtype, eps, cos_t, sin_t, rot, positions, slot_of_token, block_table, table_stride,
         static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), heads, D, R, C, page_size, halves);
   }
+  return launch_status();
+}
+
+// y: float32 or bfloat16 (y_dtype), `parts` partial sums of rows [Cq | C | R | .]; cq [tokens, Cq] and the pages of `dtype`;
+// q_weight [Cq], c_weight [C] of w_dtype.
+extern "C" int arle_latent_down(const void* y, int y_dtype, int parts, long long part_stride, long long row_stride, void* cq,
+                                int Cq, int dtype, const void* q_weight, const void* c_weight, int w_dtype, float eps,
+                                const float* cos_t, const float* sin_t, int rot, const int* positions,
+                                const int* slot_of_token, const int* block_table, int table_stride, void* k_pages,
+                                void* v_pages, int tokens, int R, int C, int page_size, int halves, void* stream) {
+  if (tokens == 0) return 0;
+  const size_t lds = static_cast<size_t>(max(Cq, C + R)) * sizeof(float);
+  if (parts < 1 || Cq < 1 || R < 0 || C < 1 || rot < 0 || rot > R || rot % 2 || page_size < 1 || (rot > 0 && (!cos_t || !sin_t)) ||
+      lds > 48 * 1024)
+    return static_cast<int>(hipErrorInvalidValue);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+#define ARLE_DOWN(TI, TT)                                                                                              \
+  latent_down_kernel<TI, TT><<<dim3(tokens, 2), kLatentThreads, lds, s>>>(                                             \
+      static_cast<const TI*>(y), parts, part_stride, row_stride, static_cast<TT*>(cq), Cq, q_weight, c_weight, w_dtype, \
+      eps, cos_t, sin_t, rot, positions, slot_of_token, block_table, table_stride, static_cast<TT*>(k_pages),          \
+      static_cast<TT*>(v_pages), R, C, page_size, halves)
+  if (dtype == kF32) {
+    if (y_dtype != kF32) return static_cast<int>(hipErrorInvalidValue);
+    ARLE_DOWN(float, float);
+  } else if (y_dtype == kF32) {
+    ARLE_DOWN(float, bf16);
+  } else {
+    ARLE_DOWN(bf16, bf16);
+  }
+#undef ARLE_DOWN
   return launch_status();
 }
 

@@ -89,7 +89,9 @@ SIGNATURES = {
     "arle_latent_attn": ("latent_attention", [_p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _p, _i, _i, _i, _p, _p,
                                               _p]),
     "arle_head_proj": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _i, _p]),
-    "arle_head_proj_mfma": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _p]),
+    "arle_head_proj_mfma": ("latent", [_p, _ll, _i, _p, _p, _ll, _i, _i, _i, _i, _i, _p, _p, _p, _i, _i, _i, _p]),
+    "arle_latent_down": ("latent", [_p, _i, _i, _ll, _ll, _p, _i, _i, _p, _p, _i, _f, _p, _p, _i, _p, _p, _p, _i, _p, _p, _i, _i, _i,
+                                    _i, _i, _p]),
     "arle_moe_route": ("moe", [_p, _ll, _i, _p, _i, _p, _i, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _f, _i, _i, _i, _i, _p]),
     "arle_moe_identity": ("moe", [_p, _ll, _i, _p, _p, _i, _i, _i, _i, _p]),
     "arle_moe_expert": ("moe", [_p, _ll, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),

@@ -1912,35 +1912,72 @@ def tanh_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
 HEAD_PROJ_MAX_K = 1024
 
 
+def _check_latent_tables(cos, sin, rotary_dims: int, rot_dim: int) -> None:
+    _need(0 <= rotary_dims <= rot_dim and rotary_dims % 2 == 0, "rotary dims must be even and within the rotated part")
+    if rotary_dims:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _need(t.dtype == torch.float32 and t.dim() == 2 and t.shape[1] == rotary_dims // 2 and t.is_contiguous(),
+                  f"{name} must be contiguous float32 [positions, rotary_dims / 2]")
+
+
 def latent_prep(q, dkv, q_full, *, heads: int, dim: int, rot_dim: int, rank: int, c_weight, eps: float, cos, sin,
                 rotary_dims: int, positions, slot_of_token, block_table, k_pages, v_pages, page_size: int,
                 halves: bool = False):
     """dkv [T, rank + rot_dim]: the first `rank` entries RMS-normed (c), the rest rotated (interleaved pairs over the
     first `rotary_dims`, or with `halves` entry i with i + rotary_dims / 2), [c | k_rot] to the key pages and c to the value pages; the rotated part of every head of
     q [T, heads * (dim + rot_dim)] goes, rotated, to the last rot_dim entries of its head in
-    q_full [T, heads * (rank + rot_dim)]."""
+    q_full [T, heads * (rank + rot_dim)].  dkv None: only the queries' side (`latent_down` has done the keys')."""
     _gpu(q, dkv, q_full, c_weight, cos, sin, positions, slot_of_token, block_table, k_pages, v_pages)
     tokens = q.shape[0]
     for name, t, width in (("q", q, heads * (dim + rot_dim)), ("dkv", dkv, rank + rot_dim),
                            ("q_full", q_full, heads * (rank + rot_dim))):
+        if t is None:
+            continue
         _rows(t, name)
         _need(t.shape == (tokens, width) and t.dtype == q.dtype and t.dtype in _CODES, f"{name} must be [T, {width}]")
     _need(c_weight.shape == (rank,) and c_weight.is_contiguous() and c_weight.dtype in _CODES, "the latent's norm weight must be [rank]")
-    _need(0 <= rotary_dims <= rot_dim and rotary_dims % 2 == 0, "rotary dims must be even and within the rotated part")
-    if rotary_dims:
-        for name, t in (("cos", cos), ("sin", sin)):
-            _need(t.dtype == torch.float32 and t.dim() == 2 and t.shape[1] == rotary_dims // 2 and t.is_contiguous(),
-                  f"{name} must be contiguous float32 [positions, rotary_dims / 2]")
+    _check_latent_tables(cos, sin, rotary_dims, rot_dim)
     _check_kv_pages(k_pages, v_pages, 1, page_size, rank + rot_dim, rank, q.dtype)
     _i32(positions, "positions", tokens)
     _i32(slot_of_token, "slot_of_token", tokens)
     _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous(),
           "block_table must be contiguous int32 [slots, pages]")
-    lib.call("arle_latent_prep", q.data_ptr(), q.stride(0), dkv.data_ptr(), dkv.stride(0), q_full.data_ptr(),
-             q_full.stride(0), _code(q), c_weight.data_ptr(), _code(c_weight), float(eps), _ptr(cos), _ptr(sin),
+    lib.call("arle_latent_prep", q.data_ptr(), q.stride(0), _ptr(dkv), dkv.stride(0) if dkv is not None else 0,
+             q_full.data_ptr(), q_full.stride(0), _code(q), c_weight.data_ptr(), _code(c_weight), float(eps), _ptr(cos), _ptr(sin),
              int(rotary_dims), positions.data_ptr(), slot_of_token.data_ptr(), block_table.data_ptr(),
              block_table.shape[1], k_pages.data_ptr(), v_pages.data_ptr(), tokens, heads, dim, rot_dim, rank,
              int(page_size), 1 if halves else 0, _stream())
+
+
+LATENT_DOWN_MAX_WIDTH = 12288
+
+
+def latent_down(y, *, q_rank: int, rank: int, rot_dim: int, q_weight, c_weight, eps: float, cos, sin, rotary_dims: int,
+                positions, slot_of_token, block_table, k_pages, v_pages, page_size: int, halves: bool = False):
+    """y [T, q_rank | rank | rot_dim] or a float32 stack [S, T, .] of its partial sums: the first q_rank entries RMS-normed
+    (returned, in the pages' type), the next `rank` RMS-normed (c), the last rotated; [c | k_rot] to the key pages and c to
+    the value pages, as `latent_prep` does."""
+    _gpu(y, q_weight, c_weight, cos, sin, positions, slot_of_token, block_table, k_pages, v_pages)
+    dtype = k_pages.dtype
+    tokens, width = y.shape[-2], y.shape[-1]
+    _need(y.dim() in (2, 3) and width == q_rank + rank + rot_dim and y.is_contiguous() and y.dtype in _CODES
+          and (y.dim() == 2 or y.dtype == torch.float32) and (dtype == torch.bfloat16 or y.dtype == torch.float32),
+          "y must be [T, q_rank + rank + rot_dim], or a float32 stack of partial sums of it")
+    _need(max(q_rank, rank + rot_dim) <= LATENT_DOWN_MAX_WIDTH, f"latents up to {LATENT_DOWN_MAX_WIDTH} entries")
+    _need(q_weight.shape == (q_rank,) and c_weight.shape == (rank,) and q_weight.dtype == c_weight.dtype and q_weight.dtype in _CODES
+          and q_weight.is_contiguous() and c_weight.is_contiguous(), "the latents' norm weights must be [q_rank] and [rank] of one type")
+    _check_latent_tables(cos, sin, rotary_dims, rot_dim)
+    _check_kv_pages(k_pages, v_pages, 1, page_size, rank + rot_dim, rank, dtype)
+    _i32(positions, "positions", tokens)
+    _i32(slot_of_token, "slot_of_token", tokens)
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous(),
+          "block_table must be contiguous int32 [slots, pages]")
+    cq = torch.empty((tokens, q_rank), dtype=dtype, device=y.device)
+    lib.call("arle_latent_down", y.data_ptr(), _code(y), y.shape[0] if y.dim() == 3 else 1, tokens * width, width, cq.data_ptr(),
+             q_rank, _CODES[dtype], q_weight.data_ptr(), c_weight.data_ptr(), _code(q_weight), float(eps), _ptr(cos), _ptr(sin),
+             int(rotary_dims), positions.data_ptr(), slot_of_token.data_ptr(), block_table.data_ptr(), block_table.shape[1],
+             k_pages.data_ptr(), v_pages.data_ptr(), tokens, rot_dim, rank, int(page_size), 1 if halves else 0, _stream())
+    return cq
 
 
 LATENT_ATTN_MAX_RANK = 256
@@ -2014,9 +2051,19 @@ def head_proj_mfma_supported(x, heads: int, in_head: int, K: int) -> bool:
             and x.data_ptr() % 16 == 0)
 
 
-def head_proj_mfma(x, wnk, out, *, heads: int, in_head: int, out_head: int):
-    """`head_proj` on the matrix cores: bfloat16, every head's matrix stored wnk [heads, N, K]."""
+def head_proj_mfma(x, wnk, out, *, heads: int, in_head: int, out_head: int, turn=None):
+    """`head_proj` on the matrix cores: bfloat16, every head's matrix stored wnk [heads, N, K].  turn = (cos, sin, positions,
+    entries, rotary dims, halves): the so many entries behind a head's K inputs go, rotated, behind its N outputs."""
     _gpu(x, wnk, out)
+    riders = (0, 0, 0, 0, 0, 0)
+    if turn is not None:
+        cos, sin, positions, entries, rotary_dims, halves = turn
+        _gpu(cos, sin, positions)
+        _check_latent_tables(cos, sin, rotary_dims, entries)
+        _i32(positions, "positions", x.shape[0])
+        _need(entries > 0 and (heads - 1) * in_head + wnk.shape[2] + entries <= x.shape[1]
+              and (heads - 1) * out_head + wnk.shape[1] + entries <= out.shape[1], "the rotated entries must lie inside the rows")
+        riders = (_ptr(cos), _ptr(sin), positions.data_ptr(), int(entries), int(rotary_dims), 1 if halves else 0)
     _rows(x, "x")
     _rows(out, "out")
     _need(wnk.dim() == 3 and wnk.shape[0] == heads and wnk.is_contiguous(), "wnk must be contiguous [heads, N, K]")
@@ -2026,7 +2073,7 @@ def head_proj_mfma(x, wnk, out, *, heads: int, in_head: int, out_head: int):
     _need(x.shape[0] == out.shape[0] and (heads - 1) * in_head + K <= x.shape[1]
           and (heads - 1) * out_head + N <= out.shape[1], "a head's numbers must lie inside its row")
     lib.call("arle_head_proj_mfma", x.data_ptr(), x.stride(0), int(in_head), wnk.data_ptr(), out.data_ptr(),
-             out.stride(0), int(out_head), x.shape[0], heads, K, N, _stream())
+             out.stride(0), int(out_head), x.shape[0], heads, K, N, *riders, _stream())
     return out
 
 

@@ -31,7 +31,8 @@ from .softcap_attention import softcap_attention
 
 @register("mixer", "latent_attention")
 class LatentAttention(Part):
-    """params: hidden_size, heads, dim, rot_dim, value_dim, rank, q_rank (int | None: the size of the queries' own latent), eps, scale, window (int | None), sink (bool),
+    """params: hidden_size, heads, dim, rot_dim, value_dim, rank, q_rank (int | None: the size of the queries' own
+    latent), eps, scale, window (int | None), sink (bool),
     gate (bool: a sigmoid gate on the heads' outputs, a projection of the mixer's input), position (PartSpec of the
     rotation over the rot_dim part)."""
 
@@ -112,15 +113,19 @@ class LatentAttention(Part):
         return [("q_dkv_g" if self.gated else "q_dkv", self.proj.out_features, self.proj.in_features, False, None), *queries,
                 ("o", self.o.out_features, self.o.in_features, False, "norm")]
 
-    def _per_head(self, x, which, out, *, in_head, out_head):
-        """out[:, head] = x[:, head] . (W_uk,h or W_uv,h^T), a matrix a head."""
+    def _per_head(self, x, which, out, *, in_head, out_head, turn=None):
+        """out[:, head] = x[:, head] . (W_uk,h or W_uv,h^T), a matrix a head.  turn: the rotation that may ride along (see
+        ops.head_proj_mfma); the answer says whether it did."""
         if self.on_matrix_cores and ops.head_proj_mfma_supported(x, self.H, in_head, self.D if which == "uk" else self.C):
-            ops.head_proj_mfma(x, self.uk_nk if which == "uk" else self.uv_nk, out, heads=self.H, in_head=in_head, out_head=out_head)
-        elif self.on_matrix_cores:      # operands that are not aligned for it after all: the plain kernel, from a turned copy
+            ops.head_proj_mfma(x, self.uk_nk if which == "uk" else self.uv_nk, out, heads=self.H, in_head=in_head, out_head=out_head,
+                               turn=turn)
+            return turn is not None
+        if self.on_matrix_cores:      # operands that are not aligned for it after all: the plain kernel, from a turned copy
             w = (self.uk_nk if which == "uk" else self.uv_nk).transpose(1, 2).contiguous()
             ops.head_proj(x, w, out, heads=self.H, in_head=in_head, out_head=out_head)
         else:
             ops.head_proj(x, self.uk if which == "uk" else self.uv_t, out, heads=self.H, in_head=in_head, out_head=out_head)
+        return False
 
     def forward(self, x, batch, cache):
         """x [T, H] -> float32 [T, H], or a float32 stack [S, T, H] to be added in order (see Linear)."""
@@ -129,15 +134,26 @@ class LatentAttention(Part):
         H, D, R, C, Dv = self.H, self.D, self.R, self.C, self.Dv
         self.position.ensure_positions(batch.max_position + 1)
         cos, sin, rot = self.position.fused_rotary()
-        y = self.proj(x)
-        first, dkv = y[:, :self.first_width], y[:, self.first_width:self.first_width + self.dkv_width]
-        q = self.uq(ops.rmsnorm(first, self.q_norm, self.eps, x.dtype)) if self.uq is not None else first
+        halves = self.position.kind != "rope_interleaved"
+        keys = dict(rot_dim=R, rank=C, c_weight=self.c_norm, eps=self.eps, cos=cos, sin=sin, rotary_dims=rot,
+                    positions=batch.positions, slot_of_token=batch.slot_of_token, block_table=cache.block_table,
+                    k_pages=cache.pages["k"], v_pages=cache.pages["v"], page_size=cache.page_size, halves=halves)
         q_full = torch.empty((x.shape[0], H * (C + R)), dtype=x.dtype, device=x.device)
-        ops.latent_prep(q, dkv, q_full, heads=H, dim=D, rot_dim=R, rank=C, c_weight=self.c_norm, eps=self.eps, cos=cos,
-                        sin=sin, rotary_dims=rot, positions=batch.positions, slot_of_token=batch.slot_of_token,
-                        block_table=cache.block_table, k_pages=cache.pages["k"], v_pages=cache.pages["v"],
-                        page_size=cache.page_size, halves=self.position.kind != "rope_interleaved")
-        self._per_head(q, "uk", q_full, in_head=D + R, out_head=C + R)
+        turned = False
+        if self.uq is not None and not self.gated:
+            # few rows: the product's partial sums go on as they are; many: in the activation type, as the library makes them
+            few = x.dtype != torch.bfloat16 or x.shape[0] <= ops.ROWS_KERNEL_MAX
+            y = self.proj(x, out_dtype=torch.float32 if few else None, partials_ok=few)
+            q, dkv = self.uq(ops.latent_down(y, q_rank=self.q_rank, q_weight=self.q_norm, **keys)), None
+            turned = self._per_head(q, "uk", q_full, in_head=D + R, out_head=C + R,
+                                    turn=(cos, sin, batch.positions, R, rot, halves))
+        else:
+            y = self.proj(x)
+            first, dkv = y[:, :self.first_width], y[:, self.first_width:self.first_width + self.dkv_width]
+            q = self.uq(ops.rmsnorm(first, self.q_norm, self.eps, x.dtype)) if self.uq is not None else first
+            self._per_head(q, "uk", q_full, in_head=D + R, out_head=C + R)
+        if not turned:
+            ops.latent_prep(q, dkv, q_full, heads=H, dim=D, **keys)
         latent = torch.empty((x.shape[0], H * C), dtype=x.dtype, device=x.device)
         if ops.latent_attn_supported(x.dtype, C, R, cache.page_size):
             ops.latent_attn(q_full, latent, cache.pages["k"], cache.pages["v"], cache.block_table, batch.seg_row0,

@@ -218,6 +218,35 @@ def test_the_latent_attention_makes_its_queries_through_a_latent_too(dtype, case
                tol=4e-2 if dtype == BF16 else None)
 
 
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("interleaved", [False, True])
+def test_a_latent_for_the_queries_goes_with_a_gate_and_with_interleaved_pairs(dtype, interleaved):
+    """Options of the part that the design does not combine itself."""
+    m = latent(4, 16, 8, 12, 32, 24, scale=0.3, rot=rot(500.0, 6))
+    raw, spec = one_layer("latent_attention", m, width=48)          # as wide as the heads' outputs together
+    mixer = spec.layers[0].mixer
+    for gate in (False, True):
+        params = dict(mixer.params, gate=gate)
+        if interleaved:
+            params["position"] = PartSpec("rope_interleaved", mixer.params["position"].params)
+        part, tensors = random_part("mixer", PartSpec(mixer.kind, params, dict(mixer.weights, g="l0.mix.g")), dtype, 31, 0.25)
+        x = rnd((40, 48), 8)
+        w = lambda name: torch.eye(48, dtype=torch.float64) if name == "o" else tensors["l0.mix." + name].double()
+        before = plain.rotate_half
+        if interleaved:     # the same turn with entry 2i beside 2i + 1: reordered, turned by halves, put back
+            order = torch.tensor([0, 2, 4, 1, 3, 5, 6, 7])
+            plain.rotate_half = lambda v, p, dims, base: before(v[..., order], p, dims, base)[..., order.argsort()]
+        try:
+            want = plain.latent_attention(x.double(), m, w, EPS)
+        finally:
+            plain.rotate_half = before
+        if gate:
+            want = want * torch.sigmoid(x.double() @ tensors["l0.mix.g"].double().T)
+        want = want @ tensors["l0.mix.o"].double().T
+        for cuts in ((1000,), (1,), (7, 2)):
+            close(run_mixer(part, x, cuts, page=16, dtype=dtype), want, dtype, f"gate {gate}, cuts {cuts}", tol=4e-2 if dtype == BF16 else None)
+
+
 def far_key_inputs(tensors, mixer, T, W, target):
     """Inputs in which the latent at `target` lies along what the last row's first head asks for: its score stands out
     among T, and its value decides the last row's output."""
