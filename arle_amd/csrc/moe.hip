@@ -10,12 +10,12 @@
 //   router's kernel also makes the one number a token that a shared expert's output is multiplied by, sigmoid(w_s h),
 //   where the caller has one.
 //
-// `moe_route`: one workgroup a token.  `moe_expert`: a workgroup takes one expert, 64 consecutive rows of the step and 64
-// output columns; it lists the rows of its 64 that chose the expert (in row order) and multiplies only those, so no
-// step sorts anything and a launch's shape follows the number of rows alone.  The result of (token t, its k-th
+// `moe_route`: one or four tokens a workgroup.  `moe_expert`: a workgroup takes one expert, 64 consecutive rows of the step
+// and 64 output columns; it lists the rows of its 64 that chose the expert (in row order) and multiplies only those, so
+// no step sorts anything and a launch's shape follows the number of rows alone.  The result of (token t, its k-th
 // choice) lies at row t * top + k: the gate|up pass leaves the activation there, the down pass the expert's output,
 // which the consumer weighs and adds in the order of k.  Every output is summed in one fixed order over K (chains
-// of 16, added in ascending order), whatever else the step holds.  bfloat16 runs the matrix-core form further down.
+// of 16, added in ascending order), whatever else the step holds.  bfloat16 runs the matrix-core forms further down.
 #include "common.h"
 
 namespace arle {
@@ -26,6 +26,9 @@ struct Best {
   float v;
   int i;
 };
+
+// What the wave's lanes wrote to LDS before this, its lanes read behind it.
+__device__ __forceinline__ void wave_lds_fence() { __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront"); }
 
 __device__ __forceinline__ Best wave_best(Best b) {
 #pragma unroll
@@ -40,11 +43,6 @@ __device__ __forceinline__ Best wave_best(Best b) {
   return b;
 }
 
-constexpr int kRouteThreads = 256;
-
-// One workgroup a token: the row goes to LDS as floats once; wave w computes the logits of experts w, w + 4, ...
-// (eight consecutive entries a lane and step where the width allows, one otherwise: an order that depends on the
-// width alone); then the first wave picks the `top` experts one after the other.
 struct RouteRule {
   int softmax;     // 0: s = sigmoid(z); 1: s = softmax(z); 2: s = z, and the weights are the softmax over the chosen z
   int groups;      // equal groups of neighbouring experts (1: no groups)
@@ -53,128 +51,149 @@ struct RouteRule {
   float scale;
 };
 
-template <typename T, typename TW, bool VEC>
-__global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __restrict__ x, long long x_stride,
-                                                                  const TW* __restrict__ w, const void* __restrict__ bias,
-                                                                  int b_dtype, const void* __restrict__ correction,
-                                                                  int c_dtype, const TW* __restrict__ shared_w,
-                                                                  float* __restrict__ shared_gate, int* __restrict__ ids,
-                                                                  float* __restrict__ weights, int width, int experts,
-                                                                  int top, const RouteRule rule) {
-  extern __shared__ float route_lds[];   // [width] the row, then [experts] the scores, [experts] the choice numbers, [groups]
+// A workgroup takes TOK tokens: their rows go to LDS as floats once; wave w computes the logits of experts w, w + waves,
+// ... for all of them, a router row read once for the TOK (eight consecutive entries a lane and step where the width
+// allows, one otherwise: an order that depends on the width alone); then wave k picks the `top` experts of token k one
+// after the other.  EPL: experts a lane looks after (experts <= 64 * EPL).
+template <typename T, typename TW, bool VEC, int THREADS, int TOK, int EPL>
+__global__ __launch_bounds__(THREADS) void moe_route_kernel(const T* __restrict__ x, long long x_stride,
+                                                            const TW* __restrict__ w, const void* __restrict__ bias,
+                                                            int b_dtype, const void* __restrict__ correction, int c_dtype,
+                                                            const TW* __restrict__ shared_w,
+                                                            float* __restrict__ shared_gate, int* __restrict__ ids,
+                                                            float* __restrict__ weights, int tokens, int width, int experts,
+                                                            int top, const RouteRule rule) {
+  // [TOK][width] the rows, then a token's [experts] scores, [experts] choice numbers and [groups]
+  extern __shared__ float route_lds[];
   float* xs = route_lds;
-  float* score = route_lds + width;
-  float* pick = score + experts;
-  float* group_best = pick + experts;
-  const int64_t t = blockIdx.x;
+  const int per_token = 2 * experts + rule.groups;
+  float* numbers = route_lds + TOK * width;
+  const int64_t t0 = static_cast<int64_t>(blockIdx.x) * TOK;
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
-  const T* row = x + t * x_stride;
-  for (int i = threadIdx.x; i < width; i += kRouteThreads) xs[i] = to_float(row[i]);
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const T* row = x + min(t0 + k, static_cast<int64_t>(tokens) - 1) * x_stride;
+    for (int i = threadIdx.x; i < width; i += THREADS) xs[k * width + i] = to_float(row[i]);
+  }
   __syncthreads();
-  for (int e = wave; e < experts + (shared_w ? 1 : 0); e += kRouteThreads / kWave) {
+  for (int e = wave; e < experts + (shared_w ? 1 : 0); e += THREADS / kWave) {
     const TW* we = e < experts ? w + static_cast<int64_t>(e) * width : shared_w;
-    float dot = 0.f;
+    float dot[TOK];
+#pragma unroll
+    for (int k = 0; k < TOK; ++k) dot[k] = 0.f;
     if (VEC) {
+#pragma unroll 4
       for (int i = 8 * lane; i < width; i += 8 * kWave) {
         const float4 lo = ld4<TW>(we + i), hi = ld4<TW>(we + i + 4);
-        dot = fmaf(xs[i], lo.x, dot); dot = fmaf(xs[i + 1], lo.y, dot); dot = fmaf(xs[i + 2], lo.z, dot); dot = fmaf(xs[i + 3], lo.w, dot);
-        dot = fmaf(xs[i + 4], hi.x, dot); dot = fmaf(xs[i + 5], hi.y, dot); dot = fmaf(xs[i + 6], hi.z, dot); dot = fmaf(xs[i + 7], hi.w, dot);
+#pragma unroll
+        for (int k = 0; k < TOK; ++k) {
+          const float* xk = xs + k * width + i;
+          const float4 a = *reinterpret_cast<const float4*>(xk), b = *reinterpret_cast<const float4*>(xk + 4);
+          dot[k] = fmaf(a.x, lo.x, dot[k]); dot[k] = fmaf(a.y, lo.y, dot[k]); dot[k] = fmaf(a.z, lo.z, dot[k]); dot[k] = fmaf(a.w, lo.w, dot[k]);
+          dot[k] = fmaf(b.x, hi.x, dot[k]); dot[k] = fmaf(b.y, hi.y, dot[k]); dot[k] = fmaf(b.z, hi.z, dot[k]); dot[k] = fmaf(b.w, hi.w, dot[k]);
+        }
       }
     } else {
-      for (int i = lane; i < width; i += kWave) dot = fmaf(xs[i], to_float(we[i]), dot);
+      for (int i = lane; i < width; i += kWave) {
+        const float v = to_float(we[i]);
+#pragma unroll
+        for (int k = 0; k < TOK; ++k) dot[k] = fmaf(xs[k * width + i], v, dot[k]);
+      }
     }
-    dot = wave_sum(dot);
-    if (lane != 0) continue;
-    if (e == experts) {
-      shared_gate[t] = 1.0f / (1.0f + expf(-dot));
-      continue;
+#pragma unroll
+    for (int k = 0; k < TOK; ++k) {
+      float z = wave_sum(dot[k]);
+      if (lane != 0 || t0 + k >= tokens) continue;
+      if (e == experts) {
+        shared_gate[t0 + k] = 1.0f / (1.0f + expf(-z));
+        continue;
+      }
+      if (bias) z += load_as_float(bias, b_dtype, e);
+      numbers[k * per_token + e] = rule.softmax ? z : 1.0f / (1.0f + expf(-z));
     }
-    if (bias) dot += load_as_float(bias, b_dtype, e);
-    score[e] = rule.softmax ? dot : 1.0f / (1.0f + expf(-dot));
   }
   __syncthreads();
-  // From here on the first wave works alone; the others only keep the barriers' count.
-  float s[kMaxExpertsPerLane], choice[kMaxExpertsPerLane];
-  if (wave == 0) {
+  // From here on wave k works for token k; what goes through LDS goes from a wave to itself.
+  if (wave >= TOK || t0 + wave >= tokens) return;
+  const int64_t t = t0 + wave;
+  float* score = numbers + wave * per_token;
+  float* pick = score + experts;
+  float* group_best = pick + experts;
+  float s[EPL], choice[EPL];
 #pragma unroll
-    for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-      const int e = lane + j * kWave;
-      s[j] = e < experts ? score[e] : (rule.softmax ? -INFINITY : 0.f);
-    }
-    if (rule.softmax == 1) {   // over all router outputs, in 32 bits: the largest logit taken off, one sum in a fixed order
-      float top_z = -INFINITY;
-#pragma unroll
-      for (int j = 0; j < kMaxExpertsPerLane; ++j) top_z = fmaxf(top_z, s[j]);
-      top_z = wave_max(top_z);
-      float sum = 0.f;
-#pragma unroll
-      for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-        s[j] = lane + j * kWave < experts ? expf(s[j] - top_z) : 0.f;
-        sum += s[j];
-      }
-      const float inv = 1.0f / wave_sum(sum);
-#pragma unroll
-      for (int j = 0; j < kMaxExpertsPerLane; ++j) s[j] *= inv;
-    }
-#pragma unroll
-    for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-      const int e = lane + j * kWave;
-      choice[j] = e < experts ? s[j] + (correction ? load_as_float(correction, c_dtype, e) : 0.f) : -INFINITY;
-      if (e < experts) pick[e] = choice[j];
-    }
+  for (int j = 0; j < EPL; ++j) {
+    const int e = lane + j * kWave;
+    s[j] = e < experts ? score[e] : (rule.softmax ? -INFINITY : 0.f);
   }
-  if (rule.groups > 1) {   // (the same for every thread of the launch)
-    __syncthreads();
+  if (rule.softmax == 1) {   // over all router outputs, in 32 bits: the largest logit taken off, one sum in a fixed order
+    float top_z = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < EPL; ++j) top_z = fmaxf(top_z, s[j]);
+    top_z = wave_max(top_z);
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < EPL; ++j) {
+      s[j] = lane + j * kWave < experts ? expf(s[j] - top_z) : 0.f;
+      sum += s[j];
+    }
+    const float inv = 1.0f / wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < EPL; ++j) s[j] *= inv;
+  }
+#pragma unroll
+  for (int j = 0; j < EPL; ++j) {
+    const int e = lane + j * kWave;
+    choice[j] = e < experts ? s[j] + (correction ? load_as_float(correction, c_dtype, e) : 0.f) : -INFINITY;
+    if (e < experts) pick[e] = choice[j];
+  }
+  if (rule.groups > 1) {
     const int per = experts / rule.groups;
-    if (wave == 0) {
-      // a group's number is the largest choice number in it; lane l looks after the groups l, l + 64, ...
-      float best[kMaxExpertsPerLane];
+    wave_lds_fence();
+    // a group's number is the largest choice number in it; lane l looks after the groups l, l + 64, ...
+    float best[EPL];
 #pragma unroll
-      for (int j = 0; j < kMaxExpertsPerLane; ++j) {
+    for (int j = 0; j < EPL; ++j) {
+      const int g = lane + j * kWave;
+      float b = -INFINITY;
+      if (g < rule.groups)
+        for (int i = 0; i < per; ++i) b = fmaxf(b, pick[g * per + i]);
+      best[j] = b;
+      if (g < rule.groups) group_best[g] = 0.f;   // 1 once the group is kept
+    }
+    wave_lds_fence();
+    for (int k = 0; k < rule.keep; ++k) {
+      Best b{-INFINITY, 0x7fffffff};
+#pragma unroll
+      for (int j = 0; j < EPL; ++j) {
         const int g = lane + j * kWave;
-        float b = -INFINITY;
-        if (g < rule.groups)
-          for (int i = 0; i < per; ++i) b = fmaxf(b, pick[g * per + i]);
-        best[j] = b;
-        if (g < rule.groups) group_best[g] = 0.f;   // 1 once the group is kept
-      }
-      for (int k = 0; k < rule.keep; ++k) {
-        Best b{-INFINITY, 0x7fffffff};
-#pragma unroll
-        for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-          const int g = lane + j * kWave;
-          if (g < rule.groups && best[j] != INFINITY && (best[j] > b.v || (best[j] == b.v && g < b.i))) {
-            b.v = best[j];
-            b.i = g;
-          }
+        if (g < rule.groups && best[j] != INFINITY && (best[j] > b.v || (best[j] == b.v && g < b.i))) {
+          b.v = best[j];
+          b.i = g;
         }
-        b = wave_best(b);
+      }
+      b = wave_best(b);
 #pragma unroll
-        for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-          if (b.i == lane + j * kWave) {
-            best[j] = INFINITY;   // taken
-            group_best[b.i] = 1.f;
-          }
+      for (int j = 0; j < EPL; ++j) {
+        if (b.i == lane + j * kWave) {
+          best[j] = INFINITY;   // taken
+          group_best[b.i] = 1.f;
         }
       }
     }
-    __syncthreads();
-    if (wave == 0) {
+    wave_lds_fence();
 #pragma unroll
-      for (int j = 0; j < kMaxExpertsPerLane; ++j) {
-        const int e = lane + j * kWave;
-        if (e < experts && group_best[e / per] == 0.f) choice[j] = -INFINITY;
-      }
+    for (int j = 0; j < EPL; ++j) {
+      const int e = lane + j * kWave;
+      if (e < experts && group_best[e / per] == 0.f) choice[j] = -INFINITY;
     }
   }
-  if (wave != 0) return;
   float sum = 0.f, mine = 0.f;   // lane k keeps the k-th chosen score (top <= 64)
   int mine_id = 0;
   unsigned taken = 0;            // bit j: this lane's expert lane + 64 j has been chosen
   for (int k = 0; k < top; ++k) {
     Best b{-INFINITY, 0x7fffffff};
 #pragma unroll
-    for (int j = 0; j < kMaxExpertsPerLane; ++j) {
+    for (int j = 0; j < EPL; ++j) {
       const int e = lane + j * kWave;
       if (e < experts && !(taken >> j & 1u) && (choice[j] > b.v || (choice[j] == b.v && e < b.i))) {
         b.v = choice[j];
@@ -184,7 +203,7 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const T* __res
     b = wave_best(b);
     float sv = 0.f;
 #pragma unroll
-    for (int j = 0; j < kMaxExpertsPerLane; ++j) {
+    for (int j = 0; j < EPL; ++j) {
       if (b.i == lane + j * kWave) {
         sv = s[j];
         taken |= 1u << j;
@@ -345,124 +364,118 @@ __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __r
   }
 }
 
-// ---- matrix-core form (bfloat16) -----------------------------------------------------------------
-// A workgroup of four waves takes one expert, 256 consecutive rows of the step and a tile of output columns (64 gate
-// and the 64 matching up columns, or 128 columns of down).  It lists the rows of its 256 that chose the expert, in row
-// order, and walks them 64 at a time: wave w multiplies rows 16 w .. 16 w + 15 of the 64 by the whole column tile
-// with `v_mfma_f32_16x16x32_bf16`.  The weight tile of a k step (128 rows of 32) goes through LDS once for the four
-// waves; a wave's own rows come straight from memory, sixteen bytes a lane, which is the A operand as it lies.  The
-// next k step's loads are in flight while this one's products run.  K a multiple of 8; rows 16-byte aligned.
+// ---- matrix-core forms (bfloat16) ----------------------------------------------------------------
+// `v_mfma_f32_16x16x32_bf16`: both operands are eight consecutive k a lane (row or column lane % 16, k from 8 (lane / 16)
+// on), the result's lane holds rows 4 (lane / 16) .. + 3 of column lane % 16.  K a multiple of 8; rows 16-byte aligned.
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
 typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
 
-constexpr int kMoeChunk = 256;     // rows of the step a workgroup looks through
-constexpr int kMoeCols = 128;      // weight rows of a tile (gate|up: 64 + 64)
-constexpr int kMoeLdsRow = 40;     // bfloat16 a weight row of 32 takes in LDS (80 bytes: no two lanes of a read on one bank)
+// ---- few rows ------------------------------------------------------------------------------------
+// With at most 64 tokens an expert has a few rows, and a launch lasts as long as its weights take to arrive.  A wave
+// takes sixteen output columns and streams their weight rows (gate|up: the sixteen gate rows and the matching up rows)
+// from memory straight into the A operand through a ring of registers; the rows that chose the expert lie in LDS, a slice
+// of K at a time, as the B operand.
+constexpr int kFewRing = 8;        // steps of 32 k in flight
 
-template <int MODE>
-__global__ __launch_bounds__(256) void moe_expert_mfma_kernel(const bf16* __restrict__ x, long long x_stride,
-                                                              const bf16* __restrict__ w, const int* __restrict__ ids,
-                                                              void* __restrict__ out, int tokens, int top, int N, int K) {
-  constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
-  __shared__ int list_src[kMoeChunk], list_dst[kMoeChunk];
-  __shared__ int wave_count[4];
-  __shared__ __attribute__((aligned(16))) bf16 wt[kMoeCols * kMoeLdsRow];
-  const int e = blockIdx.z;
-  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, n = lane % 16, g = lane / 16;
-  {
-    const int t = blockIdx.x * kMoeChunk + threadIdx.x;
+template <int MODE, int MT>        // MT tiles of sixteen rows at most
+__global__ __launch_bounds__(256) void moe_expert_few_kernel(const bf16* __restrict__ x, long long x_stride,
+                                                             const bf16* __restrict__ w, const int* __restrict__ ids,
+                                                             void* __restrict__ out, int tokens, int top, int N, int K) {
+  constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;
+  constexpr int kSlice = 1024 / MT, kRow = kSlice + 8;       // K of a slice; what a row of it takes in LDS
+  __shared__ int list_src[64], list_dst[64];
+  __shared__ int count;
+  __shared__ __attribute__((aligned(16))) bf16 xs[16 * MT * kRow];
+  const int e = blockIdx.y, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, n = lane % 16, g = lane / 16;
+  if (wave == 0) {
     int slot = -1;
-    if (t < tokens)
+    if (lane < tokens)
       for (int k = 0; k < top; ++k)
-        if (ids[static_cast<int64_t>(t) * top + k] == e) slot = k;
+        if (ids[static_cast<int64_t>(lane) * top + k] == e) slot = k;
     const unsigned long long chose = __ballot(slot >= 0);
-    if (lane == 0) wave_count[wave] = __popcll(chose);
-    __syncthreads();
-    int before = 0;
-    for (int i = 0; i < wave; ++i) before += wave_count[i];
     if (slot >= 0) {
-      const int rank = before + __popcll(chose & ((1ull << lane) - 1ull));
-      list_src[rank] = TOKENS ? t : t * top + slot;
-      list_dst[rank] = t * top + slot;
+      const int rank = __popcll(chose & ((1ull << lane) - 1ull));
+      list_src[rank] = TOKENS ? lane : lane * top + slot;
+      list_dst[rank] = lane * top + slot;
+    }
+    if (lane == 0) count = __popcll(chose);
+  }
+  __syncthreads();
+  const int rows = count;
+  if (rows == 0) return;
+  const int col0 = blockIdx.x * 64 + wave * 16;
+  const bf16* we = w + static_cast<int64_t>(e) * (GATE_UP ? 2 : 1) * N * K;
+  const bf16* wg = we + static_cast<int64_t>(min(col0 + n, N - 1)) * K;
+  const bf16* wu = wg + (GATE_UP ? static_cast<int64_t>(N) * K : 0);
+  const int steps = (K + 31) / 32, tiles = (rows + 15) / 16;
+  u32x4_t ring[kFewRing], ring_u[GATE_UP ? kFewRing : 1];
+  auto fetch = [&](int step, int at) {      // a piece past K is the last piece again; what multiplies it is zero
+    const int k = min(32 * step + 8 * g, K - 8);
+    ring[at] = *reinterpret_cast<const u32x4_t*>(wg + k);
+    if (GATE_UP) ring_u[at] = *reinterpret_cast<const u32x4_t*>(wu + k);
+  };
+#pragma unroll
+  for (int i = 0; i < kFewRing; ++i) fetch(i, i);
+  f32x4_t acc[MT], acc_u[GATE_UP ? MT : 1];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    acc[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (GATE_UP) acc_u[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const u32x4_t zero = {0, 0, 0, 0};
+  for (int k0 = 0; k0 < K; k0 += kSlice) {
+    __syncthreads();      // the slice before has been read
+    for (int i = threadIdx.x; i < rows * (kSlice / 8); i += 256) {
+      const int r = i / (kSlice / 8), c = 8 * (i % (kSlice / 8));
+      *reinterpret_cast<u32x4_t*>(&xs[r * kRow + c]) =
+          k0 + c < K ? *reinterpret_cast<const u32x4_t*>(x + static_cast<int64_t>(list_src[r]) * x_stride + k0 + c) : zero;
     }
     __syncthreads();
-  }
-  const int rows = wave_count[0] + wave_count[1] + wave_count[2] + wave_count[3];
-  if (rows == 0) return;
-  const int cols = GATE_UP ? kMoeCols / 2 : kMoeCols;     // output columns of the tile
-  const int n0 = blockIdx.y * cols;
-  const bf16* we = w + static_cast<int64_t>(e) * (GATE_UP ? 2 : 1) * N * K;
-  // the weight row this thread copies into LDS (two pieces of 8 of a row of 32), or none past N
-  const int wr = threadIdx.x / 2, wpiece = (threadIdx.x % 2) * 16;
-  const int wcol = GATE_UP ? (wr < 64 ? n0 + wr : n0 + wr - 64) : n0 + wr;
-  const bool w_in = wcol < N;
-  const bf16* wsrc = we + static_cast<int64_t>(GATE_UP && wr >= 64 ? N + wcol : wcol) * K;
-  const u32x4_t zero = {0, 0, 0, 0};
-  for (int sub = 0; sub * 64 < rows; ++sub) {
-    const int r = sub * 64 + wave * 16 + n;
-    const bf16* arow = x + static_cast<int64_t>(list_src[min(r, rows - 1)]) * x_stride;
-    f32x4_t acc[8];
+    const int last = min(steps, (k0 + kSlice) / 32);
+    for (int s0 = k0 / 32; s0 < last; s0 += kFewRing) {
 #pragma unroll
-    for (int j = 0; j < 8; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    u32x4_t a_next, w_next[2];
-    auto fetch = [&](int k0) {
-      const int ka = k0 + 8 * g;
-      a_next = ka < K ? *reinterpret_cast<const u32x4_t*>(arow + ka) : zero;
+      for (int i = 0; i < kFewRing; ++i) {
+        const bf16x8_t a = __builtin_bit_cast(bf16x8_t, ring[i]), u = __builtin_bit_cast(bf16x8_t, ring_u[GATE_UP ? i : 0]);
+        fetch(s0 + i + kFewRing, i);
+        const int c = 32 * (s0 + i) - k0 + 8 * g;
+        if (s0 + i < last) {
 #pragma unroll
-      for (int h = 0; h < 2; ++h) {
-        const int kw = k0 + wpiece + 8 * h;
-        w_next[h] = (w_in && kw < K) ? *reinterpret_cast<const u32x4_t*>(wsrc + kw) : zero;
-      }
-    };
-    fetch(0);
-    for (int k0 = 0; k0 < K; k0 += 32) {
-      const u32x4_t a_now = a_next;
-      __syncthreads();      // the tile before has been read by every wave
-#pragma unroll
-      for (int h = 0; h < 2; ++h) *reinterpret_cast<u32x4_t*>(&wt[wr * kMoeLdsRow + wpiece + 8 * h]) = w_next[h];
-      __syncthreads();
-      if (k0 + 32 < K) fetch(k0 + 32);
-      const bf16x8_t a_op = __builtin_bit_cast(bf16x8_t, a_now);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const u32x4_t b = *reinterpret_cast<const u32x4_t*>(&wt[(16 * j + n) * kMoeLdsRow + 8 * g]);
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a_op, __builtin_bit_cast(bf16x8_t, b), acc[j], 0, 0, 0);
+          for (int m = 0; m < MT; ++m) {
+            if (m < tiles) {
+              const bf16x8_t b = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(&xs[min(16 * m + n, rows - 1) * kRow + c]));
+              acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[m], 0, 0, 0);
+              if (GATE_UP) acc_u[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u, b, acc_u[m], 0, 0, 0);
+            }
+          }
+        }
       }
     }
-    // acc[j][i] is the product of row 4 g + i of the wave's sixteen and weight row 16 j + n of the tile
+  }
+  // acc[m][i]: output column 4 g + i of the wave's sixteen, listed row 16 m + n
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int r = 16 * m + n;
+    if (r >= rows) continue;
+    const int64_t dst = static_cast<int64_t>(list_dst[r]) * N;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int rr = sub * 64 + wave * 16 + 4 * g + i;
-      if (rr >= rows) continue;
-      const int64_t dst = static_cast<int64_t>(list_dst[rr]) * N;
-      if (GATE_UP) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int col = n0 + 16 * j + n;
-          const float gt = acc[j][i];
-          if (col < N) static_cast<bf16*>(out)[dst + col] = from_float<bf16>(gt / (1.0f + expf(-gt)) * acc[j + 4][i]);
-        }
-      } else {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int col = n0 + 16 * j + n;
-          if (col >= N) continue;
-          if (MODE == kUp)
-            static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(acc[j][i]));
-          else
-            static_cast<float*>(out)[dst + col] = acc[j][i];
-        }
-      }
+      const int col = col0 + 4 * g + i;
+      if (col >= N) continue;
+      const float z = acc[m][i];
+      if (GATE_UP)
+        static_cast<bf16*>(out)[dst + col] = from_float<bf16>(z / (1.0f + expf(-z)) * acc_u[GATE_UP ? m : 0][i]);
+      else if (MODE == kUp)
+        static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(z));
+      else
+        static_cast<float*>(out)[dst + col] = z;
     }
-    __syncthreads();        // before the next 64 rows overwrite the tile
   }
 }
 
-// ---- the same for many rows --------------------------------------------------------------------
-// With a few hundred rows an expert the form above reads every weight fragment from LDS once for sixteen rows, and
-// what a launch waits for is the passes over the weights: every workgroup streams its weight tile over all of K.  Here
-// a workgroup of RG x 4 waves (RG 1 or 2) looks through RG x 256 rows of the step and takes RG x 64 listed rows and 256 weight rows
+// ---- many rows ------------------------------------------------------------------------------------
+// With a few hundred rows an expert what a launch waits for is the passes over the weights: every workgroup streams its
+// weight tile over all of K.  Here a workgroup of RG x 4 waves (RG 1 or 2) looks through RG x 256 rows of the step and takes RG x 64 listed rows and 256 weight rows
 // (128 gate and the 128 matching up columns, or 256 columns of down) a k step, both through LDS: the weight tile is
 // fetched once for all RG groups of 64 rows, and a wave multiplies the 64 rows of its group by 64 weight rows (32
 // gate and their 32 up columns): sixteen products for four row and four weight fragments, twice a k step of 64.  Two
@@ -640,22 +653,35 @@ extern "C" int arle_moe_route(const void* x, long long x_stride, int x_dtype, co
     return static_cast<int>(hipErrorInvalidValue);
   hipStream_t s = static_cast<hipStream_t>(stream);
   const RouteRule rule{softmax, groups, keep, normalize, scale};
-  const size_t lds = static_cast<size_t>(width + 2 * experts + groups) * sizeof(float);
-  if (lds > 60 * 1024) return static_cast<int>(hipErrorInvalidValue);
   const bool vec = width % 8 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 && reinterpret_cast<uintptr_t>(shared_w) % 16 == 0;
-#define ARLE_ROUTE_V(TX, TWT, V)                                                                                   \
-  do {                                                                                                             \
-    static bool raised = false;                                                                                    \
-    if (!raised && lds > 48 * 1024) {                                                                              \
-      const hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_route_kernel<TX, TWT, V>),     \
-                                                 hipFuncAttributeMaxDynamicSharedMemorySize, 60 * 1024);           \
-      if (err != hipSuccess) return static_cast<int>(err);                                                         \
-      raised = true;                                                                                               \
-    }                                                                                                              \
-    moe_route_kernel<TX, TWT, V><<<tokens, kRouteThreads, lds, s>>>(static_cast<const TX*>(x), x_stride,           \
-                                                                    static_cast<const TWT*>(w), bias, b_dtype,      \
-                                                                    correction, c_dtype, static_cast<const TWT*>(shared_w), \
-                                                                    shared_gate, ids, weights, width, experts, top, rule); \
+  // many tokens share each router row four at a time; few are latency, a wave an expert
+  const auto bytes = [&](int tok) { return static_cast<size_t>(tok) * (width + 2 * experts + groups) * sizeof(float); };
+  const int tok = tokens > 128 && bytes(4) <= 80 * 1024 ? 4 : 1;
+  const size_t lds = bytes(tok);
+  if (lds > 80 * 1024) return static_cast<int>(hipErrorInvalidValue);
+#define ARLE_ROUTE_K(TX, TWT, V, TH, TK, EPL)                                                                          \
+  do {                                                                                                                 \
+    static bool raised = false;                                                                                        \
+    if (!raised && lds > 48 * 1024) {                                                                                  \
+      const hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_route_kernel<TX, TWT, V, TH, TK, EPL>), \
+                                                 hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);               \
+      if (err != hipSuccess) return static_cast<int>(err);                                                             \
+      raised = true;                                                                                                   \
+    }                                                                                                                  \
+    moe_route_kernel<TX, TWT, V, TH, TK, EPL><<<(tokens + TK - 1) / TK, TH, lds, s>>>(                                 \
+        static_cast<const TX*>(x), x_stride, static_cast<const TWT*>(w), bias, b_dtype, correction, c_dtype,           \
+        static_cast<const TWT*>(shared_w), shared_gate, ids, weights, tokens, width, experts, top, rule);              \
+  } while (0)
+#define ARLE_ROUTE_T(TX, TWT, V, EPL)                          \
+  do {                                                         \
+    if (tok == 4) ARLE_ROUTE_K(TX, TWT, V, 256, 4, EPL);       \
+    else ARLE_ROUTE_K(TX, TWT, V, 1024, 1, EPL);               \
+  } while (0)
+#define ARLE_ROUTE_V(TX, TWT, V)                                        \
+  do {                                                                  \
+    if (experts <= kWave) ARLE_ROUTE_T(TX, TWT, V, 1);                  \
+    else if (experts <= 4 * kWave) ARLE_ROUTE_T(TX, TWT, V, 4);         \
+    else ARLE_ROUTE_T(TX, TWT, V, kMaxExpertsPerLane);                  \
   } while (0)
 #define ARLE_ROUTE(TX, TWT)                          \
   do {                                               \
@@ -669,6 +695,8 @@ extern "C" int arle_moe_route(const void* x, long long x_stride, int x_dtype, co
   }
 #undef ARLE_ROUTE
 #undef ARLE_ROUTE_V
+#undef ARLE_ROUTE_T
+#undef ARLE_ROUTE_K
   return launch_status();
 }
 
@@ -723,13 +751,22 @@ extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w,
 #undef ARLE_TILES
       return launch_status();
     }
-    const int cols = mode == kGateUp ? kMoeCols / 2 : kMoeCols;
-    const dim3 mgrid((tokens + kMoeChunk - 1) / kMoeChunk, (N + cols - 1) / cols, experts);
-#define ARLE_MFMA(MODE)                                                                                           \
-  moe_expert_mfma_kernel<MODE><<<mgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), \
-                                                     ids, out, tokens, top, N, K)
-    if (mode == kGateUp) ARLE_MFMA(kGateUp); else if (mode == kUp) ARLE_MFMA(kUp); else ARLE_MFMA(kDown);
-#undef ARLE_MFMA
+    const dim3 fgrid((N + 63) / 64, experts);
+#define ARLE_FEW(MODE, MT)                                                                                            \
+  moe_expert_few_kernel<MODE, MT><<<fgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), \
+                                                        ids, out, tokens, top, N, K)
+#define ARLE_FEW_MT(MODE)          \
+  do {                             \
+    if (tokens <= 16)              \
+      ARLE_FEW(MODE, 1);           \
+    else if (tokens <= 32)         \
+      ARLE_FEW(MODE, 2);           \
+    else                           \
+      ARLE_FEW(MODE, 4);           \
+  } while (0)
+    if (mode == kGateUp) ARLE_FEW_MT(kGateUp); else if (mode == kUp) ARLE_FEW_MT(kUp); else ARLE_FEW_MT(kDown);
+#undef ARLE_FEW_MT
+#undef ARLE_FEW
     return launch_status();
   }
   const dim3 grid((tokens + kEM - 1) / kEM, (N + kEN - 1) / kEN, experts);
