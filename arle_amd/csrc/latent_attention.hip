@@ -82,7 +82,7 @@ __device__ __forceinline__ int unknown(int v) {
 
 // A tile in LDS, in pieces of eight numbers: piece p of key row r lies at r * KP + (p ^ (r & 15)), piece p of value row c
 // at c * 8 + (p ^ ((c >> 1) & 7)), so that the sixteen lanes that are served together never share a bank.
-template <int NCT, int NDS>   // tiles of 32 of C; steps of 16 of D at most
+template <int NCT, int NDS>   // tiles of 32 of C; steps of 16 of D, of which those past D multiply zeros of the query
 __global__ __launch_bounds__(kLaThreads, NCT <= 6 ? 2 : 1) void latent_attn_portion_kernel(const LatentArgs a) {
   constexpr int KP = (2 * NDS + 15) / 16 * 16;              // pieces a key row takes
   __shared__ __attribute__((aligned(16))) bf16 ks[kLaKeys * KP * 8];
@@ -116,7 +116,10 @@ __global__ __launch_bounds__(kLaThreads, NCT <= 6 ? 2 : 1) void latent_attn_port
   const int nds = a.D / 16, np = a.D / 8;
   u32x4_t qf[NDS];
 #pragma unroll
-  for (int s = 0; s < NDS; ++s) qf[s] = s < nds ? *reinterpret_cast<const u32x4_t*>(a.q + row * a.D + 16 * s + 8 * g) : u32x4_t{0, 0, 0, 0};
+  for (int s = 0; s < NDS; ++s) {
+    const u32x4_t v = *reinterpret_cast<const u32x4_t*>(a.q + row * a.D + 16 * min(s, nds - 1) + 8 * g);
+    qf[s] = s < nds ? v : u32x4_t{0, 0, 0, 0};
+  }
   f32x16_t o[NCT];
 #pragma unroll
   for (int c = 0; c < NCT; ++c)
@@ -127,18 +130,23 @@ __global__ __launch_bounds__(kLaThreads, NCT <= 6 ? 2 : 1) void latent_attn_port
   // the pages of a tile's four groups of sixteen keys, asked for a tile ahead; keys outside [kmin, kmax] are fetched as
   // the nearest one inside (their pages may be gone, or not there yet)
   auto inside = [&](int key) { return min(max(key, kmin), kmax); };
-  int ids[4];
+  int id0, id1, id2, id3;
   auto ask = [&](int t0) {
-#pragma unroll
-    for (int j = 0; j < 4; ++j) ids[j] = table[inside(t0 + 16 * j) >> a.page_shift];
+    id0 = table[inside(t0) >> a.page_shift];
+    id1 = table[inside(t0 + 16) >> a.page_shift];
+    id2 = table[inside(t0 + 32) >> a.page_shift];
+    id3 = table[inside(t0 + 48) >> a.page_shift];
   };
-  auto page_of = [&](int in_tile) { return in_tile < 32 ? (in_tile < 16 ? ids[0] : ids[1]) : (in_tile < 48 ? ids[2] : ids[3]); };
+  auto page_of = [&](int in_tile) {
+    const int low_half = in_tile & 16 ? id1 : id0, high_half = in_tile & 16 ? id3 : id2;
+    return in_tile & 32 ? high_half : low_half;
+  };
   ask(kmin / kLaKeys * kLaKeys);
   for (int t0 = kmin / kLaKeys * kLaKeys; t0 <= kmax; t0 += kLaKeys) {
     const int id = unknown(tid), ln = id % 32, lg = id / 32 % 2;
     __syncthreads();                                        // the tile before has been read
     if (page >= kLaKeys && t0 >= kmin && t0 + kLaKeys - 1 <= kmax) {      // all of it in one page
-      const int64_t first = static_cast<int64_t>(__builtin_amdgcn_readfirstlane(ids[0])) * page, off = t0 & (page - 1);
+      const int64_t first = static_cast<int64_t>(__builtin_amdgcn_readfirstlane(id0)) * page, off = t0 & (page - 1);
       const bf16* kbase = a.k_pages + (first + off) * a.D;
       const bf16* vbase = a.v_pages + first * a.C + off;
 #pragma unroll
@@ -191,7 +199,7 @@ __global__ __launch_bounds__(kLaThreads, NCT <= 6 ? 2 : 1) void latent_attn_port
       const bf16* krow = ks + (32 * h + kr) * KP * 8;
 #pragma unroll
       for (int d = 0; d < NDS; ++d)
-        if (d < nds) s = mfma32(*reinterpret_cast<const u32x4_t*>(krow + ((2 * d + lg) ^ (kr & 15)) * 8), qf[d], s);
+        s = mfma32(*reinterpret_cast<const u32x4_t*>(krow + ((2 * d + lg) ^ (kr & 15)) * 8), qf[d], s);
       float top = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
@@ -270,7 +278,10 @@ __global__ __launch_bounds__(kLaThreads) void latent_attn_decode_kernel(const La
   }
   u32x4_t qf[NDS];
 #pragma unroll
-  for (int s = 0; s < NDS; ++s) qf[s] = s < nds ? *reinterpret_cast<const u32x4_t*>(a.q + row * a.D + 16 * s + 8 * g) : u32x4_t{0, 0, 0, 0};
+  for (int s = 0; s < NDS; ++s) {
+    const u32x4_t v = *reinterpret_cast<const u32x4_t*>(a.q + row * a.D + 16 * min(s, nds - 1) + 8 * g);
+    qf[s] = s < nds ? v : u32x4_t{0, 0, 0, 0};
+  }
   f32x16_t o[NCT];
 #pragma unroll
   for (int c = 0; c < NCT; ++c)
@@ -301,8 +312,7 @@ __global__ __launch_bounds__(kLaThreads) void latent_attn_decode_kernel(const La
 #pragma unroll
     for (int i = 0; i < 16; ++i) s[i] = 0.f;
 #pragma unroll
-    for (int d = 0; d < NDS; ++d)
-      if (d < nds) s = mfma32(kf[d], qf[d], s);
+    for (int d = 0; d < NDS; ++d) s = mfma32(kf[d], qf[d], s);
     float top = -INFINITY;
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
@@ -453,12 +463,16 @@ extern "C" int arle_latent_attn(const void* q, void* out, const void* k_pages, c
                      static_cast<const bf16*>(v_pages), table, table_stride, seg_row0, seg_slot, seg_start, segments, H, D, C,
                      __builtin_ctz(page_size), scale * kLog2e, window, sink, sink_dtype};
   hipStream_t s = static_cast<hipStream_t>(stream);
-#define ARLE_LA(NCT)                                                                                                   \
+#define ARLE_LA_D(NCT, NDS)                                                                                            \
   do {                                                                                                                 \
     if (splits == 0)                                                                                                   \
-      latent_attn_portion_kernel<NCT, 2 * NCT + 4><<<items, kLaThreads, 0, s>>>(a);                                    \
+      latent_attn_portion_kernel<NCT, NDS><<<items, kLaThreads, 0, s>>>(a);                                            \
     else                                                                                                               \
-      latent_attn_decode_kernel<NCT, 2 * NCT + 4><<<dim3(segments, splits, (H + 31) / 32), kLaThreads, 0, s>>>(a, splits, part_o, part_ml); \
+      latent_attn_decode_kernel<NCT, NDS><<<dim3(segments, splits, (H + 31) / 32), kLaThreads, 0, s>>>(a, splits, part_o, part_ml); \
+  } while (0)
+#define ARLE_LA(NCT)                                                                     \
+  do {                                                                                   \
+    if (R <= 32) ARLE_LA_D(NCT, 2 * NCT + 2); else ARLE_LA_D(NCT, 2 * NCT + 4);          \
   } while (0)
   switch (C / 32) {
     case 1: ARLE_LA(1); break;
@@ -471,6 +485,7 @@ extern "C" int arle_latent_attn(const void* q, void* out, const void* k_pages, c
     default: ARLE_LA(8); break;
   }
 #undef ARLE_LA
+#undef ARLE_LA_D
   if (splits > 1) latent_attn_merge_kernel<<<dim3(segments, H), kWave, 0, s>>>(a, splits, part_o, part_ml);
   return launch_status();
 }
