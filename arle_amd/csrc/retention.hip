@@ -279,19 +279,18 @@ __device__ __forceinline__ ChunkAt find_chunk(const int* seg_row0, int segments,
   return ChunkAt{0, 0, 0};
 }
 
-// Four entries d .. d + 3 of a row x of D entries turned by the angles at `cs`, `sn` (half entries a position).
+// Four entries d .. d + 3 of a row x of D entries turned by the angles at `cs`, `sn` (half entries a position).  The loads
+// stand under no condition: entries that do not turn fetch an angle and drop it.
 __device__ __forceinline__ float4 turned4(const float* x, int d, int rot, const float* cs, const float* sn) {
-  float4 v = ld4<float>(x + d);
+  const float4 v = ld4<float>(x + d);
+  if (rot == 0) return v;
   const int half = rot / 2;
-  if (d < rot) {
-    const bool first = d < half;
-    const int a = first ? d : d - half;
-    const float4 o = ld4<float>(x + (first ? d + half : d - half)), c = ld4<float>(cs + a);
-    float4 s = ld4<float>(sn + a);
-    if (first) s = float4{-s.x, -s.y, -s.z, -s.w};
-    v = float4{fmaf(v.x, c.x, o.x * s.x), fmaf(v.y, c.y, o.y * s.y), fmaf(v.z, c.z, o.z * s.z), fmaf(v.w, c.w, o.w * s.w)};
-  }
-  return v;
+  const bool turns = d < rot, first = d < half;
+  const int a = turns ? (first ? d : d - half) : 0;
+  const float4 o = ld4<float>(x + (turns ? (first ? d + half : d - half) : d)), c = ld4<float>(cs + a), s = ld4<float>(sn + a);
+  const float sign = first ? -1.f : 1.f;
+  const float4 t = {fmaf(v.x, c.x, sign * o.x * s.x), fmaf(v.y, c.y, sign * o.y * s.y), fmaf(v.z, c.z, sign * o.z * s.z), fmaf(v.w, c.w, sign * o.w * s.w)};
+  return turns ? t : v;
 }
 
 struct ChunkArgs {
@@ -311,56 +310,73 @@ struct ChunkArgs {
 };
 
 // U^T of a chunk: work[item, h, e, d] = sum_j g^(n-1-j) k_j[d] v_j[e].
+// NE: tiles of sixteen columns a wave takes at a time; the columns are padded with zeros to whole groups of them.
+template <int NE>
 __global__ __launch_bounds__(kRetThreads) void retention_chunk_sum_kernel(const ChunkArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const ChunkAt at = find_chunk(a.seg_row0, a.segments, blockIdx.x);
   if (at.rows == 0) return;
   const int h = blockIdx.y, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, n = lane % 16, g = lane / 16;
-  const int D = a.D, Dv = a.Dv, DP = (D + 15) / 16 * 16, EP = (Dv + 15) / 16 * 16, kr = DP + 4, vr = EP + 4;
+  const int D = a.D, Dv = a.Dv, DP = (D + 15) / 16 * 16, EP = (Dv + 16 * NE - 1) / (16 * NE) * 16 * NE, kr = DP + 4, vr = EP + 4;
   float* ks = lds;                      // [64][DP + 4]
   float* vs = lds + kChunk * kr;        // [64][EP + 4]
   const int64_t qw = static_cast<int64_t>(a.H) * D;
   const float* pw = a.powers + h * (kChunk + 1);
   const float k_scale = 1.0f / sqrtf(static_cast<float>(D));
   const int steps = (at.rows + 15) / 16;      // sixteen rows at a time; rows past the chunk's are zero
-  const float4 zero = {0.f, 0.f, 0.f, 0.f};
-  for (int i = tid; i < steps * 16 * (DP / 4); i += kRetThreads) {
-    const int r = i / (DP / 4), d = 4 * (i % (DP / 4));
-    float4 v = zero;
-    if (r < at.rows && d < D) {
-      const int64_t t = at.row0 + r, ang = static_cast<int64_t>(a.positions[t]) * (a.rot / 2);
-      v = turned4(a.y + t * a.row_stride + qw + h * D, d, a.rot, a.cos_t + ang, a.sin_t + ang);
-      const float f = k_scale * pw[at.rows - 1 - r];
-      v = float4{v.x * f, v.y * f, v.z * f, v.w * f};
+  // Staged four pieces a thread at a time, their loads in flight together: a piece past the chunk's rows or past a row's
+  // entries fetches one inside and becomes zero.
+  const int64_t pos0 = a.positions[at.row0];      // a segment's positions follow one another
+  const float* y0 = a.y + at.row0 * a.row_stride + qw;
+  for (int base = 0; base < steps * 16 * (DP / 4); base += 4 * kRetThreads) {
+    float4 v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = base + u * kRetThreads + tid, r = min(i / (DP / 4), at.rows - 1), d = min(4 * (i % (DP / 4)), D - 4);
+      const int64_t ang = (pos0 + r) * (a.rot / 2);
+      v[u] = turned4(y0 + r * a.row_stride + h * D, d, a.rot, a.cos_t + ang, a.sin_t + ang);
     }
-    *reinterpret_cast<float4*>(&ks[r * kr + d]) = v;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = base + u * kRetThreads + tid, r = i / (DP / 4), d = 4 * (i % (DP / 4));
+      const float f = (r < at.rows && d < D) ? k_scale * pw[max(at.rows - 1 - r, 0)] : 0.f;
+      if (i < steps * 16 * (DP / 4)) *reinterpret_cast<float4*>(&ks[r * kr + d]) = float4{v[u].x * f, v[u].y * f, v[u].z * f, v[u].w * f};
+    }
   }
-  for (int i = tid; i < steps * 16 * (EP / 4); i += kRetThreads) {
-    const int r = i / (EP / 4), e = 4 * (i % (EP / 4));
-    *reinterpret_cast<float4*>(&vs[r * vr + e]) =
-        (r < at.rows && e < Dv) ? ld4<float>(a.y + (at.row0 + r) * a.row_stride + 2 * qw + h * Dv + e) : zero;
+  for (int base = 0; base < steps * 16 * (EP / 4); base += 4 * kRetThreads) {
+    float4 v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = base + u * kRetThreads + tid, r = min(i / (EP / 4), at.rows - 1), e = min(4 * (i % (EP / 4)), Dv - 4);
+      v[u] = ld4<float>(y0 + r * a.row_stride + qw + h * Dv + e);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = base + u * kRetThreads + tid, r = i / (EP / 4), e = 4 * (i % (EP / 4));
+      if (i < steps * 16 * (EP / 4))
+        *reinterpret_cast<float4*>(&vs[r * vr + e]) = (r < at.rows && e < Dv) ? v[u] : float4{0.f, 0.f, 0.f, 0.f};
+    }
   }
   __syncthreads();
   float* dst = a.work + (static_cast<int64_t>(blockIdx.x) * a.H + h) * D * Dv;
   for (int d0 = 16 * wave; d0 < DP; d0 += 16 * kRetWaves) {
-    for (int e0 = 0; e0 < EP; e0 += 128) {
-      f32x4_t acc[8];
+    for (int e0 = 0; e0 < EP; e0 += 16 * NE) {
+      f32x4_t acc[NE];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      for (int j = 0; j < NE; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
       for (int s = 0; s < steps; ++s) {
         const int r = 16 * s + 4 * g;
         const float* kp = ks + r * kr + d0 + n;
         const float4 ka = {kp[0], kp[kr], kp[2 * kr], kp[3 * kr]};
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          if (e0 + 16 * j < EP) {
-            const float* vp = vs + r * vr + e0 + 16 * j + n;
-            acc[j] = mfma4(ka, float4{vp[0], vp[vr], vp[2 * vr], vp[3 * vr]}, acc[j]);
-          }
+        for (int j = 0; j < NE; ++j) {
+          const float* vp = vs + r * vr + e0 + 16 * j + n;
+          acc[j] = mfma4(ka, float4{vp[0], vp[vr], vp[2 * vr], vp[3 * vr]}, acc[j]);
         }
       }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
+      for (int j = 0; j < NE; ++j) {
         const int e = e0 + 16 * j + n, d = d0 + 4 * g;
         if (e < Dv && d < D) st4<float>(dst + static_cast<int64_t>(e) * D + d, float4{acc[j][0], acc[j][1], acc[j][2], acc[j][3]});
       }
@@ -412,14 +428,17 @@ __global__ __launch_bounds__(kRetThreads) void retention_chunk_out_kernel(const 
   const ChunkAt at = find_chunk(a.seg_row0, a.segments, blockIdx.x);
   if (at.rows == 0) return;
   const int h = blockIdx.y, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave, n = lane % 16, g = lane / 16;
-  const int D = a.D, Dv = a.Dv, EP = (Dv + 15) / 16 * 16, vr = EP + 4;
-  float* ps = lds;                                 // [64][68]: the masked scores
-  float* qs = lds + kChunk * kSliceRow;            // [64][68], then k's slice; later v, [64][EP + 4]
+  const int D = a.D, Dv = a.Dv;
+  constexpr int EP = 16 * NV, vr = EP + 4;         // columns, those past Dv zero
+  float* qs = lds;                                 // [64][68] q's slice, then k's; later v, [64][EP + 4]
   float* ks = qs + kChunk * kSliceRow;
   float* vs = qs;
+  float* ss = lds + kChunk * max(2 * kSliceRow, vr);   // [EP][68] the state's slice; later the masked scores, [64][68]
+  float* ps = ss;
   const int64_t qw = static_cast<int64_t>(a.H) * D;
   const float k_scale = 1.0f / sqrtf(static_cast<float>(D));
   if (tid <= kChunk) pw[tid] = a.powers[h * (kChunk + 1) + tid];
+  const int64_t pos0 = a.positions[at.row0];       // a segment's positions follow one another
   const float* S0 = a.work + (static_cast<int64_t>(blockIdx.x) * a.H + h) * D * Dv;     // [e][d]
   const int blocks = (at.rows + 15) / 16;          // row blocks of sixteen that hold rows
   const float4 zero = {0.f, 0.f, 0.f, 0.f};
@@ -428,35 +447,51 @@ __global__ __launch_bounds__(kRetThreads) void retention_chunk_out_kernel(const 
   for (int j = 0; j < 4; ++j) p[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int j = 0; j < NV; ++j) o[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float4 v_next[NV];                               // the chunk's values, 64 rows of EP entries over the workgroup
+#pragma unroll
+  for (int x = 0; x < NV; ++x) {
+    const int i = x * kRetThreads + tid, r = min(i / (EP / 4), at.rows - 1), e = min(4 * (i % (EP / 4)), Dv - 4);
+    v_next[x] = ld4<float>(a.y + (at.row0 + r) * a.row_stride + 2 * qw + h * Dv + e);
+  }
   for (int d0 = 0; d0 < D; d0 += kSliceD) {
+    float4 s_next[NV];                             // EP rows of 64 over the workgroup
+#pragma unroll
+    for (int x = 0; x < NV; ++x) {
+      const int i = x * kRetThreads + tid, e = min(i / (kSliceD / 4), Dv - 1), d = min(d0 + 4 * (i % (kSliceD / 4)), D - 4);
+      s_next[x] = ld4<float>(S0 + static_cast<int64_t>(e) * D + d);
+    }
     __syncthreads();                               // the slice before has been read
-    for (int i = tid; i < 2 * kChunk * (kSliceD / 4); i += kRetThreads) {
-      const int which = i / (kChunk * (kSliceD / 4)), r = i / (kSliceD / 4) % kChunk, c = 4 * (i % (kSliceD / 4)), d = d0 + c;
-      float4 v = zero;
-      if (r < at.rows && d < D) {
-        const int64_t t = at.row0 + r, ang = static_cast<int64_t>(a.positions[t]) * (a.rot / 2);
-        v = turned4(a.y + t * a.row_stride + which * qw + h * D, d, a.rot, a.cos_t + ang, a.sin_t + ang);
-        if (which) v = float4{v.x * k_scale, v.y * k_scale, v.z * k_scale, v.w * k_scale};
-      }
-      *reinterpret_cast<float4*>(&qs[(which * kChunk + r) * kSliceRow + c]) = v;
+#pragma unroll 2
+    for (int x = 0; x < kChunk * (kSliceD / 4) / kRetThreads; ++x) {
+      const int i = x * kRetThreads + tid, r = i / (kSliceD / 4), c = 4 * (i % (kSliceD / 4)), rr = min(r, at.rows - 1);
+      const int d = min(d0 + c, D - 4);
+      const bool in = r < at.rows && d0 + c < D;
+      const int64_t ang = (pos0 + rr) * (a.rot / 2);
+      const float* row = a.y + (at.row0 + rr) * a.row_stride + h * D;
+      const float4 q4 = turned4(row, d, a.rot, a.cos_t + ang, a.sin_t + ang), k4 = turned4(row + qw, d, a.rot, a.cos_t + ang, a.sin_t + ang);
+      *reinterpret_cast<float4*>(&qs[r * kSliceRow + c]) = in ? q4 : zero;
+      *reinterpret_cast<float4*>(&ks[r * kSliceRow + c]) =
+          in ? float4{k4.x * k_scale, k4.y * k_scale, k4.z * k_scale, k4.w * k_scale} : zero;
+    }
+#pragma unroll
+    for (int x = 0; x < NV; ++x) {                 // (past D the query's slice is zero, columns past Dv are dropped)
+      const int i = x * kRetThreads + tid;
+      *reinterpret_cast<float4*>(&ss[(i / (kSliceD / 4)) * kSliceRow + 4 * (i % (kSliceD / 4))]) = s_next[x];
     }
     __syncthreads();
     if (wave < blocks) {
-      for (int kk = 0; kk < kSliceD && d0 + kk < D; kk += 16) {
+#pragma unroll
+      for (int kk = 0; kk < kSliceD; kk += 16) {   // (past D the slices of q and k are zero)
         const int c = kk + 4 * g;
         const float4 qa = *reinterpret_cast<const float4*>(&qs[(16 * wave + n) * kSliceRow + c]);
-        const float* sp = S0 + min(d0 + c, D - 4);          // (past D the query's slice is zero)
-        float4 sb[NV];
 #pragma unroll
-        for (int j = 0; j < NV; ++j) sb[j] = ld4<float>(sp + static_cast<int64_t>(min(16 * j + n, Dv - 1)) * D);
+        for (int j = 0; j < 4; ++j) p[j] = mfma4(qa, *reinterpret_cast<const float4*>(&ks[(16 * j + n) * kSliceRow + c]), p[j]);
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (j <= wave) p[j] = mfma4(qa, *reinterpret_cast<const float4*>(&ks[(16 * j + n) * kSliceRow + c]), p[j]);
-#pragma unroll
-        for (int j = 0; j < NV; ++j) o[j] = mfma4(qa, sb[j], o[j]);
+        for (int j = 0; j < NV; ++j) o[j] = mfma4(qa, *reinterpret_cast<const float4*>(&ss[(16 * j + n) * kSliceRow + c]), o[j]);
       }
     }
   }
+  __syncthreads();                                 // the last slices have been read by every wave
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int r = 16 * wave + 4 * g + i;
@@ -468,11 +503,19 @@ __global__ __launch_bounds__(kRetThreads) void retention_chunk_out_kernel(const 
 #pragma unroll
     for (int j = 0; j < NV; ++j) o[j][i] *= pw[r + 1];
   }
-  __syncthreads();                                 // q and k have been read by every wave
-  for (int i = tid; i < blocks * 16 * (EP / 4); i += kRetThreads) {
-    const int r = i / (EP / 4), e = 4 * (i % (EP / 4));
-    *reinterpret_cast<float4*>(&vs[r * vr + e]) =
-        (r < at.rows && e < Dv) ? ld4<float>(a.y + (at.row0 + r) * a.row_stride + 2 * qw + h * Dv + e) : zero;
+  // the gates are asked for now, in front of the last products (rows and columns past the end: one inside, dropped)
+  float gates[4][NV];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int64_t t = at.row0 + min(16 * wave + 4 * g + i, at.rows - 1);
+    const float* gate = a.y + t * a.row_stride + 2 * qw + static_cast<int64_t>(a.H) * Dv + h * Dv;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) gates[i][j] = gate[min(16 * j + n, Dv - 1)];
+  }
+#pragma unroll
+  for (int x = 0; x < NV; ++x) {
+    const int i = x * kRetThreads + tid, r = i / (EP / 4), e = 4 * (i % (EP / 4));
+    *reinterpret_cast<float4*>(&vs[r * vr + e]) = (r < at.rows && e < Dv) ? v_next[x] : zero;
   }
   __syncthreads();
   if (wave >= blocks) return;
@@ -481,10 +524,8 @@ __global__ __launch_bounds__(kRetThreads) void retention_chunk_out_kernel(const 
     const float4 pa = *reinterpret_cast<const float4*>(&ps[(16 * wave + n) * kSliceRow + r]);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      if (16 * j < EP) {
-        const float* vp = vs + r * vr + 16 * j + n;
-        o[j] = mfma4(pa, float4{vp[0], vp[vr], vp[2 * vr], vp[3 * vr]}, o[j]);
-      }
+      const float* vp = vs + r * vr + 16 * j + n;
+      o[j] = mfma4(pa, float4{vp[0], vp[vr], vp[2 * vr], vp[3 * vr]}, o[j]);
     }
   }
 #pragma unroll
@@ -497,11 +538,10 @@ __global__ __launch_bounds__(kRetThreads) void retention_chunk_out_kernel(const 
     const float inv = 1.0f / sqrtf(lanes16_sum(ss) / static_cast<float>(Dv) + eps);
     if (r >= at.rows) continue;
     const int64_t t = at.row0 + r;
-    const float* gate = a.y + t * a.row_stride + 2 * qw + static_cast<int64_t>(a.H) * Dv + h * Dv;
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int e = 16 * j + n;
-      if (e < Dv) store_from_float(out, out_dtype, (t * a.H + h) * Dv + e, o[j][i] * inv * gate_act(gate[e], kActSilu));
+      if (e < Dv) store_from_float(out, out_dtype, (t * a.H + h) * Dv + e, o[j][i] * inv * gate_act(gates[i][j], kActSilu));
     }
   }
 }
@@ -574,30 +614,34 @@ extern "C" int arle_retention_chunks(const float* y, long long row_stride, const
     return static_cast<int>(hipErrorInvalidValue);
   const ChunkArgs a{y, row_stride, cos_t, sin_t, rot, positions, seg_row0, seg_slot, segments, powers, s_state, work, H, D, Dv};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const int DP = (D + 15) / 16 * 16, EP = (Dv + 15) / 16 * 16;
-  const size_t sum_lds = static_cast<size_t>(kChunk) * (DP + 4 + EP + 4) * sizeof(float);
+  const int DP = (D + 15) / 16 * 16;
+  const int columns = Dv <= 64 ? 64 : (Dv <= 128 ? 128 : 256);
+  const size_t sum_lds = static_cast<size_t>(kChunk) * (DP + 4 + columns + 4) * sizeof(float);
+  const size_t out_lds = (static_cast<size_t>(kChunk) * max(2 * kSliceRow, columns + 4) + static_cast<size_t>(columns) * kSliceRow) * sizeof(float);
   static bool raised = false;
   if (!raised) {
-    const void* kernels[] = {reinterpret_cast<const void*>(&retention_chunk_sum_kernel),
+    const void* kernels[] = {reinterpret_cast<const void*>(&retention_chunk_sum_kernel<4>),
+                             reinterpret_cast<const void*>(&retention_chunk_sum_kernel<8>),
                              reinterpret_cast<const void*>(&retention_chunk_out_kernel<4>),
                              reinterpret_cast<const void*>(&retention_chunk_out_kernel<8>),
                              reinterpret_cast<const void*>(&retention_chunk_out_kernel<16>)};
     for (const void* f : kernels) {
-      const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 140 * 1024);
+      const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024);
       if (e != hipSuccess) return static_cast<int>(e);
     }
     raised = true;
   }
-  retention_chunk_sum_kernel<<<dim3(items, H), kRetThreads, sum_lds, s>>>(a);
-  retention_chunk_carry_kernel<<<dim3(segments, H, (D / 4 * Dv + kRetThreads - 1) / kRetThreads), kRetThreads, 0, s>>>(a);
-  const size_t out_lds = static_cast<size_t>(kChunk) * (kSliceRow + max(2 * kSliceRow, EP + 4)) * sizeof(float);
   const dim3 grid(items, H);
-  if (EP <= 64) {
+  if (columns == 64)
+    retention_chunk_sum_kernel<4><<<grid, kRetThreads, sum_lds, s>>>(a);
+  else
+    retention_chunk_sum_kernel<8><<<grid, kRetThreads, sum_lds, s>>>(a);
+  retention_chunk_carry_kernel<<<dim3(segments, H, (D / 4 * Dv + kRetThreads - 1) / kRetThreads), kRetThreads, 0, s>>>(a);
+  if (columns == 64)
     retention_chunk_out_kernel<4><<<grid, kRetThreads, out_lds, s>>>(a, eps, out, out_dtype);
-  } else if (EP <= 128) {
+  else if (columns == 128)
     retention_chunk_out_kernel<8><<<grid, kRetThreads, out_lds, s>>>(a, eps, out, out_dtype);
-  } else {
+  else
     retention_chunk_out_kernel<16><<<grid, kRetThreads, out_lds, s>>>(a, eps, out, out_dtype);
-  }
   return launch_status();
 }

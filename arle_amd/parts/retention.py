@@ -29,7 +29,7 @@ class RetentionMixer(Part):
 
     graph_safe = True  # rows, slots and positions are read on the GPU; launches depend on shapes only
 
-    CHUNKS_FROM = 17    # rows of the longest portion from which on the form over chunks is ahead
+    CHUNKS_FROM = 192    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
 
     @classmethod
     def declare_weights(cls, params):

@@ -102,12 +102,14 @@ def run_mixer(part, x, cuts, *, page=4, dtype=F32):
 CUTS = [(1000,), (1,), (2,), (5, 2, 7, 3, 1, 16, 2)]
 
 
-def mixer_case(kind, mixer, dtype, seed, T, *, page=4, loud=(), std=0.3, cuts=CUTS, tol=None, limits=None):
+def mixer_case(kind, mixer, dtype, seed, T, *, page=4, loud=(), std=0.3, cuts=CUTS, tol=None, limits=None, setup=None):
     """A mixer alone against its plain function, in every cutting; in float32 the cuttings agree bit for bit.
     loud: positions whose input dwarfs the others', so that a key seen or hidden by mistake shows.
     limits(x, w, want) -> a bound for every row beside the tolerance."""
     raw, spec = one_layer(kind, mixer)
     part, tensors = random_part("mixer", spec.layers[0].mixer, dtype, seed, std)
+    if setup is not None:
+        setup(part)
     x = rnd((T, raw["width"]), seed + 100)
     for p in loud:
         if 0 <= p < T:
@@ -364,8 +366,11 @@ RET_CUTS = CUTS + [(64, 1), (63, 65, 2), (17, 1, 1, 33), (128, 3)]
 def test_retention_equals_the_plain_recurrence_in_every_cut(dtype, case):
     mixer, T = RETENTIONS[case]
     # loud rows at a chunk's borders and at the start: their terms are heard as far as the decay reaches
-    mixer_case("retention", mixer, dtype, 200 + 20 * case, T, loud=(0, 63, 64), std=0.25, cuts=RET_CUTS,
-               tol=2e-4 if dtype == F32 else None, limits=product_jitter("retention", mixer, dtype))
+    # in bfloat16 with the form over chunks from seventeen rows on, and row by row however long
+    for chunks_from in (17, 10 ** 6) if dtype == BF16 else (None,):
+        mixer_case("retention", mixer, dtype, 200 + 20 * case, T, loud=(0, 63, 64), std=0.25, cuts=RET_CUTS,
+                   tol=2e-4 if dtype == F32 else None, limits=product_jitter("retention", mixer, dtype),
+                   setup=lambda part: chunks_from and setattr(part, "CHUNKS_FROM", chunks_from))
 
 
 OP_CASES = [
@@ -523,6 +528,26 @@ def test_the_products_of_ungated_experts_next_to_each_other():
             outs = ops.moe_expert(act, down.to(DEV, dtype), ids.to(DEV), ops.MOE_DOWN)
             want = torch.einsum("tjn,tjkn->tjk", act.double().cpu().view(tokens, top, N), down.double()[ids.long()])
             close(outs.view(tokens, top, K), want, F32, f"down {tokens} {dtype}", tol=1e-5)
+
+
+@pytest.mark.parametrize("tokens,E,top,N,K", [(1, 4, 2, 96, 2568), (16, 3, 2, 40, 1096), (30, 2, 1, 130, 1304), (64, 3, 2, 72, 2056),
+                                              (8, 16, 4, 200, 264), (33, 1, 1, 20, 32)])
+def test_the_experts_products_of_few_rows_in_slices_of_a_long_row(tokens, E, top, N, K):
+    """Rows in one, two and four tiles of sixteen; a row longer than a slice and no multiple of it; columns that end
+    inside a tile; gated and ungated."""
+    x, up, gate_up = rnd((tokens, K), 1), rnd((E, N, K), 2, K ** -0.5), rnd((E, 2 * N, K), 3, K ** -0.5)
+    ids = torch.stack([torch.randperm(E, generator=torch.Generator().manual_seed(t))[:top] for t in range(tokens)]).to(torch.int32)
+    d = lambda t: t.to(DEV, BF16)
+    pick = lambda w: torch.einsum("tk,tjnk->tjn", x.double(), w.double()[ids.long()])
+    got = ops.moe_expert(d(x), d(up), ids.to(DEV), ops.MOE_UP)
+    close(got.view(tokens, top, N), torch.relu(pick(up)) ** 2, BF16, "up", tol=1e-2)
+    z = pick(gate_up)
+    got = ops.moe_expert(d(x), d(gate_up), ids.to(DEV), ops.MOE_GATE_UP)
+    close(got.view(tokens, top, N), plain.silu(z[..., :N]) * z[..., N:], BF16, "gate and up", tol=1e-2)
+    rows = rnd((tokens * top, K), 4)
+    got = ops.moe_expert(d(rows), d(up), ids.to(DEV), ops.MOE_DOWN)
+    want = torch.einsum("rk,rnk->rn", rows.double(), up.double()[ids.long().flatten()])
+    close(got, want, F32, "down", tol=1e-5)
 
 
 # ----------------------------------------------------------------------------------- whole models
