@@ -91,7 +91,13 @@ __global__ __launch_bounds__(kLatentThreads) void latent_down_kernel(
   float ss = 0.f;
   for (int i = threadIdx.x; i < width; i += kLatentThreads) {
     float v = to_float(src[i]);
-    for (int p = 1; p < parts; ++p) v += to_float(src[p * part_stride + i]);
+    for (int p0 = 1; p0 < parts; p0 += 4) {      // added in order, four in flight (a part past the last is fetched again and dropped)
+      float e[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) e[u] = to_float(src[min(p0 + u, parts - 1) * part_stride + i]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v += p0 + u < parts ? e[u] : 0.f;
+    }
     row[i] = v;
     if (i < normed) ss = fmaf(v, v, ss);
   }

@@ -808,6 +808,14 @@ def sovutar_config(shape: str, layers: int) -> dict:
             "logit_softcap": 30.0, "layers": out}
 
 
+def latent_attention_work(m: dict, layers: int, tokens: int, batch: int, keys: float) -> dict:
+    """The attention over latents: `keys` keys a row; decoded rows read each request's latents twice (as keys and turned,
+    as values)."""
+    pair = 2 * m["kv_rank"] + m["rot_dim"]
+    work = (layers * batch * keys * pair * 2 if tokens == batch else 0, layers * tokens * keys * m["heads"] * 2 * pair)
+    return {"latent_attn_portion": work, "latent_attn_decode": work}
+
+
 def sovutar_work(raw: dict, q: dict, tokens: int, batch: int, context: int) -> dict:
     """Ideal work of the kernels that are new with this design, per step: kernel family -> (bytes, flops)."""
     W, L = raw["width"], len(raw["layers"])
@@ -823,8 +831,8 @@ def sovutar_work(raw: dict, q: dict, tokens: int, batch: int, context: int) -> d
     span = a["mask"]["size"]
     keys_a = (context % span if decode else min(span, tokens) / 2) or 1
     keys_l = min(m["mask"]["size"], context) if decode else min(m["mask"]["size"], tokens / 2)
-    attn_bytes = (n_att * batch * keys_a * G * (D + Dv) * 2 + n_lat * batch * keys_l * (2 * C + R) * 2) if decode else 0
-    attn_flops = n_att * tokens * keys_a * H * 2 * (D + Dv) + n_lat * tokens * keys_l * LH * 2 * (2 * C + R)
+    attn_bytes = n_att * batch * keys_a * G * (D + Dv) * 2 if decode else 0
+    attn_flops = n_att * tokens * keys_a * H * 2 * (D + Dv)
     active = min(E, batch * top) if decode else E
     return {
         "norm_add_kernel": (tokens * W * (L * (4 + 8 + 2) + L * ((top + 1) * 4 + 8 + 2)), 0),
@@ -833,6 +841,7 @@ def sovutar_work(raw: dict, q: dict, tokens: int, batch: int, context: int) -> d
         "head_proj": (n_lat * (tokens * LH * (LD + 2 * C + LDv) * 2 + LH * C * (LD + LDv) * 2),
                       n_lat * tokens * LH * C * (LD + LDv) * 2),
         "attn_softcap_mfma_kernel": (attn_bytes, attn_flops),
+        **latent_attention_work(m, n_lat, tokens, batch, keys_l),
         "moe_route_kernel": (L * (tokens + E) * W * 2, 0),
         "moe_expert": (L * (active * 3 * W * F * 2 + tokens * top * (W * 2 + F * 4 + W * 4)), L * tokens * top * 3 * W * F * 2),
     }
@@ -941,8 +950,7 @@ def retudra_work(raw: dict, q: dict, tokens: int, batch: int, context: int) -> d
         m = of("latent_attention")[0]["mixer"]
         LH, LD, R, LDv, C = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
         keys = context if decode else tokens / 2
-        att_bytes += n_lat * batch * keys * (2 * C + R) * 2 if decode else 0
-        att_flops += n_lat * tokens * keys * LH * 2 * (2 * C + R)
+        work.update(latent_attention_work(m, n_lat, tokens, batch, keys))
         work["latent_prep_kernel"] = (n_lat * tokens * (LH * R * 2 + (C + R) + 2 * C + R) * 2, 0)
         work["head_proj"] = (n_lat * (tokens * LH * (LD + 2 * C + LDv) * 2 + LH * C * (LD + LDv) * 2),
                              n_lat * tokens * LH * C * (LD + LDv) * 2)
@@ -1017,12 +1025,9 @@ def nafezen_work(raw: dict, tokens: int, batch: int, context: int) -> dict:
         m = of("latent_attention")[0]["mixer"]
         LH, LD, R, LDv, C, Cq = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["q_rank"]
         keys = context if decode else tokens / 2
-        work["attn_softcap_mfma_kernel"] = (n_lat * batch * keys * (2 * C + R) * 2 if decode else 0,
-                                            n_lat * tokens * keys * LH * 2 * (2 * C + R))
-        work["rmsnorm"] = (n_lat * tokens * Cq * 4, 0)
+        work.update(latent_attention_work(m, n_lat, tokens, batch, keys))
         work["latent_down"] = (n_lat * tokens * ((Cq + C + R) * 4 + (Cq + 2 * C + R) * 2), 0)
-        work["latent_prep_kernel"] = (n_lat * tokens * (LH * R * 2 + (C + R) + 2 * C + R) * 2, 0)
-        work["head_proj"] = (n_lat * (tokens * LH * (LD + 2 * C + LDv) * 2 + LH * C * (LD + LDv) * 2),
+        work["head_proj"] = (n_lat * (tokens * LH * (LD + 2 * R + 2 * C + LDv) * 2 + LH * C * (LD + LDv) * 2),
                              n_lat * tokens * LH * C * (LD + LDv) * 2)
     if n_ret:
         r = of("retention")[0]["mixer"]
