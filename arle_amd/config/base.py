@@ -109,3 +109,20 @@ def read_stop_token_ids(model_dir: str, eos_token_id: int | None) -> tuple:
 
 
 Validator = Callable[[Any], None]
+
+
+def read_section(raw: Any, keys: Sequence[Key], where: str) -> dict:
+    """`read_keys` of a nested object; an error names the object."""
+    try:
+        return read_keys(raw, keys)
+    except ConfigError as exc:
+        raise ConfigError(f"{where}: {exc}") from None
+
+
+def require_positive(where: str, **values) -> None:
+    """Sizes and counts: at least one, and within what a 32-bit index reaches."""
+    for name, v in values.items():
+        if v <= 0:
+            raise ConfigError(f"{where}: `{name}` must be positive")
+        if v > 2 ** 31 - 1:
+            raise ConfigError(f"{where}: `{name}` = {v} is beyond what a 32-bit index reaches")

@@ -79,7 +79,7 @@ __global__ __launch_bounds__(kWave) void attn_softcap_simt_kernel(
     const T* __restrict__ v_pages, const int* __restrict__ block_table, int table_stride,
     const int* __restrict__ positions, const int* __restrict__ slot_of_token, int nq, int nkv, int Dk, int Dv,
     int page_size, float scale, float cap, const void* __restrict__ r1, const void* __restrict__ r2, int r_dtype,
-    int window, int chunk, const void* __restrict__ sink, int sink_dtype, int keep_first) {
+    int window, int chunk, const void* __restrict__ sink, int sink_dtype, int keep_first, float out_scale) {
   extern __shared__ float qs[];  // [Dk]
   const int t = blockIdx.x;
   const int h = blockIdx.y;
@@ -158,7 +158,7 @@ __global__ __launch_bounds__(kWave) void attn_softcap_simt_kernel(
     keep = expf(m - m_all);
     l = l * keep + expf(sk - m_all);
   }
-  const float inv_l = keep / l;
+  const float inv_l = keep / l * out_scale;
 #pragma unroll
   for (int i = 0; i < kCapMaxD / kWave; ++i) {
     const int d = lane + i * kWave;
@@ -311,7 +311,8 @@ extern "C" int arle_attn_softcap_simt(const void* q, long long q_stride, void* o
                                       int table_stride, const int* positions, const int* slot_of_token, int tokens,
                                       int nq, int nkv, int Dk, int Dv, int page_size, float scale, float cap,
                                       const void* r1, const void* r2, int r_dtype, int window, int chunk,
-                                      const void* sink, int sink_dtype, int keep_first, void* stream) {
+                                      const void* sink, int sink_dtype, int keep_first, float out_scale,
+                                      void* stream) {
   if (tokens == 0) return 0;
   if (Dk > kCapMaxD || Dv > kCapMaxD || nkv < 1 || nq % nkv != 0 || nq > 65535 || window < 0 || chunk < 0 ||
       keep_first < 0 || (keep_first > 0 && window == 0))
@@ -323,12 +324,14 @@ extern "C" int arle_attn_softcap_simt(const void* q, long long q_stride, void* o
     attn_softcap_simt_kernel<float><<<grid, kWave, lds, s>>>(
         static_cast<const float*>(q), q_stride, static_cast<float*>(out), o_stride, static_cast<const float*>(k_pages),
         static_cast<const float*>(v_pages), block_table, table_stride, positions, slot_of_token, nq, nkv, Dk, Dv,
-        page_size, scale, cap, r1, r2, r_dtype, window, chunk, sink, sink_dtype, keep_first);
+        page_size, scale, cap, r1, r2, r_dtype, window, chunk, sink, sink_dtype, keep_first,
+        out_scale);
   } else {
     attn_softcap_simt_kernel<bf16><<<grid, kWave, lds, s>>>(
         static_cast<const bf16*>(q), q_stride, static_cast<bf16*>(out), o_stride, static_cast<const bf16*>(k_pages),
         static_cast<const bf16*>(v_pages), block_table, table_stride, positions, slot_of_token, nq, nkv, Dk, Dv,
-        page_size, scale, cap, r1, r2, r_dtype, window, chunk, sink, sink_dtype, keep_first);
+        page_size, scale, cap, r1, r2, r_dtype, window, chunk, sink, sink_dtype, keep_first,
+        out_scale);
   }
   return launch_status();
 }
@@ -421,6 +424,7 @@ struct CapArgs {
   const void* sink; int sink_dtype;   // [nq] or null: exp(sink_h) joins the softmax's denominator
   int merge_floats;   // floats of dynamic LDS in front of the page ids
   int keep_first;     // with a window: the request's first so many keys stay visible behind it (0: none)
+  float out_scale;    // a factor on the output, in 32 bits
 };
 
 // KC: chunks of 32 of the key size held (Dk <= 32 KC); VC: chunks of 16 of the value size (Dv <= 16 VC).
@@ -668,7 +672,7 @@ void attn_softcap_mfma_kernel(const CapArgs a) {
       l_all += part_l[w * 16 + n] * f[w];
     }
     if (!live) return;
-    const float inv_l = 1.0f / l_all;
+    const float inv_l = a.out_scale / l_all;
     bf16* orow = a.out + static_cast<int64_t>(row) * a.o_stride + head * a.Dv;
     for (int c = wave; c < n_vc; c += WAVES) {
       f32x4_t o = {0.f, 0.f, 0.f, 0.f};
@@ -685,10 +689,10 @@ void attn_softcap_mfma_kernel(const CapArgs a) {
     return;
   }
   if (!live) return;
-  float inv_l = 1.0f / l_run;
+  float inv_l = a.out_scale / l_run;
   if (a.sink) {
     const float m_all = fmaxf(m_run, sink), keep = __expf(m_run - m_all);
-    inv_l = keep / (l_run * keep + __expf(sink - m_all));
+    inv_l = keep / (l_run * keep + __expf(sink - m_all)) * a.out_scale;
   }
   bf16* orow = a.out + static_cast<int64_t>(row) * a.o_stride + head * a.Dv;
 #pragma unroll
@@ -733,7 +737,7 @@ extern "C" int arle_attn_softcap_mfma(const void* q, long long q_stride, void* o
                                       int segments, int row_blocks, int heads_mode, int nq, int nkv, int Dk, int Dv,
                                       int page_size, float scale, float cap, const void* r1, const void* r2,
                                       int r_dtype, int window, int chunk, const void* sink, int sink_dtype,
-                                      int keep_first, void* stream) {
+                                      int keep_first, float out_scale, void* stream) {
   if (segments == 0) return 0;
   // (kept first keys go with a window alone: under the chunk rule a row's chunk would have to hold them)
   if (Dk % 8 || Dk > 256 || Dv % 16 || Dv > 256 || page_size % 16 || nkv < 1 || nq % nkv || nq > 65535 ||
@@ -743,7 +747,8 @@ extern "C" int arle_attn_softcap_mfma(const void* q, long long q_stride, void* o
   const CapArgs a{static_cast<const bf16*>(q), q_stride, static_cast<bf16*>(out), o_stride,
                   static_cast<const bf16*>(k_pages), static_cast<const bf16*>(v_pages), block_table, table_stride,
                   seg_row0, seg_slot, seg_start, segments, nq, nkv, Dk, Dv, page_size, scale, cap, r1, r2, r_dtype, window,
-                  chunk, sink, sink_dtype, heads_mode ? kCapSplitWaves * ((Dv / 16) * kWave * 4 + 32) : 0, keep_first};
+                  chunk, sink, sink_dtype, heads_mode ? kCapSplitWaves * ((Dv / 16) * kWave * 4 + 32) : 0, keep_first,
+                  out_scale};
   // pages an item can see: its rows' windows (or everything the block table maps) and the tiles' rounding to 32 keys;
   // nothing of a step's lengths, so that a captured launch holds for every later step of its shape
   const long long mapped = static_cast<long long>(table_stride) * page_size;

@@ -226,10 +226,10 @@ __global__ __launch_bounds__(kGdThreads) void gated_delta_scan_kernel(
 }
 
 // One wave a (row, head): o / rms(o) * w * act(gate), act silu or sigmoid (a kAct code).
-template <typename T>
+template <typename T, typename TOut>
 __global__ __launch_bounds__(kWave) void gated_delta_output_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                                    long long gate_stride, const void* __restrict__ weight,
-                                                                   int w_dtype, float eps, T* __restrict__ out, int H,
+                                                                   int w_dtype, float eps, TOut* __restrict__ out, int H,
                                                                    int Dv, int act) {
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x;
@@ -239,7 +239,7 @@ __global__ __launch_bounds__(kWave) void gated_delta_output_kernel(const float* 
   const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(Dv) + eps);
   for (int d = lane; d < Dv; d += kWave) {
     const float z = to_float(gate[t * gate_stride + h * Dv + d]);
-    out[(t * H + h) * Dv + d] = from_float<T>(row[d] * inv * load_as_float(weight, w_dtype, d) * gate_act(z, act));
+    out[(t * H + h) * Dv + d] = from_float<TOut>(row[d] * inv * load_as_float(weight, w_dtype, d) * gate_act(z, act));
   }
 }
 
@@ -282,17 +282,19 @@ extern "C" int arle_gated_delta_scan(const void* q, long long q_stride, const vo
 }
 
 extern "C" int arle_gated_delta_output(const void* o, const void* gate, long long gate_stride, int dtype,
-                                       const void* weight, int w_dtype, float eps, void* out, int tokens, int H, int Dv,
-                                       int act, void* stream) {
+                                       const void* weight, int w_dtype, float eps, void* out, int out_dtype, int tokens,
+                                       int H, int Dv, int act, void* stream) {
   if (tokens == 0) return 0;
   dim3 grid(tokens, H);
   hipStream_t s = static_cast<hipStream_t>(stream);
+#define ARLE_GDO(T, TO)                                                                                              \
+  gated_delta_output_kernel<T, TO><<<grid, kWave, 0, s>>>(static_cast<const float*>(o), static_cast<const T*>(gate), \
+                                                          gate_stride, weight, w_dtype, eps, static_cast<TO*>(out), H, Dv, act)
   if (dtype == kF32) {
-    gated_delta_output_kernel<float><<<grid, kWave, 0, s>>>(static_cast<const float*>(o), static_cast<const float*>(gate),
-                                                            gate_stride, weight, w_dtype, eps, static_cast<float*>(out), H, Dv, act);
+    if (out_dtype == kF32) ARLE_GDO(float, float); else ARLE_GDO(float, bf16);
   } else {
-    gated_delta_output_kernel<bf16><<<grid, kWave, 0, s>>>(static_cast<const float*>(o), static_cast<const bf16*>(gate),
-                                                           gate_stride, weight, w_dtype, eps, static_cast<bf16*>(out), H, Dv, act);
+    if (out_dtype == kF32) ARLE_GDO(bf16, float); else ARLE_GDO(bf16, bf16);
   }
+#undef ARLE_GDO
   return launch_status();
 }

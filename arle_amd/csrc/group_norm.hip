@@ -4,7 +4,7 @@
 //   out_j = x_j / sqrt(mean of x^2 over the group of j + eps) * w_j
 //
 // A row of `width` entries is `groups` equal groups of consecutive entries; with one group it is the plain RMS norm.
-// The terms are what the sublayers in front left to be added (addend.h: tensors, stacks of partial sums, weighted
+// `plain`: no norm and no weight, out_j = x_j (the sum of the residual and the terms in another type).  The terms are what the sublayers in front left to be added (addend.h: tensors, stacks of partial sums, weighted
 // outputs of experts, a factor per row).  The source is the float32 residual, or rows of a table picked by index (an
 // embedding that is normed on its way into the residual); rows picked by index are not written back.  Statistics, sums
 // and the weight are 32-bit; a row's arithmetic depends on nothing but the row.
@@ -33,9 +33,9 @@ __device__ __forceinline__ void group_scales(const float* ssq, float* inv, int g
 template <typename TIn, typename TOut, typename TW, int THREADS, int VPT>
 __global__ __launch_bounds__(THREADS) void group_norm_vec_kernel(const TIn* __restrict__ x, int64_t x_stride,
                                                                  float* __restrict__ back, const Terms terms,
-                                                                 const TW* __restrict__ w, TOut* __restrict__ out,
+                                                                 const TW* __restrict__ w, TOut* __restrict__ out, int64_t out_stride,
                                                                  const int* __restrict__ rows, int width, int groups,
-                                                                 float eps) {
+                                                                 float eps, int plain) {
   extern __shared__ float lds[];   // [width / 4] partial sums of squares, then [groups] scales
   float* ssq = lds;
   float* inv = lds + width / 4;
@@ -95,6 +95,14 @@ __global__ __launch_bounds__(THREADS) void group_norm_vec_kernel(const TIn* __re
       ssq[i / 4] = (v[j].x * v[j].x + v[j].y * v[j].y) + (v[j].z * v[j].z + v[j].w * v[j].w);
     }
   }
+  if (plain) {
+#pragma unroll
+    for (int j = 0; j < VPT; ++j) {
+      const int i = 4 * (tid + j * THREADS);
+      if (i < width) st4<TOut>(out + r * out_stride + i, v[j]);
+    }
+    return;
+  }
   __syncthreads();
   const int size = width / groups;
   group_scales<THREADS>(ssq, inv, groups, size / 4, static_cast<float>(size), eps);
@@ -104,7 +112,7 @@ __global__ __launch_bounds__(THREADS) void group_norm_vec_kernel(const TIn* __re
     const int i = 4 * (tid + j * THREADS);
     if (i < width) {
       const float s = inv[i / size];
-      st4<TOut>(out + r * width + i, float4{v[j].x * s * wv[j].x, v[j].y * s * wv[j].y, v[j].z * s * wv[j].z, v[j].w * s * wv[j].w});
+      st4<TOut>(out + r * out_stride + i, float4{v[j].x * s * wv[j].x, v[j].y * s * wv[j].y, v[j].z * s * wv[j].z, v[j].w * s * wv[j].w});
     }
   }
 }
@@ -115,9 +123,9 @@ constexpr int kGroupThreads = 256;
 template <typename TIn, typename TOut, typename TW>
 __global__ __launch_bounds__(kGroupThreads) void group_norm_kernel(const TIn* __restrict__ x, int64_t x_stride,
                                                                    float* __restrict__ back, const Terms terms,
-                                                                   const TW* __restrict__ w, TOut* __restrict__ out,
+                                                                   const TW* __restrict__ w, TOut* __restrict__ out, int64_t out_stride,
                                                                    const int* __restrict__ rows, int width, int groups,
-                                                                   float eps) {
+                                                                   float eps, int plain) {
   extern __shared__ float lds[];   // [width] the row, then [groups] scales
   float* xs = lds;
   float* inv = lds + width;
@@ -135,8 +143,10 @@ __global__ __launch_bounds__(kGroupThreads) void group_norm_kernel(const TIn* __
       v += sum;
     }
     if (back) back[src * width + i] = v;
+    if (plain) out[r * out_stride + i] = from_float<TOut>(v);
     xs[i] = v;
   }
+  if (plain) return;
   __syncthreads();
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, size = width / groups;
   for (int g = wave; g < groups; g += kGroupThreads / kWave) {
@@ -147,22 +157,23 @@ __global__ __launch_bounds__(kGroupThreads) void group_norm_kernel(const TIn* __
   }
   __syncthreads();
   for (int i = threadIdx.x; i < width; i += kGroupThreads)
-    out[r * width + i] = from_float<TOut>(xs[i] * inv[i / size] * to_float(w[i]));
+    out[r * out_stride + i] = from_float<TOut>(xs[i] * inv[i / size] * to_float(w[i]));
 }
 
 constexpr int kGroupLdsMax = 128 * 1024;   // [width] + [groups] floats of the plain kernel at width 16384, one group an entry
 
 template <typename TIn, typename TOut, typename TW>
 static int launch_group_norm(const void* x, long long x_stride, float* back, const Terms& terms, const void* w, void* out,
-                             const int* rows, int n_rows, int width, int groups, float eps, bool vec, hipStream_t s) {
+                             long long out_stride, const int* rows, int n_rows, int width, int groups, float eps, int plain,
+                             bool vec, hipStream_t s) {
   const TIn* xp = static_cast<const TIn*>(x);
   const TW* wp = static_cast<const TW*>(w);
   TOut* op = static_cast<TOut*>(out);
   if (vec) {
     const size_t lds = static_cast<size_t>(width / 4 + groups) * sizeof(float);   // at most 32 KB
 #define ARLE_GN(THREADS, VPT)                                                                                          \
-  group_norm_vec_kernel<TIn, TOut, TW, THREADS, VPT><<<n_rows, THREADS, lds, s>>>(xp, x_stride, back, terms, wp, op, rows, \
-                                                                                  width, groups, eps)
+  group_norm_vec_kernel<TIn, TOut, TW, THREADS, VPT><<<n_rows, THREADS, lds, s>>>(xp, x_stride, back, terms, wp, op, \
+                                                                                  out_stride, rows, width, groups, eps, plain)
     if (width <= 1024) {
       ARLE_GN(256, 1);
     } else if (n_rows <= 512 && width <= 4096) {   // few rows: the latency of one access a thread
@@ -187,7 +198,8 @@ static int launch_group_norm(const void* x, long long x_stride, float* back, con
     if (e != hipSuccess) return static_cast<int>(e);
     raised = true;
   }
-  group_norm_kernel<TIn, TOut, TW><<<n_rows, kGroupThreads, lds, s>>>(xp, x_stride, back, terms, wp, op, rows, width, groups, eps);
+  group_norm_kernel<TIn, TOut, TW><<<n_rows, kGroupThreads, lds, s>>>(xp, x_stride, back, terms, wp, op, out_stride, rows,
+                                                                      width, groups, eps, plain);
   return launch_status();
 }
 
@@ -196,15 +208,17 @@ static int launch_group_norm(const void* x, long long x_stride, float* back, con
 using namespace arle;
 
 // x: rows of x_dtype, x_stride elements apart; back: float32 [*, width] that the sums are written to (the residual, which
-// x then is), or null.  Three addends (null pointers: none), float32, indexed like x.  out [n_rows, width] of out_dtype.
+// x then is), or null.  Three addends (null pointers: none), float32, indexed like x.  out [n_rows, width] of out_dtype,
+// rows out_stride apart; plain: see above (w then is any `width` readable entries of w_dtype).
 // rows: which rows of x (null: 0..n_rows-1).  groups divides width; width <= 16384.
 extern "C" int arle_group_norm(const void* x, int x_dtype, long long x_stride, float* back, const float* a, int a_parts,
                                long long a_part_stride, long long a_row_stride, const float* a_weights, int a_w_row,
                                int a_w_part, const float* b, int b_parts, long long b_part_stride, long long b_row_stride,
                                const float* b_weights, int b_w_row, int b_w_part, const float* c, int c_parts,
                                long long c_part_stride, long long c_row_stride, const float* c_weights, int c_w_row,
-                               int c_w_part, const void* w, int w_dtype, void* out, int out_dtype, const int* rows,
-                               int n_rows, int width, int groups, float eps, void* stream) {
+                               int c_w_part, const void* w, int w_dtype, void* out, long long out_stride,
+                               int out_dtype, const int* rows, int n_rows, int width, int groups, float eps, int plain,
+                               void* stream) {
   if (n_rows == 0) return 0;
   if (width < 1 || width > 16384 || groups < 1 || width % groups || (a && a_parts < 1) || (b && b_parts < 1) || (c && c_parts < 1))
     return static_cast<int>(hipErrorInvalidValue);
@@ -212,11 +226,11 @@ extern "C" int arle_group_norm(const void* x, int x_dtype, long long x_stride, f
                      {b, b_parts, b_part_stride, b_row_stride, b_weights, b_w_row, b_w_part},
                      {c, c_parts, c_part_stride, c_row_stride, c_weights, c_w_row, c_w_part}}};
   auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
-  bool vec = (width / groups) % 4 == 0 && x_stride % 4 == 0 && al(x) && al(back) && al(w) && al(out);
+  bool vec = (width / groups) % 4 == 0 && x_stride % 4 == 0 && al(x) && al(back) && al(w) && al(out) && out_stride % 4 == 0;
   for (const Addend& t : terms.t) vec = vec && (!t.p || (al(t.p) && t.part_stride % 4 == 0 && t.row_stride % 4 == 0));
   hipStream_t s = static_cast<hipStream_t>(stream);
 #define ARLE_GNL(TI, TO, TWT) \
-  return launch_group_norm<TI, TO, TWT>(x, x_stride, back, terms, w, out, rows, n_rows, width, groups, eps, vec, s)
+  return launch_group_norm<TI, TO, TWT>(x, x_stride, back, terms, w, out, out_stride, rows, n_rows, width, groups, eps, plain, vec, s)
 #define ARLE_GNO(TI, TO)                                          \
   do {                                                            \
     if (w_dtype == kF32) ARLE_GNL(TI, TO, float);                 \

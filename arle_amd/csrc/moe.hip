@@ -258,6 +258,8 @@ constexpr int kExpertThreads = 256;
 //   kGateUp: w [experts, 2 N, K] (gate rows, then up rows), rows of x are tokens, out[(t top + k), n] = silu(g) u of type T
 //   kUp:     w [experts, N, K], rows of x are tokens, out[(t top + k), n] = max(u, 0)^2 of type T
 //   kDown:   w [experts, N, K], rows of x are t top + k, out float32 [(t top + k), n]
+// in_scale (kGateUp, kUp): null, or a factor for every (token, choice) on the expert's input, which by linearity is one on
+// the 32-bit sums in front of the activation.
 constexpr int kDown = 0, kGateUp = 1, kUp = 2;
 
 __device__ __forceinline__ float squared_relu(float u) {
@@ -268,7 +270,8 @@ __device__ __forceinline__ float squared_relu(float u) {
 template <typename T, int MODE>
 __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __restrict__ x, long long x_stride,
                                                                     const T* __restrict__ w, const int* __restrict__ ids,
-                                                                    void* __restrict__ out, int tokens, int top, int N,
+                                                                    const float* __restrict__ in_scale, void* __restrict__ out,
+                                                                    int tokens, int top, int N,
                                                                     int K) {
   constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
   __shared__ int list_t[kEM], list_k[kEM];
@@ -347,16 +350,17 @@ __global__ __launch_bounds__(kExpertThreads) void moe_expert_kernel(const T* __r
   for (int i = 0; i < 4; ++i) {
     const int r = ty * 4 + i;
     if (r >= rows) continue;
-    const int64_t dst = (static_cast<int64_t>(list_t[r]) * top + list_k[r]) * N;
+    const int64_t item = static_cast<int64_t>(list_t[r]) * top + list_k[r], dst = item * N;
+    const float f = MODE != kDown && in_scale ? in_scale[item] : 1.0f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
       if (GATE_UP) {
-        const float g = acc[i][j];
-        static_cast<T*>(out)[dst + n] = from_float<T>(g / (1.0f + expf(-g)) * acc_u[i][j]);
+        const float g = f * acc[i][j];
+        static_cast<T*>(out)[dst + n] = from_float<T>(g / (1.0f + expf(-g)) * (f * acc_u[i][j]));
       } else if (MODE == kUp) {
-        static_cast<T*>(out)[dst + n] = from_float<T>(squared_relu(acc[i][j]));
+        static_cast<T*>(out)[dst + n] = from_float<T>(squared_relu(f * acc[i][j]));
       } else {
         static_cast<float*>(out)[dst + n] = acc[i][j];
       }
@@ -381,7 +385,8 @@ constexpr int kFewRing = 8;        // steps of 32 k in flight
 template <int MODE, int MT>        // MT tiles of sixteen rows at most
 __global__ __launch_bounds__(256) void moe_expert_few_kernel(const bf16* __restrict__ x, long long x_stride,
                                                              const bf16* __restrict__ w, const int* __restrict__ ids,
-                                                             void* __restrict__ out, int tokens, int top, int N, int K) {
+                                                             const float* __restrict__ in_scale, void* __restrict__ out,
+                                                             int tokens, int top, int N, int K) {
   constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;
   constexpr int kSlice = 1024 / MT, kRow = kSlice + 8;       // K of a slice; what a row of it takes in LDS
   __shared__ int list_src[64], list_dst[64];
@@ -458,13 +463,14 @@ __global__ __launch_bounds__(256) void moe_expert_few_kernel(const bf16* __restr
     const int r = 16 * m + n;
     if (r >= rows) continue;
     const int64_t dst = static_cast<int64_t>(list_dst[r]) * N;
+    const float f = MODE != kDown && in_scale ? in_scale[list_dst[r]] : 1.0f;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int col = col0 + 4 * g + i;
       if (col >= N) continue;
-      const float z = acc[m][i];
+      const float z = f * acc[m][i];
       if (GATE_UP)
-        static_cast<bf16*>(out)[dst + col] = from_float<bf16>(z / (1.0f + expf(-z)) * acc_u[GATE_UP ? m : 0][i]);
+        static_cast<bf16*>(out)[dst + col] = from_float<bf16>(z / (1.0f + expf(-z)) * (f * acc_u[GATE_UP ? m : 0][i]));
       else if (MODE == kUp)
         static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(z));
       else
@@ -488,7 +494,8 @@ constexpr int kBigRows = 64;        // listed rows of a group of four waves
 template <int MODE, int RG, int BK>
 __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* __restrict__ x, long long x_stride,
                                                                     const bf16* __restrict__ w, const int* __restrict__ ids,
-                                                                    void* __restrict__ out, int tokens, int top, int N,
+                                                                    const float* __restrict__ in_scale, void* __restrict__ out,
+                                                                    int tokens, int top, int N,
                                                                     int K) {
   constexpr bool GATE_UP = MODE == kGateUp, TOKENS = MODE != kDown;   // TOKENS: rows of x are tokens
   constexpr int kThreads = 256 * RG, kWaves = 4 * RG, kRows = kBigRows * RG;
@@ -611,12 +618,13 @@ __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* 
         const int rr = first + 16 * i + 4 * g + c;
         if (rr >= rows) continue;
         const int64_t dst = static_cast<int64_t>(list_dst[rr]) * N;
+        const float f = MODE != kDown && in_scale ? in_scale[list_dst[rr]] : 1.0f;
         if (GATE_UP) {
 #pragma unroll
           for (int j = 0; j < 2; ++j) {
             const int col = n0 + cw * 32 + 16 * j + n;
-            const float gt = acc[i][j][c];
-            if (col < N) static_cast<bf16*>(out)[dst + col] = from_float<bf16>(gt / (1.0f + expf(-gt)) * acc[i][j + 2][c]);
+            const float gt = f * acc[i][j][c];
+            if (col < N) static_cast<bf16*>(out)[dst + col] = from_float<bf16>(gt / (1.0f + expf(-gt)) * (f * acc[i][j + 2][c]));
           }
         } else {
 #pragma unroll
@@ -624,7 +632,7 @@ __global__ __launch_bounds__(256 * RG) void moe_expert_tiles_kernel(const bf16* 
             const int col = n0 + cw * 64 + 16 * j + n;
             if (col >= N) continue;
             if (MODE == kUp)
-              static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(acc[i][j][c]));
+              static_cast<bf16*>(out)[dst + col] = from_float<bf16>(squared_relu(f * acc[i][j][c]));
             else
               static_cast<float*>(out)[dst + col] = acc[i][j][c];
           }
@@ -714,8 +722,9 @@ extern "C" int arle_moe_identity(const void* x, long long x_stride, int dtype, c
   return launch_status();
 }
 
-// mode: kGateUp, kUp or kDown (see above); out [T * top, N] of `dtype`, or of float32 for kDown.
-extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w, const int* ids, void* out, int dtype,
+// mode: kGateUp, kUp or kDown (see above); in_scale float32 [T, top] or null; out [T * top, N] of `dtype`, or of float32 for kDown.
+extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w, const int* ids, const float* in_scale,
+                               void* out, int dtype,
                                int mode, int tokens, int experts, int top, int N, int K, void* stream) {
   if (tokens == 0) return 0;
   if (mode < 0 || mode > 2 || experts < 1 || experts > 65535 || top < 1 || N < 1 || K < 1 || (N + kEN - 1) / kEN > 65535)
@@ -729,7 +738,7 @@ extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w,
       const bf16* wb = static_cast<const bf16*>(w);
 #define ARLE_TILES(GU, RGS)                                                                                      \
   moe_expert_tiles_kernel<GU, RGS, 64><<<dim3((tokens + 256 * RGS - 1) / (256 * RGS), (N + bcols - 1) / bcols, experts), \
-                                         256 * RGS, 0, s>>>(xb, x_stride, wb, ids, out, tokens, top, N, K)
+                                         256 * RGS, 0, s>>>(xb, x_stride, wb, ids, in_scale, out, tokens, top, N, K)
 #define ARLE_TILES_MODE(RGS)              \
   do {                                    \
     if (mode == kGateUp)                  \
@@ -754,7 +763,7 @@ extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w,
     const dim3 fgrid((N + 63) / 64, experts);
 #define ARLE_FEW(MODE, MT)                                                                                            \
   moe_expert_few_kernel<MODE, MT><<<fgrid, 256, 0, s>>>(static_cast<const bf16*>(x), x_stride, static_cast<const bf16*>(w), \
-                                                        ids, out, tokens, top, N, K)
+                                                        ids, in_scale, out, tokens, top, N, K)
 #define ARLE_FEW_MT(MODE)          \
   do {                             \
     if (tokens <= 16)              \
@@ -772,7 +781,7 @@ extern "C" int arle_moe_expert(const void* x, long long x_stride, const void* w,
   const dim3 grid((tokens + kEM - 1) / kEM, (N + kEN - 1) / kEN, experts);
 #define ARLE_EXPERT(TT, GU)                                                                                         \
   moe_expert_kernel<TT, GU><<<grid, kExpertThreads, 0, s>>>(static_cast<const TT*>(x), x_stride,                    \
-                                                            static_cast<const TT*>(w), ids, out, tokens, top, N, K)
+                                                            static_cast<const TT*>(w), ids, in_scale, out, tokens, top, N, K)
 #define ARLE_EXPERT_MODE(TT)              \
   do {                                    \
     if (mode == kGateUp)                  \

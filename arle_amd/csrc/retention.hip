@@ -13,7 +13,7 @@
 //       o_i = g^(i+1) S_0^T q_i + sum_(j<=i) g^(i-j) (q_i . k_j) v_j,    S_n = g^n S_0 + sum_j g^(n-1-j) k_j v_j^T
 //     One kernel makes every chunk's own sum, one carries the state over the chunks (entry by entry, nothing but
 //     S <- g^n S + U), one makes the outputs; chunks and heads are all parallel.  The powers of g come from a table.
-#include "common.h"
+#include "chunks.h"
 
 namespace arle {
 
@@ -255,7 +255,7 @@ __global__ __launch_bounds__(kRetThreads) void retention_decode_kernel(
 // v_mfma_f32_16x16x4_f32: a lane gives A[i = lane % 16][k = lane / 16] and B[k][j = lane % 16]; the result's lane holds
 // rows 4 (lane / 16) .. + 3 of column lane % 16.  Operands that lie along k are read four at a time: the four products
 // of sixteen k take k = 4 g + j, j = 0..3, g = lane / 16, the same for both operands.
-constexpr int kChunk = 64;
+constexpr int kChunk = kChunkRows;
 constexpr int kSliceD = 64, kSliceRow = kSliceD + 4;    // a slice of q and k in LDS, a row padded by four
 
 __device__ __forceinline__ f32x4_t mfma4(const float4& a, const float4& b, f32x4_t acc) {
@@ -263,20 +263,6 @@ __device__ __forceinline__ f32x4_t mfma4(const float4& a, const float4& b, f32x4
   acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
   acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
-}
-
-struct ChunkAt {
-  int seg, row0, rows;   // the request's segment; the chunk's first row in the step; its rows (<= 64), 0: no such chunk
-};
-
-// The item-th chunk of all segments, in order.
-__device__ __forceinline__ ChunkAt find_chunk(const int* seg_row0, int segments, int item) {
-  for (int seg = 0; seg < segments; ++seg) {
-    const int a = seg_row0[seg], n = seg_row0[seg + 1] - a, chunks = (n + kChunk - 1) / kChunk;
-    if (item < chunks) return ChunkAt{seg, a + item * kChunk, min(kChunk, n - item * kChunk)};
-    item -= chunks;
-  }
-  return ChunkAt{0, 0, 0};
 }
 
 // Four entries d .. d + 3 of a row x of D entries turned by the angles at `cs`, `sn` (half entries a position).  The loads

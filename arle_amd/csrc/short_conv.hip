@@ -2,6 +2,7 @@
 // steps through a per-request state of the last taps-1 inputs.
 //
 //   y_t[c] = (ADD ? u_t[c] : 0) + sum_{j < taps} w[c][j] * u_(t - taps + 1 + j)[c],    u := input (+ bias)
+//   (out_bias: added to y in front of the silu.)
 //   (SILU: y <- y / (1 + exp(-y)) on the way out.  The entry point's `add_input` holds both: bit 0 ADD, bit 1 SILU.)
 //
 // The rows of one request are consecutive in the step; an input further back than the request's first row of
@@ -19,8 +20,8 @@ constexpr int kConvAdd = 1, kConvSilu = 2;
 __device__ __forceinline__ float conv_out(float y, int flags) { return (flags & kConvSilu) ? y / (1.0f + expf(-y)) : y; }
 
 __global__ void causal_conv_kernel(const void* __restrict__ u, long long u_stride, int u_dtype,
-                                   const void* __restrict__ bias, int bias_dtype, const void* __restrict__ w,
-                                   int w_dtype, const void* __restrict__ state, int state_dtype,
+                                   const void* __restrict__ bias, int bias_dtype, const void* __restrict__ out_bias,
+                                   int ob_dtype, const void* __restrict__ w, int w_dtype, const void* __restrict__ state, int state_dtype,
                                    const int* __restrict__ slot_of_token, void* __restrict__ out,
                                    long long out_stride, int out_dtype, int channels, int taps, int add_input) {
   const int t = blockIdx.x;
@@ -36,7 +37,7 @@ __global__ void causal_conv_kernel(const void* __restrict__ u, long long u_strid
   // rows of the same request right before this one in the step (at most taps-1 matter)
   int mine = 0;
   while (mine < taps - 1 && t - mine - 1 >= 0 && slot_of_token[t - mine - 1] == slot) ++mine;
-  float acc = (add_input & kConvAdd) ? now : 0.f;
+  float acc = ((add_input & kConvAdd) ? now : 0.f) + (out_bias ? load_as_float(out_bias, ob_dtype, c) : 0.f);
   acc = fmaf(load_as_float(w, w_dtype, static_cast<int64_t>(c) * taps + taps - 1), now, acc);
   for (int back = 1; back < taps; ++back) {
     float v;
@@ -56,7 +57,7 @@ __global__ void causal_conv_kernel(const void* __restrict__ u, long long u_strid
 // loads stands under a condition on data (which rows are the step's is the same for the whole workgroup).
 template <typename T, int TAPS>
 __global__ void causal_conv_vec_kernel(const T* __restrict__ u, long long u_stride, const T* __restrict__ bias,
-                                       const T* __restrict__ w, const T* __restrict__ state,
+                                       const T* __restrict__ out_bias, const T* __restrict__ w, const T* __restrict__ state,
                                        const int* __restrict__ slot_of_token, T* __restrict__ out, long long out_stride,
                                        int channels, int add_input) {
   const int t = blockIdx.x;
@@ -85,10 +86,11 @@ __global__ void causal_conv_vec_kernel(const T* __restrict__ u, long long u_stri
 #pragma unroll
     for (int i = 0; i < 4; ++i) wt[(4 * j + i) / TAPS][(4 * j + i) % TAPS] = e[i];
   }
-  float acc[4];
+  const float4 ob = out_bias ? ld4<T>(out_bias + c) : float4{0.f, 0.f, 0.f, 0.f};
+  float acc[4] = {ob.x, ob.y, ob.z, ob.w};
   const float now[4] = {in[0].x, in[0].y, in[0].z, in[0].w};
 #pragma unroll
-  for (int i = 0; i < 4; ++i) acc[i] = fmaf(wt[i][TAPS - 1], now[i], (add_input & kConvAdd) ? now[i] : 0.f);
+  for (int i = 0; i < 4; ++i) acc[i] = fmaf(wt[i][TAPS - 1], now[i], ((add_input & kConvAdd) ? now[i] : 0.f) + acc[i]);
 #pragma unroll
   for (int back = 1; back < TAPS; ++back) {
     const float v[4] = {in[back].x, in[back].y, in[back].z, in[back].w};
@@ -132,7 +134,7 @@ using namespace arle;
 // u [T, channels] rows u_stride apart; out likewise; w [channels, taps] or null (then out = u + bias);
 // state [slots, taps-1, channels]; slot_of_token int32 [T].
 extern "C" int arle_causal_conv(const void* u, long long u_stride, int u_dtype, const void* bias, int bias_dtype,
-                                const void* w, int w_dtype, const void* state, int state_dtype,
+                                const void* out_bias, int ob_dtype, const void* w, int w_dtype, const void* state, int state_dtype,
                                 const int* slot_of_token, void* out, long long out_stride, int out_dtype, int tokens,
                                 int channels, int taps, int add_input, void* stream) {
   if (tokens == 0 || channels == 0) return 0;
@@ -140,12 +142,12 @@ extern "C" int arle_causal_conv(const void* u, long long u_stride, int u_dtype, 
   hipStream_t s = static_cast<hipStream_t>(stream);
   const auto at16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   if (w && taps >= 2 && taps <= 4 && channels % 4 == 0 && u_stride % 4 == 0 && out_stride % 4 == 0 && at16(u) && at16(out) &&
-      at16(state) && u_dtype == out_dtype && w_dtype == out_dtype && state_dtype == out_dtype &&
-      (!bias || bias_dtype == out_dtype)) {
+      at16(state) && at16(w) && at16(bias) && at16(out_bias) && u_dtype == out_dtype && w_dtype == out_dtype && state_dtype == out_dtype &&
+      (!bias || bias_dtype == out_dtype) && (!out_bias || ob_dtype == out_dtype)) {
     dim3 vgrid(tokens, (channels / 4 + 255) / 256);
 #define ARLE_CONV(T, TAPS)                                                                                          \
   causal_conv_vec_kernel<T, TAPS><<<vgrid, 256, 0, s>>>(static_cast<const T*>(u), u_stride, static_cast<const T*>(bias), \
-                                                        static_cast<const T*>(w), static_cast<const T*>(state),       \
+                                                        static_cast<const T*>(out_bias), static_cast<const T*>(w), static_cast<const T*>(state), \
                                                         slot_of_token, static_cast<T*>(out), out_stride, channels,    \
                                                         add_input)
     if (out_dtype == kF32) {
@@ -158,7 +160,7 @@ extern "C" int arle_causal_conv(const void* u, long long u_stride, int u_dtype, 
   }
   dim3 grid(tokens, (channels + 255) / 256);
   causal_conv_kernel<<<grid, 256, 0, static_cast<hipStream_t>(stream)>>>(
-      u, u_stride, u_dtype, bias, bias_dtype, w, w_dtype, state, state_dtype, slot_of_token, out, out_stride,
+      u, u_stride, u_dtype, bias, bias_dtype, out_bias, ob_dtype, w, w_dtype, state, state_dtype, slot_of_token, out, out_stride,
       out_dtype, channels, taps, add_input);
   return launch_status();
 }

@@ -48,10 +48,11 @@ SOURCES = {
     "group_norm": "group_norm.hip",
     "latent_attention": "latent_attention.hip",
     "retention": "retention.hip",
+    "decay_scan": "decay_scan.hip",
     "host": "host/runtime.cpp",
 }
 HEADERS = ("common.h", "attention_static.h", "attention_args.h", "attention_stream.h", "attention_portions.h",
-           "attention_portions_dma.h", "addend.h")
+           "attention_portions_dma.h", "addend.h", "chunks.h", "lane_sums.h")
 HOST_LIBS = ("host",)   # plain C++: page pool, block tables, step packing
 HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-shared"]
 

@@ -1457,12 +1457,13 @@ CONV_MAX_TAPS = 16
 
 
 def causal_conv(u: torch.Tensor, weight, state, slot_of_token: torch.Tensor, *, bias=None, add_input: bool = False,
-                out_dtype: torch.dtype | None = None, silu: bool = False):
+                out_dtype: torch.dtype | None = None, silu: bool = False, out_bias=None):
     """y_t = (u_t if add_input) + sum_j weight[:, j] * u_(t - taps + 1 + j) per channel, over the rows of each request
     (consecutive in u) and, further back, over its state [slots, taps-1, C]; u counts with `bias` added.  weight
-    None: y = u + bias.  silu: y / (1 + exp(-y)) is what comes out.  The state is not changed: `conv_state_update`
+    None: y = u + bias.  out_bias [C]: added to y.  silu: y / (1 + exp(-y)) is
+    what comes out.  The state is not changed: `conv_state_update`
     does that once the step's rows are done."""
-    _gpu(u, weight, state, slot_of_token, bias)
+    _gpu(u, weight, state, slot_of_token, bias, out_bias)
     _rows(u, "u")
     tokens, channels = u.shape
     _i32(slot_of_token, "slot_of_token", tokens)
@@ -1477,10 +1478,14 @@ def causal_conv(u: torch.Tensor, weight, state, slot_of_token: torch.Tensor, *, 
                   and state.is_contiguous() and state.dtype in _CODES, "conv state must be [slots, taps-1, channels]")
     if bias is not None:
         _need(bias.shape == (channels,) and bias.is_contiguous() and bias.dtype in _CODES, "conv bias must be [channels]")
+    if out_bias is not None:
+        _need(weight is not None and out_bias.shape == (channels,) and out_bias.is_contiguous() and out_bias.dtype in _CODES,
+              "a bias behind the convolution must be [channels]")
     out = torch.empty((tokens, channels), dtype=out_dtype or u.dtype, device=u.device)
     has_state = weight is not None and taps > 1
     lib.call("arle_causal_conv", u.data_ptr(), u.stride(0), _code(u), _ptr(bias), _code(bias) if bias is not None else 0,
-             _ptr(weight), _code(weight) if weight is not None else 0, state.data_ptr() if has_state else 0,
+             _ptr(out_bias), _code(out_bias) if out_bias is not None else 0, _ptr(weight),
+             _code(weight) if weight is not None else 0, state.data_ptr() if has_state else 0,
              _code(state) if has_state else 0, slot_of_token.data_ptr(), out.data_ptr(), out.stride(0), _code(out),
              tokens, channels, taps, (1 if add_input else 0) | (2 if silu else 0), _stream())
     return out
@@ -1631,11 +1636,12 @@ def qkv_norm_store(q, k, v, *, num_q_heads: int, num_kv_heads: int, key_dim: int
 def attn_softcap_simt(q, out, k_pages, v_pages, block_table, positions, slot_of_token, *, num_q_heads: int,
                       num_kv_heads: int, key_dim: int, value_dim: int, page_size: int, scale: float,
                       softcap: float = 0.0, r1=None, r2=None, window: int = 0, chunk: int = 0, sink=None,
-                      keep_first: int = 0):
+                      keep_first: int = 0, out_scale: float = 1.0):
     """Causal attention of every row over its request's pages: scores scale (q . k), soft-capped (softcap > 0), less
     r1_h ln(1 + r2_h distance) (r1, r2 [heads] given), over the last `window` keys (0: all) and, with `chunk` > 0,
     over the keys of the row's own chunk of so many positions only; `sink` [heads]: exp(sink_h) joins the softmax's
-    denominator; `keep_first` (with a window): the request's first so many keys stay visible behind the window."""
+    denominator; `keep_first` (with a window): the request's first so many keys stay visible behind the window;
+    `out_scale`: a factor on the output, in 32 bits."""
     _need(keep_first >= 0 and (keep_first == 0 or window > 0), "kept first keys go with a window")
     _gpu(q, out, k_pages, v_pages, block_table, positions, slot_of_token, r1, r2, sink)
     _check_sink(sink, num_q_heads, window, chunk)
@@ -1659,7 +1665,7 @@ def attn_softcap_simt(q, out, k_pages, v_pages, block_table, positions, slot_of_
              v_pages.data_ptr(), _code(q), block_table.data_ptr(), block_table.shape[1], positions.data_ptr(),
              slot_of_token.data_ptr(), tokens, num_q_heads, num_kv_heads, key_dim, value_dim, page_size, float(scale),
              float(softcap), _ptr(r1), _ptr(r2), _code(r1) if r1 is not None else 0, int(window), int(chunk), _ptr(sink),
-             _code(sink) if sink is not None else 0, int(keep_first), _stream())
+             _code(sink) if sink is not None else 0, int(keep_first), float(out_scale), _stream())
     return out
 
 
@@ -1705,7 +1711,7 @@ def _softcap_lds_limit() -> int:
 def attn_softcap_mfma(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, seg_start, *, max_qlen: int,
                       num_q_heads: int, num_kv_heads: int, key_dim: int, value_dim: int, page_size: int, scale: float,
                       softcap: float = 0.0, r1=None, r2=None, window: int = 0, chunk: int = 0, sink=None,
-                      keep_first: int = 0):
+                      keep_first: int = 0, out_scale: float = 1.0):
     """`attn_softcap_simt` on the matrix cores, bfloat16: sixteen rows of a segment a wave, or (when every segment is
     one decoded row) one row's q heads of a kv head, sixteen at a time, a wave.  keep_first (with a window and no
     chunks): the request's first so many keys stay visible to rows whose window has passed them."""
@@ -1746,7 +1752,7 @@ def attn_softcap_mfma(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot,
              seg_start.data_ptr(), segments, row_blocks, 1 if heads_mode else 0, num_q_heads, num_kv_heads, key_dim,
              value_dim, page_size, float(scale), float(softcap), _ptr(r1), _ptr(r2),
              _code(r1) if r1 is not None else 0, int(window), int(chunk), _ptr(sink),
-             _code(sink) if sink is not None else 0, int(keep_first), _stream())
+             _code(sink) if sink is not None else 0, int(keep_first), float(out_scale), _stream())
     return out
 
 
@@ -1802,6 +1808,13 @@ def wide_norm_store(q, k, v, *, num_q_heads: int, num_kv_heads: int, key_dim: in
 NORM_ADD_MAX_WIDTH = 16384
 
 
+class EveryRow:
+    """An addend that is the same row for every token: float32 [W]."""
+
+    def __init__(self, row: torch.Tensor):
+        self.row = row
+
+
 class Scaled:
     """An addend with one factor a row: `delta` (float32 [T, W] or a stack [S, T, W] of partial sums) times `factor`
     (float32 [T])."""
@@ -1813,22 +1826,31 @@ class Scaled:
 def _addend_tensors(term) -> tuple:
     if isinstance(term, Scaled):
         return (term.delta, term.factor)
-    return term if isinstance(term, tuple) else (term,)
+    if isinstance(term, EveryRow):
+        return (term.row,)
+    return tuple(t for t in term if t is not None) if isinstance(term, tuple) else (term,)
 
 
 def _addend_args(term, rows: int, width: int):
     """(pointer, parts, part stride, row stride, factors' pointer, their stride a row and a part) of one float32 addend:
-    a tensor [T, W]; a stack [S, T, W] of partial sums; (outputs [T, n, W], weights [T, n]); or a `Scaled` one."""
+    a tensor [T, W]; a stack [S, T, W] of partial sums; (outputs [T, n, W], weights [T, n] or None: all 1); a `Scaled` one;
+    or `EveryRow`."""
     if term is None:
         return (0, 0, 0, 0, 0, 0, 0)
     if isinstance(term, Scaled):
         _need(term.factor.shape == (rows,) and term.factor.dtype == torch.float32 and term.factor.is_contiguous(),
               "an addend's factor must be contiguous float32 [T]")
         return _addend_args(term.delta, rows, width)[:4] + (term.factor.data_ptr(), 1, 0)
+    if isinstance(term, EveryRow):
+        _need(term.row.shape == (width,) and term.row.dtype == torch.float32 and term.row.is_contiguous(),
+              "a row for every token must be contiguous float32 [W]")
+        return (term.row.data_ptr(), 1, 0, 0, 0, 0, 0)
     if isinstance(term, tuple):
         outs, weights = term
         _need(outs.dim() == 3 and outs.shape[0] == rows and outs.shape[2] == width and outs.is_contiguous()
               and outs.dtype == torch.float32, "weighted outputs must be contiguous float32 [T, n, W]")
+        if weights is None:
+            return (outs.data_ptr(), outs.shape[1], width, outs.shape[1] * width, 0, 0, 0)
         _need(weights.shape == outs.shape[:2] and weights.dtype == torch.float32 and weights.is_contiguous(),
               "their weights must be contiguous float32 [T, n]")
         return (outs.data_ptr(), outs.shape[1], width, outs.shape[1] * width, weights.data_ptr(), outs.shape[1], 1)
@@ -1894,8 +1916,29 @@ def group_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, o
     for i in range(GROUP_NORM_MAX_TERMS):
         args += _addend_args(terms[i] if i < len(terms) else None, x.shape[0], width)
     lib.call("arle_group_norm", x.data_ptr(), _code(x), x.stride(0), x.data_ptr() if terms and rows is None else 0, *args,
-             weight.data_ptr(), _code(weight), out.data_ptr(), _code(out), _ptr(rows), n_rows, width, int(groups), float(eps),
-             _stream())
+             weight.data_ptr(), _code(weight), out.data_ptr(), width, _code(out), _ptr(rows), n_rows, width, int(groups),
+             float(eps), 0, _stream())
+    return out
+
+
+def add_terms_into(x: torch.Tensor, terms, out: torch.Tensor) -> torch.Tensor:
+    """out [T, W] (a view whose rows may lie further apart) = x + the sum of up to three `terms` (see `_addend_args`), in
+    out's type; x (float32 [T, W]) keeps its values."""
+    terms = [t.float() if torch.is_tensor(t) and t.dtype == torch.bfloat16 else t for t in terms]
+    _need(len(terms) <= GROUP_NORM_MAX_TERMS, f"at most {GROUP_NORM_MAX_TERMS} terms are added")
+    _gpu(x, out, *[y for t in terms for y in _addend_tensors(t)])
+    _rows(out, "out")
+    _need(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "x must be contiguous float32 [T, W]")
+    rows, width = x.shape
+    _need(out.shape == x.shape and out.dtype in _CODES and 0 < width <= GROUP_NORM_MAX_WIDTH,
+          f"out must be [T, W] with widths up to {GROUP_NORM_MAX_WIDTH}")
+    if rows == 0:
+        return out
+    args = []
+    for i in range(GROUP_NORM_MAX_TERMS):
+        args += _addend_args(terms[i] if i < len(terms) else None, rows, width)
+    lib.call("arle_group_norm", x.data_ptr(), 0, x.stride(0), 0, *args, x.data_ptr(), 0, out.data_ptr(), out.stride(0),
+             _code(out), 0, rows, width, 1, 0.0, 1, _stream())
     return out
 
 
@@ -2138,13 +2181,13 @@ def moe_identity(x, ids, outs, first: int):
     return outs
 
 
-def moe_expert(x, w, ids, which: int):
+def moe_expert(x, w, ids, which: int, in_scale=None):
     """The chosen experts' products.  MOE_GATE_UP: x [T, K], w [experts, 2N, K] (gate rows, then up rows) ->
     silu(gate) * up as [T * top, N] of x's type, row t * top + k for token t's k-th choice.  MOE_UP: the same for
     w [experts, N, K] without a gate -> max(up, 0)^2.  MOE_DOWN: x [T * top, K], w [experts, N, K] -> float32
-    [T * top, N]."""
+    [T * top, N].  in_scale (not with MOE_DOWN): float32 [T, top], a factor on the input of each chosen expert."""
     _need(which in (MOE_DOWN, MOE_GATE_UP, MOE_UP), "unknown expert product")
-    _gpu(x, w, ids)
+    _gpu(x, w, ids, in_scale)
     _rows(x, "x")
     _need(ids.dtype == torch.int32 and ids.dim() == 2 and ids.is_contiguous(), "ids must be contiguous int32 [T, top]")
     tokens, top = ids.shape
@@ -2152,9 +2195,11 @@ def moe_expert(x, w, ids, which: int):
           "w must be contiguous [experts, N, K] of x's type")
     _need(x.shape[0] == (tokens * top if which == MOE_DOWN else tokens), "x has a row a token (up) or a row a choice (down)")
     _need(which != MOE_GATE_UP or w.shape[1] % 2 == 0, "gate|up has an even number of rows")
+    _need(in_scale is None or (which != MOE_DOWN and in_scale.shape == ids.shape and in_scale.dtype == torch.float32
+                               and in_scale.is_contiguous()), "in_scale must be contiguous float32 [T, top]")
     N = w.shape[1] // 2 if which == MOE_GATE_UP else w.shape[1]
     out = torch.empty((tokens * top, N), dtype=torch.float32 if which == MOE_DOWN else x.dtype, device=x.device)
-    lib.call("arle_moe_expert", x.data_ptr(), x.stride(0), w.data_ptr(), ids.data_ptr(), out.data_ptr(), _code(x),
+    lib.call("arle_moe_expert", x.data_ptr(), x.stride(0), w.data_ptr(), ids.data_ptr(), _ptr(in_scale), out.data_ptr(), _code(x),
              int(which), tokens, w.shape[0], top, N, x.shape[1], _stream())
     return out
 
@@ -2409,7 +2454,7 @@ def gated_delta_output(o, gate, weight, eps: float, *, heads: int, value_dim: in
     _need(heads <= _GRID_Y_MAX, "too many heads")
     out = torch.empty((tokens, width), dtype=gate.dtype, device=o.device)
     lib.call("arle_gated_delta_output", o.data_ptr(), gate.data_ptr(), gate.stride(0), _code(gate), weight.data_ptr(),
-             _code(weight), float(eps), out.data_ptr(), tokens, heads, value_dim, int(act), _stream())
+             _code(weight), float(eps), out.data_ptr(), _code(out), tokens, heads, value_dim, int(act), _stream())
     return out
 
 
@@ -2505,4 +2550,103 @@ def retention_chunks(y, powers, s_state, seg_row0, seg_slot, eps: float, out_dty
              _ptr(sin) if rotary_dims else 0, int(rotary_dims), positions.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(),
              powers.data_ptr(), s_state.data_ptr(), segments, items, work.data_ptr(), float(eps), out.data_ptr(), _code(out),
              H, D, Dv, _stream())
+    return out
+
+
+# ------------------------------------------------- linear attention with decays made from the tokens
+
+DECAY_SCAN_MAX_KEY_DIM = 256
+DECAY_CHUNK = 64
+
+
+def _f32_vector(t, n: int, name: str) -> None:
+    _need(t.shape == (n,) and t.dtype == torch.float32 and t.is_contiguous() and t.is_cuda, f"{name} must be contiguous float32 [{n}]")
+
+
+def _check_segments(s_state, seg_row0, seg_slot, H: int, D: int, Dv: int) -> int:
+    _gpu(s_state, seg_row0, seg_slot)
+    _need(0 < D <= DECAY_SCAN_MAX_KEY_DIM and 0 < Dv and 0 < H <= _GRID_Y_MAX, f"key sizes up to {DECAY_SCAN_MAX_KEY_DIM}")
+    _need(s_state.dim() == 4 and tuple(s_state.shape[1:]) == (H, D, Dv) and s_state.dtype == torch.float32
+          and s_state.is_contiguous(), "the state is float32 [slots, heads, D, Dv]")
+    _i32(seg_slot, "seg_slot")
+    _i32(seg_row0, "seg_row0", seg_slot.numel() + 1)
+    return seg_slot.numel()
+
+
+def state_space_rows(x, B, C, dt, a_log, dt_bias, skip, s_state, seg_row0, seg_slot, *, heads: int, groups: int, state: int,
+                     value_dim: int):
+    """The state-space recurrence over the rows of every segment, row by row (see csrc/decay_scan.hip): x [T, heads * P], B
+    and C [T, groups * N] of one type, dt float32 [T, >= heads] (raw step sizes), a_log, dt_bias, skip float32 [heads],
+    s_state float32 [slots, heads, N, P].  Returns S^T C + skip x, float32 [T, heads * P]."""
+    H, G, N, P = heads, groups, state, value_dim
+    segments = _check_segments(s_state, seg_row0, seg_slot, H, N, P)
+    tokens = x.shape[0]
+    _need(G > 0 and H % G == 0, "heads must be a multiple of the groups")
+    for name, t, width in (("x", x, H * P), ("B", B, G * N), ("C", C, G * N)):
+        _gpu(t)
+        _rows(t, name)
+        _need(t.shape == (tokens, width) and t.dtype == x.dtype and t.dtype in _CODES, f"{name} must be [T, {width}] of one type")
+    _gpu(dt)
+    _rows(dt, "dt")
+    _need(dt.dtype == torch.float32 and dt.shape[0] == tokens and dt.shape[1] >= H, "dt must be float32 [T, >= heads]")
+    for name, t in (("a_log", a_log), ("dt_bias", dt_bias), ("skip", skip)):
+        _f32_vector(t, H, name)
+    out = torch.empty((tokens, H * P), dtype=torch.float32, device=x.device)
+    lib.call("arle_decay_scan", C.data_ptr(), C.stride(0), B.data_ptr(), B.stride(0), x.data_ptr(), x.stride(0), _code(x),
+             dt.data_ptr(), dt.stride(0), 0, a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(), 1.0, s_state.data_ptr(),
+             seg_row0.data_ptr(), seg_slot.data_ptr(), segments, out.data_ptr(), H, G, N, P, _stream())
+    return out
+
+
+def gated_group_norm(y, z, weight, eps: float, *, groups: int, factor: float, out):
+    """out [T, W] (a view of z's type) = y * silu(z), each of `groups` equal runs of entries divided by its own root mean
+    square, times weight (float32 [W]) and `factor`; y float32 [T, W]."""
+    _gpu(y, z, out)
+    tokens, width = y.shape
+    _need(y.dtype == torch.float32 and y.is_contiguous(), "y must be contiguous float32 [T, W]")
+    for name, t in (("z", z), ("out", out)):
+        _rows(t, name)
+        _need(t.shape == (tokens, width) and t.dtype == z.dtype and t.dtype in _CODES, f"{name} must be [T, W] of one type")
+    _f32_vector(weight, width, "weight")
+    _need(groups >= 1 and width % groups == 0 and width // groups <= 16384 and groups <= _GRID_Y_MAX, "groups out of range")
+    lib.call("arle_gated_group_norm", y.data_ptr(), z.data_ptr(), z.stride(0), _code(z), weight.data_ptr(), float(eps),
+             float(factor), out.data_ptr(), out.stride(0), tokens, width, int(groups), _stream())
+    return out
+
+
+def _gated_linear_check(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, H: int, D: int, Dv: int) -> int:
+    """The narrow middle's width."""
+    _check_segments(s_state, seg_row0, seg_slot, H, D, Dv)
+    _gpu(y, a2)
+    _need(a2.dim() == 2 and a2.shape[0] == H * D and a2.is_contiguous() and a2.dtype in _CODES, "a2 must be contiguous [heads * D, rank]")
+    rank, width = a2.shape[1], 2 * H * (D + Dv)
+    _need(y.dim() in (2, 3) and y.shape[-1] >= width + rank and y.dtype == torch.float32 and y.is_contiguous(),
+          "y must be contiguous float32 [T, q | k | v | gate | middle] (or a stack of partial sums of it)")
+    _f32_vector(a2_bias, H * D, "a2_bias")
+    _f32_vector(norm, Dv, "norm")
+    return rank
+
+
+def gated_linear_rows(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, tau: float, heads: int,
+                      key_dim: int, value_dim: int):
+    """Gated linear attention over the rows of every segment, row by row (see csrc/decay_scan.hip): y float32
+    [T, q | k | v | gate | middle | ...], a2 [heads * D, rank] and a2_bias float32 [heads * D] of the decays, norm float32
+    [Dv].  Returns [T, heads * Dv] of `out_dtype`, normed and gated."""
+    H, D, Dv = heads, key_dim, value_dim
+    rank = _gated_linear_check(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, H, D, Dv)
+    _need(y.dim() == 2, "the rows' form takes whole sums")
+    T, segments = y.shape[0], seg_slot.numel()
+    qw, vw = H * D, H * Dv
+    q, k, v, g, m = (y[:, a:b] for a, b in ((0, qw), (qw, 2 * qw), (2 * qw, 2 * qw + vw), (2 * qw + vw, 2 * qw + 2 * vw),
+                                            (2 * qw + 2 * vw, 2 * qw + 2 * vw + rank)))
+    decay = torch.empty((T, qw), dtype=torch.float32, device=y.device)
+    lib.call("arle_decay_gates", m.data_ptr(), y.stride(0), a2.data_ptr(), _code(a2), a2_bias.data_ptr(), 1.0 / tau,
+             seg_row0.data_ptr(), segments, 0, 0, decay.data_ptr(), T, rank, qw, _stream())
+    o = torch.empty((T, vw), dtype=torch.float32, device=y.device)
+    lib.call("arle_decay_scan", q.data_ptr(), y.stride(0), k.data_ptr(), y.stride(0), v.data_ptr(), y.stride(0), 0,
+             decay.data_ptr(), qw, 1, 0, 0, 0, float(D) ** -0.5, s_state.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(),
+             segments, o.data_ptr(), H, H, D, Dv, _stream())
+    out = torch.empty((T, vw), dtype=out_dtype, device=y.device)
+    lib.call("arle_gated_delta_output", o.data_ptr(), g.data_ptr(), y.stride(0), 0, norm.data_ptr(), 0, float(eps),
+             out.data_ptr(), _code(out), T, H, Dv, 0, _stream())
     return out

@@ -12,9 +12,9 @@ import sys
 
 from ..kernels import ops
 from ..parts import base  # noqa: F401  (registries)
-from ..parts import (attention, block, embedding, feed_forward, gated_delta, hyper, latent_attention,  # noqa: F401  registers the stock parts
-                     mixer_pair, mlstm, moe, norm, position, retention, rotary_attention, short_conv, softcap_attention,
-                     token_side, wide_norm_attention)
+from ..parts import (attention, block, embedding, feed_forward, gated_delta, gated_linear, hyper, latent_attention,  # noqa: F401  registers the stock parts
+                     loop, mixer_pair, mlstm, moe, norm, position, retention, rotary_attention, short_conv, softcap_attention,
+                     state_space, token_side, wide_norm_attention)
 from ..parts.base import Runtime, build_part, expected_tensors, lookup
 from ..parts.spec import ModelSpec
 
@@ -84,8 +84,10 @@ def debug_dump(residual, delta, label: str) -> None:
         factor = 1.0
         if isinstance(term, ops.Scaled):
             term, factor = term.delta, term.factor[-1]
-        if isinstance(term, tuple):     # outputs of experts and their weights
-            row = row + (term[0][-1] * term[1][-1][:, None]).sum(0)
+        if isinstance(term, ops.EveryRow):
+            row = row + term.row
+        elif isinstance(term, tuple):     # outputs of experts and their weights (None: all 1)
+            row = row + (term[0][-1] if term[1] is None else term[0][-1] * term[1][-1][:, None]).sum(0)
         else:
             row = row + (term.float().sum(0) if term.dim() == 3 else term.float())[-1] * factor
         if bias is not None:

@@ -6,7 +6,7 @@
     over the chosen z alone, times scale;
     expert: down(silu(gate h) * (up h)), or (form "squared_relu") down(max(up h, 0)^2), no biases; the last `identity` outputs of the router stand for experts without
     tensors that hand back h itself;
-    out = sum over the chosen experts of weight_e expert_e(h)  +  shared(h), or with `shared_gate` sigmoid(W_s h) shared(h),
+    out = sum over the chosen experts of weight_e expert_e(h) (weigh "input": of expert_e(weight_e h))  +  shared(h), or with `shared_gate` sigmoid(W_s h) shared(h),
     one number a token
 
 The router's kernel leaves the chosen experts and their weights on the GPU; the experts' kernel finds, workgroup by
@@ -32,7 +32,7 @@ class SigmoidMoE(Part):
     """params: hidden_size, experts (those with tensors), top, expert_size, scale, correction (bool),
     shared_size (int | None), shared_gate (bool), form ("gated_silu", the default, or "squared_relu": of the experts and
     the shared one), bias (bool: of the router), score ("sigmoid", the default, "softmax" or "softmax_chosen"), normalize (bool, default True),
-    groups (default 1), keep_groups (default 1), identity (default 0: router outputs behind the experts' that stand
+    weigh ("output", the default, or "input": what a chosen expert's weight multiplies), groups (default 1), keep_groups (default 1), identity (default 0: router outputs behind the experts' that stand
     for experts which hand back their input; groups and the softmax run over experts and these together)."""
 
     graph_safe = True  # launches depend on shapes only; what a token chose is read on the GPU
@@ -92,6 +92,11 @@ class SigmoidMoE(Part):
         self.correction = tensors.get("correction")
         self.bias = tensors.get("bias")
         self.shared_gate = tensors.get("shared_gate")
+        self.weigh = params.get("weigh") or "output"
+        if self.weigh not in ("output", "input"):
+            raise ValueError("an expert's weight multiplies its output or its input")
+        if self.weigh == "input" and self.identity:
+            raise ValueError("experts that hand back their input take their weight on the output")
         E = self.E
         self.gated = self._form(params) == "gated_silu"
         names = ("gate", "up", "down") if self.gated else ("up", "down")
@@ -107,18 +112,19 @@ class SigmoidMoE(Part):
             raise ValueError("a shared expert's gate without a shared expert")
 
     def forward(self, x):
-        """x [T, H] -> the addends of the output: [(outputs float32 [T, top, H], weights float32 [T, top])] and, with
+        """x [T, H] -> the addends of the output: [(outputs float32 [T, top, H], weights float32 [T, top] or None)] and, with
         a shared expert, its output (float32 [T, H] or a float32 stack of partial sums; with a gate, `ops.Scaled`)."""
         w_dtype = self.up.dtype
         xe = x if x.dtype == w_dtype else x.to(w_dtype)
         ids, weights, *gate = ops.moe_route(x, self.router, self.correction, top=self.top, scale=self.scale,
                                             score=self.score, groups=self.groups, keep_groups=self.keep_groups,
                                             normalize=self.normalize, bias=self.bias, shared_gate=self.shared_gate)
-        act = ops.moe_expert(xe, self.up, ids, ops.MOE_GATE_UP if self.gated else ops.MOE_UP)
+        on_input = self.weigh == "input"
+        act = ops.moe_expert(xe, self.up, ids, ops.MOE_GATE_UP if self.gated else ops.MOE_UP, weights if on_input else None)
         outs = ops.moe_expert(act, self.down, ids, ops.MOE_DOWN)
         if self.identity:
             ops.moe_identity(x, ids, outs, self.E)
-        terms = [(outs.view(x.shape[0], self.top, -1), weights)]
+        terms = [(outs.view(x.shape[0], self.top, -1), None if on_input else weights)]
         if self.shared is not None:
             y = self.shared.forward(x)
             terms.append(ops.Scaled(y, gate[0]) if gate else y)

@@ -34,7 +34,8 @@ SINKS = (None, "zero", "learned")
 class RotaryAttention(Part):
     """params: hidden_size, num_q_heads, num_kv_heads, key_dim, value_dim, eps, scale, softcap (0: none),
     qk_norm (one of QK_NORMS), sink (one of SINKS), position (PartSpec of a position part, or None),
-    window (int | None)."""
+    window (int | None), project_out (bool, default True; False: one of a joined pair of mixers, which owns the products in
+    front and behind, and calls `heads`)."""
 
     graph_safe = True  # positions, slots and lengths are read on the GPU; launches depend on shapes only
 
@@ -49,11 +50,17 @@ class RotaryAttention(Part):
         qw, kw, vw = cls._widths(params)
         decl = {"q": WeightDecl((qw, h)), "k": WeightDecl((kw, h)), "v": WeightDecl((vw, h)),
                 "o": WeightDecl((h, params["num_q_heads"] * params["value_dim"]))}
+        if not params.get("project_out", True):
+            del decl["o"]
         if params.get("qk_norm") == "weighted_before":
             decl.update(q_norm=WeightDecl((params["key_dim"],), init="ones"), k_norm=WeightDecl((params["key_dim"],), init="ones"))
         if params.get("sink") == "learned":
             decl["sink"] = WeightDecl((params["num_q_heads"],), init="normal")
         return decl
+
+    @classmethod
+    def output_width(cls, params):
+        return params["num_q_heads"] * params["value_dim"]
 
     @classmethod
     def children(cls, params):
@@ -87,7 +94,8 @@ class RotaryAttention(Part):
         if len({t.dtype for t in mats}) != 1:
             raise ValueError("q, k and v projections must be stored in one type")
         self.widths = self._widths(params)
-        self.proj = Linear(torch.cat(mats, dim=0).contiguous(), rt.weight_tiles)
+        self.in_weight = torch.cat(mats, dim=0).contiguous()
+        self.in_width, self.heads_width = int(self.in_weight.shape[0]), self.nq * self.Dv
         self.q_norm, self.k_norm = tensors.get("q_norm"), tensors.get("k_norm")
         self.sink = None
         if self.sink_kind == "learned":
@@ -95,21 +103,29 @@ class RotaryAttention(Part):
         elif self.sink_kind == "zero":
             self.sink = torch.zeros(self.nq, dtype=torch.float32, device=rt.device)
         self.position = (children or {}).get("position")
-        self.o = Linear(tensors["o"], rt.weight_tiles)
+        self.proj = self.o = None
+        if params.get("project_out", True):
+            self.proj, self.o = Linear(self.in_weight, rt.weight_tiles), Linear(tensors["o"], rt.weight_tiles)
 
     def products(self):
-        if self.proj.weight.dtype != torch.bfloat16:
+        if self.proj is None or self.proj.weight.dtype != torch.bfloat16:
             return []
         return [("qkv", self.proj.out_features, self.proj.in_features, False, None),
                 ("o", self.o.out_features, self.o.in_features, False, "norm")]
 
     def forward(self, x, batch, cache):
         """x [T, H] -> float32 [T, H], or a float32 stack [S, T, H] to be added in order (see Linear)."""
+        out = torch.empty((x.shape[0], self.heads_width), dtype=x.dtype, device=x.device)
+        self.heads(self.proj(x), x, batch, cache, out)
+        return self.o(out, out_dtype=torch.float32, partials_ok=True)   # it goes into the 32-bit residual unrounded
+
+    def heads(self, y, x, batch, cache, out, factor: float = 1.0):
+        """From y [T, in_width], the product of `in_weight` with x (q is changed in place), what the output projection
+        reads, times `factor`, into the view out [T, heads_width]."""
         if not cache.writes:
             raise ValueError("this attention keeps keys and values of its own")
         Q, K, _ = self.widths
-        y = self.proj(x)
-        q, k, v = y[:, :Q], y[:, Q:Q + K], y[:, Q + K:]
+        q, k, v = y[:, :Q], y[:, Q:Q + K], y[:, Q + K:self.in_width]
         cos = sin = None
         rotary_dim, interleaved = 0, False
         if self.position is not None:
@@ -121,8 +137,6 @@ class RotaryAttention(Part):
                              interleaved=interleaved, positions=batch.positions, slot_of_token=batch.slot_of_token,
                              block_table=cache.block_table, k_pages=cache.pages["k"], v_pages=cache.pages["v"],
                              page_size=cache.page_size)
-        out = torch.empty((x.shape[0], self.nq * self.Dv), dtype=x.dtype, device=x.device)
         softcap_attention(q, out, cache, batch, num_q_heads=self.nq, num_kv_heads=self.nkv, key_dim=self.Dk,
                           value_dim=self.Dv, scale=self.scale, softcap=self.softcap, r1=None, r2=None,
-                          window=self.window, sink=self.sink)
-        return self.o(out, out_dtype=torch.float32, partials_ok=True)   # it goes into the 32-bit residual unrounded
+                          window=self.window, sink=self.sink, out_scale=factor)

@@ -15,11 +15,13 @@ from .base import Part, WeightDecl, register
 
 
 class ShortConv:
-    """One convolution weight [channels, taps] (None: no convolution) with an optional bias on its input."""
+    """One convolution weight [channels, taps] (None: no convolution) with an optional bias on its input (`bias`) or
+    behind it (`out_bias`)."""
 
-    def __init__(self, weight, bias=None):
+    def __init__(self, weight, bias=None, out_bias=None):
         self.weight = weight
         self.bias = bias
+        self.out_bias = out_bias
         self.taps = int(weight.shape[1]) if weight is not None else 1
 
     @staticmethod
@@ -30,7 +32,8 @@ class ShortConv:
     def __call__(self, u, batch, state_view, add_input: bool = False, silu: bool = False):
         """The convolution of the step's rows (with `silu`, its silu); the requests' states move on by the rows they brought."""
         state = state_view.state if (state_view is not None and self.taps > 1) else None
-        y = ops.causal_conv(u, self.weight, state, batch.slot_of_token, bias=self.bias, add_input=add_input, silu=silu)
+        y = ops.causal_conv(u, self.weight, state, batch.slot_of_token, bias=self.bias, add_input=add_input, silu=silu,
+                            out_bias=self.out_bias)
         if state is not None:
             ops.conv_state_update(u, state, batch.seg_row0, batch.seg_slot, bias=self.bias)
         return y
