@@ -108,16 +108,46 @@ __global__ __launch_bounds__(kWave) void rotary_qkv_store_kernel(
   }
 }
 
+// What a step of decoded rows has in front of it: the 32-bit partial sums of the product that made q, k and v, a row's columns
+// q | k | v, added in order and rounded on the way in.
+struct QkvSums {
+  const float* p;
+  int parts;
+  long long part_stride, row_stride;
+};
+
+// Eight consecutive entries of the sums' column `col`, rounded to bfloat16.
+__device__ __forceinline__ uint4 summed8(const QkvSums& a, int64_t t, int col) {
+  float s[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  const float* p = a.p + t * a.row_stride + col;
+  for (int i0 = 0; i0 < a.parts; i0 += 4) {
+    float4 e[4][2];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const float* part = p + min(i0 + u, a.parts - 1) * a.part_stride;
+      e[u][0] = ld4<float>(part);
+      e[u][1] = ld4<float>(part + 4);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const bool in = i0 + u < a.parts;
+      s[0] += in ? e[u][0].x : 0.f; s[1] += in ? e[u][0].y : 0.f; s[2] += in ? e[u][0].z : 0.f; s[3] += in ? e[u][0].w : 0.f;
+      s[4] += in ? e[u][1].x : 0.f; s[5] += in ? e[u][1].y : 0.f; s[6] += in ? e[u][1].z : 0.f; s[7] += in ? e[u][1].w : 0.f;
+    }
+  }
+  return uint4{pack_bf16x2(s[0], s[1]), pack_bf16x2(s[2], s[3]), pack_bf16x2(s[4], s[5]), pack_bf16x2(s[6], s[7])};
+}
+
 // LPH: lanes of a head (a power of two, 8 LPH >= Dk).  A row's lanes: (nq + nkv) LPH for q and k, then Dv / 8 for
 // every head of v.
-template <int LPH>
+template <int LPH, bool SUMS>
 __global__ __launch_bounds__(256) void rotary_qkv_store_x8_kernel(
     bf16* __restrict__ q, long long q_stride, const bf16* __restrict__ k, long long k_stride, const bf16* __restrict__ v,
     long long v_stride, const void* __restrict__ q_weight, const void* __restrict__ k_weight, int w_dtype, float eps,
     int unit_after, const float* __restrict__ cos_t, const float* __restrict__ sin_t, int R, int interleaved,
     const int* __restrict__ positions, const int* __restrict__ slot_of_token, const int* __restrict__ block_table,
     int table_stride, bf16* __restrict__ k_pages, bf16* __restrict__ v_pages, int nq, int nkv, int Dk, int Dv,
-    int page_size) {
+    int page_size, const QkvSums sums) {
   const int64_t t = blockIdx.x;
   const int idx = blockIdx.y * 256 + threadIdx.x, lane = threadIdx.x % kWave;
   const int qk_lanes = (nq + nkv) * LPH, qk_padded = (qk_lanes + kWave - 1) / kWave * kWave, v_units = Dv / 8;
@@ -127,7 +157,9 @@ __global__ __launch_bounds__(256) void rotary_qkv_store_x8_kernel(
     const int e = idx - qk_padded;
     if (e >= nkv * v_units) return;
     const int g = e / v_units, u = e % v_units;
-    const uint4 raw = *reinterpret_cast<const uint4*>(v + t * v_stride + g * Dv + 8 * u);
+    uint4 raw;
+    if constexpr (SUMS) raw = summed8(sums, t, (nq + nkv) * Dk + g * Dv + 8 * u);
+    else raw = *reinterpret_cast<const uint4*>(v + t * v_stride + g * Dv + 8 * u);
     uint16_t* dst = reinterpret_cast<uint16_t*>(v_pages) +
                     ((static_cast<int64_t>(page) * nkv + g) * Dv + 8 * u) * page_size + pos % page_size;
     const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
@@ -139,11 +171,16 @@ __global__ __launch_bounds__(256) void rotary_qkv_store_x8_kernel(
   const int y = min(idx / LPH, nq + nkv - 1), u = idx % LPH;
   const bool is_q = y < nq, live = idx < qk_lanes && 8 * u < Dk;
   const int g = is_q ? y : y - nq;
-  const bf16* src = is_q ? q + t * q_stride + g * Dk : k + t * k_stride + g * Dk;
   const void* weight = is_q ? q_weight : k_weight;
   float x[8];
   {
-    const uint4 raw = *reinterpret_cast<const uint4*>(src + (live ? 8 * u : 0));
+    uint4 raw;
+    if constexpr (SUMS) {
+      raw = summed8(sums, t, y * Dk + (live ? 8 * u : 0));
+    } else {
+      const bf16* src = is_q ? q + t * q_stride + g * Dk : k + t * k_stride + g * Dk;
+      raw = *reinterpret_cast<const uint4*>(src + (live ? 8 * u : 0));
+    }
     const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -231,11 +268,11 @@ extern "C" int arle_rotary_qkv_store(void* q, long long q_stride, const void* k,
     if ((lanes + 255) / 256 <= 65535) {
       const dim3 grid(tokens, (lanes + 255) / 256);
 #define ARLE_ROT_X8(LPH)                                                                                             \
-  rotary_qkv_store_x8_kernel<LPH><<<grid, 256, 0, s>>>(                                                              \
+  rotary_qkv_store_x8_kernel<LPH, false><<<grid, 256, 0, s>>>(                                                       \
       static_cast<bf16*>(q), q_stride, static_cast<const bf16*>(k), k_stride, static_cast<const bf16*>(v), v_stride, \
       q_weight, k_weight, w_dtype, eps, unit_after, static_cast<const float*>(cos_t),                                \
       static_cast<const float*>(sin_t), rotary_dim, interleaved, positions, slot_of_token, block_table,              \
-      table_stride, static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), nq, nkv, Dk, Dv, page_size)
+      table_stride, static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), nq, nkv, Dk, Dv, page_size, QkvSums{})
       switch (lph) {
         case 1: ARLE_ROT_X8(1); break;
         case 2: ARLE_ROT_X8(2); break;
@@ -263,5 +300,45 @@ extern "C" int arle_rotary_qkv_store(void* q, long long q_stride, const void* k,
         rotary_dim, interleaved, positions, slot_of_token, block_table, table_stride, static_cast<bf16*>(k_pages),
         static_cast<bf16*>(v_pages), nq, nkv, Dk, Dv, page_size);
   }
+  return launch_status();
+}
+
+// The same from the 32-bit partial sums of the product (columns q | k | v from sums on), bfloat16: q goes to q_out [T, nq * Dk].
+// Dk and Dv multiples of 8, Dk up to 512, pointers 16-byte aligned, strides multiples of 4; the halves pairing rotates a
+// multiple of 16 entries.
+extern "C" int arle_rotary_sums_store(const float* sums, int parts, long long part_stride, long long row_stride, void* q_out,
+                                      const void* q_weight, const void* k_weight, int w_dtype, float eps, int unit_after,
+                                      const void* cos_t, const void* sin_t, int rotary_dim, int interleaved,
+                                      const int* positions, const int* slot_of_token, const int* block_table,
+                                      int table_stride, void* k_pages, void* v_pages, int tokens, int nq, int nkv, int Dk,
+                                      int Dv, int page_size, void* stream) {
+  if (tokens == 0) return 0;
+  const auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  if (parts < 1 || Dk < 8 || Dk > 512 || Dk % 8 || Dv < 8 || Dv % 8 || rotary_dim < 0 || rotary_dim > Dk || rotary_dim % 2 ||
+      (!interleaved && rotary_dim % 16) || part_stride % 4 || row_stride % 4 || !al(sums) || !al(q_out) || !al(k_pages))
+    return static_cast<int>(hipErrorInvalidValue);
+  int lph = 1;
+  while (8 * lph < Dk) lph *= 2;
+  const int lanes = ((nq + nkv) * lph + 63) / 64 * 64 + nkv * (Dv / 8);
+  if ((lanes + 255) / 256 > 65535) return static_cast<int>(hipErrorInvalidValue);
+  const dim3 grid(tokens, (lanes + 255) / 256);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const QkvSums a{sums, parts, part_stride, row_stride};
+#define ARLE_ROT_SUMS(LPH)                                                                                            \
+  rotary_qkv_store_x8_kernel<LPH, true><<<grid, 256, 0, s>>>(                                                         \
+      static_cast<bf16*>(q_out), static_cast<long long>(nq) * Dk, nullptr, 0, nullptr, 0, q_weight, k_weight, w_dtype, eps, \
+      unit_after, static_cast<const float*>(cos_t), static_cast<const float*>(sin_t), rotary_dim, interleaved, positions, \
+      slot_of_token, block_table, table_stride, static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), nq, nkv, Dk, Dv, \
+      page_size, a)
+  switch (lph) {
+    case 1: ARLE_ROT_SUMS(1); break;
+    case 2: ARLE_ROT_SUMS(2); break;
+    case 4: ARLE_ROT_SUMS(4); break;
+    case 8: ARLE_ROT_SUMS(8); break;
+    case 16: ARLE_ROT_SUMS(16); break;
+    case 32: ARLE_ROT_SUMS(32); break;
+    default: ARLE_ROT_SUMS(64); break;
+  }
+#undef ARLE_ROT_SUMS
   return launch_status();
 }

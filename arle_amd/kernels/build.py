@@ -49,6 +49,8 @@ SOURCES = {
     "latent_attention": "latent_attention.hip",
     "retention": "retention.hip",
     "decay_scan": "decay_scan.hip",
+    "gated_linear": "gated_linear.hip",
+    "state_space": "state_space.hip",
     "host": "host/runtime.cpp",
 }
 HEADERS = ("common.h", "attention_static.h", "attention_args.h", "attention_stream.h", "attention_portions.h",

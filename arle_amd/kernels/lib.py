@@ -88,6 +88,14 @@ SIGNATURES = {
                                        _i, _p]),
     "arle_decay_gates": ("decay_scan", [_p, _ll, _p, _i, _p, _f, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
     "arle_gated_group_norm": ("decay_scan", [_p, _p, _ll, _i, _p, _f, _f, _p, _ll, _i, _i, _i, _p]),
+    "arle_gated_linear_decode": ("gated_linear", [_p, _i, _ll, _ll, _p, _i, _i, _p, _f, _p, _p, _p, _p, _f, _p, _i, _i, _i, _i, _i,
+                                                  _p]),
+    "arle_gated_linear_chunks": ("gated_linear", [_p, _ll, _p, _p, _p, _p, _p, _i, _i, _p, _f, _p, _i, _i, _i, _i, _p]),
+    "arle_state_space_decode": ("state_space", [_p, _i, _ll, _ll, _p, _i, _p, _i, _p, _i, _p, _p, _p, _p, _p, _p, _p, _p, _f, _f,
+                                                _i, _p, _ll, _i, _i, _i, _i, _i, _p]),
+    "arle_state_space_chunks": ("state_space", [_p, _ll, _p, _ll, _p, _p, _p, _p, _p, _i, _i, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
+    "arle_rotary_sums_store": ("rotary_store", [_p, _i, _ll, _ll, _p, _p, _p, _i, _f, _i, _p, _p, _i, _i, _p, _p, _p, _i, _p, _p,
+                                                _i, _i, _i, _i, _i, _i, _p]),
     "arle_latent_prep": ("latent", [_p, _ll, _p, _ll, _p, _ll, _i, _p, _i, _f, _p, _p, _i, _p, _p, _p, _i, _p, _p, _i, _i,
                                     _i, _i, _i, _i, _i, _p]),
     "arle_latent_attn": ("latent_attention", [_p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _p, _i, _i, _i, _p, _p,

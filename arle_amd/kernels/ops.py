@@ -2393,6 +2393,49 @@ def rotary_qkv_store(q, k, v, *, num_q_heads: int, num_kv_heads: int, key_dim: i
              num_kv_heads, key_dim, value_dim, int(page_size), _stream())
 
 
+def rotary_sums_supported(key_dim: int, value_dim: int, rotary_dim: int, interleaved: bool) -> bool:
+    """Whether `rotary_sums_store` takes heads of these sizes."""
+    return key_dim % 8 == 0 and key_dim <= 512 and value_dim % 8 == 0 and (interleaved or rotary_dim % 16 == 0)
+
+
+def rotary_sums_store(y, first: int, *, num_q_heads: int, num_kv_heads: int, key_dim: int, value_dim: int, eps: float,
+                      q_weight=None, k_weight=None, unit_after: bool = False, cos=None, sin=None, rotary_dim: int = 0,
+                      interleaved: bool = False, positions, slot_of_token, block_table, k_pages, v_pages, page_size: int):
+    """`rotary_qkv_store` from y, float32 [T, .] or a stack [S, T, .] of partial sums to be added in order, whose columns from
+    `first` on are q | k | v; they are rounded to bfloat16 on the way.  Returns q, bfloat16 [T, heads * Dk]."""
+    _gpu(y, q_weight, k_weight, cos, sin, positions, slot_of_token, block_table, k_pages, v_pages)
+    tokens, width = y.shape[-2:]
+    columns = (num_q_heads + num_kv_heads) * key_dim + num_kv_heads * value_dim
+    _need(y.dim() in (2, 3) and y.dtype == torch.float32 and y.is_contiguous() and 0 <= first and first + columns <= width,
+          "y must be contiguous float32 with the columns q | k | v")
+    _need(width % 4 == 0 and first % 4 == 0 and rotary_sums_supported(key_dim, value_dim, rotary_dim, interleaved),
+          "sizes outside this form's")
+    _need((q_weight is None) == (k_weight is None), "give both norm weights or neither")
+    w_code = 0
+    if q_weight is not None:
+        for w in (q_weight, k_weight):
+            _need(w.shape == (key_dim,) and w.is_contiguous() and w.dtype in _CODES, "a q/k norm weight must be [Dk]")
+        _need(q_weight.dtype == k_weight.dtype, "q and k norm weights must be of one type")
+        w_code = _code(q_weight)
+    _need(0 <= rotary_dim <= key_dim and rotary_dim % 2 == 0, "rotary_dim must be even and at most the key size")
+    if rotary_dim:
+        for name, t in (("cos", cos), ("sin", sin)):
+            _need(t is not None and t.dtype == torch.float32 and t.dim() == 2 and t.shape[1] == rotary_dim // 2
+                  and t.is_contiguous(), f"{name} must be contiguous float32 [positions, rotary_dim / 2]")
+    _check_kv_pages(k_pages, v_pages, num_kv_heads, page_size, key_dim, value_dim, torch.bfloat16)
+    _i32(positions, "positions", tokens)
+    _i32(slot_of_token, "slot_of_token", tokens)
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous(),
+          "block_table must be contiguous int32 [slots, pages]")
+    q = torch.empty((tokens, num_q_heads * key_dim), dtype=torch.bfloat16, device=y.device)
+    lib.call("arle_rotary_sums_store", y.data_ptr() + 4 * first, y.shape[0] if y.dim() == 3 else 1, tokens * width, width,
+             q.data_ptr(), _ptr(q_weight), _ptr(k_weight), w_code, float(eps), 1 if unit_after else 0, _ptr(cos), _ptr(sin),
+             int(rotary_dim), 1 if interleaved else 0, positions.data_ptr(), slot_of_token.data_ptr(),
+             block_table.data_ptr(), block_table.shape[1], k_pages.data_ptr(), v_pages.data_ptr(), tokens, num_q_heads,
+             num_kv_heads, key_dim, value_dim, int(page_size), _stream())
+    return q
+
+
 # ------------------------------------------------------------------------- gated delta rule
 
 GATED_DELTA_MAX_KEY_DIM = 256
@@ -2649,4 +2692,136 @@ def gated_linear_rows(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, eps: fl
     out = torch.empty((T, vw), dtype=out_dtype, device=y.device)
     lib.call("arle_gated_delta_output", o.data_ptr(), g.data_ptr(), y.stride(0), 0, norm.data_ptr(), 0, float(eps),
              out.data_ptr(), _code(out), T, H, Dv, 0, _stream())
+    return out
+
+
+_DECAY_WORK_BYTES = 4 << 30        # most memory for the states in front of the chunks
+_DECAY_CHUNK_MAX_DV = 256
+_GATED_LINEAR_DECODE_MAX_DV = 1024
+_GATED_LINEAR_DECODE_MAX_RANK = 256
+
+
+def _chunk_items(tokens: int, segments: int) -> int:
+    """No fewer than the chunks of 64 rows of all segments together."""
+    return tokens // DECAY_CHUNK + segments
+
+
+def gated_linear_decode_supported(value_dim: int, rank: int) -> bool:
+    """Whether `gated_linear_decode` takes these sizes."""
+    return value_dim % 4 == 0 and value_dim <= _GATED_LINEAR_DECODE_MAX_DV and rank <= _GATED_LINEAR_DECODE_MAX_RANK
+
+
+def gated_linear_decode(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, tau: float, heads: int,
+                        key_dim: int, value_dim: int):
+    """`gated_linear_rows` for steps of one row a segment, in one kernel; y may be the stack of the product's partial sums."""
+    rank = _gated_linear_check(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, heads, key_dim, value_dim)
+    _need(y.shape[-2] == seg_slot.numel(), "one row a segment")
+    _need(gated_linear_decode_supported(value_dim, rank), "sizes outside this form's")
+    T, width = y.shape[-2:]
+    out = torch.empty((T, heads * value_dim), dtype=out_dtype, device=y.device)
+    lib.call("arle_gated_linear_decode", y.data_ptr(), y.shape[0] if y.dim() == 3 else 1, T * width, width, a2.data_ptr(),
+             _code(a2), rank, a2_bias.data_ptr(), 1.0 / tau, norm.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(),
+             s_state.data_ptr(), float(eps), out.data_ptr(), _code(out), seg_slot.numel(), heads, key_dim, value_dim, _stream())
+    return out
+
+
+def gated_linear_chunks_supported(tokens: int, segments: int, heads: int, key_dim: int, value_dim: int) -> bool:
+    """Whether the form over chunks on the matrix cores takes these sizes."""
+    work = _chunk_items(tokens, segments) * heads * key_dim * value_dim * 4
+    return key_dim % 4 == 0 and value_dim % 4 == 0 and value_dim <= _DECAY_CHUNK_MAX_DV and work <= _DECAY_WORK_BYTES
+
+
+def gated_linear_chunks(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, eps: float, out_dtype, *, tau: float, heads: int,
+                        key_dim: int, value_dim: int):
+    """`gated_linear_rows` over chunks of 64 rows on the matrix cores (float32 products; see csrc/gated_linear.hip)."""
+    H, D, Dv = heads, key_dim, value_dim
+    rank = _gated_linear_check(y, a2, a2_bias, norm, s_state, seg_row0, seg_slot, H, D, Dv)
+    T, segments = y.shape[0], seg_slot.numel()
+    _need(y.dim() == 2 and y.shape[1] % 4 == 0 and gated_linear_chunks_supported(T, segments, H, D, Dv), "sizes outside the chunks' form")
+    items = _chunk_items(T, segments)
+    sums = torch.empty((T, H * D), dtype=torch.float32, device=y.device)
+    middle = y.data_ptr() + 4 * 2 * H * (D + Dv)
+    lib.call("arle_decay_gates", middle, y.stride(0), a2.data_ptr(), _code(a2), a2_bias.data_ptr(), 1.0 / tau, seg_row0.data_ptr(),
+             segments, items, 1, sums.data_ptr(), T, rank, H * D, _stream())
+    work = torch.empty((items, H, Dv, D), dtype=torch.float32, device=y.device)
+    out = torch.empty((T, H * Dv), dtype=out_dtype, device=y.device)
+    lib.call("arle_gated_linear_chunks", y.data_ptr(), y.stride(0), sums.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(),
+             norm.data_ptr(), s_state.data_ptr(), segments, items, work.data_ptr(), float(eps), out.data_ptr(), _code(out), H, D, Dv,
+             _stream())
+    return out
+
+
+_STATE_SPACE_MAX_P = 256
+
+
+def state_space_decode_supported(state: int, value_dim: int) -> bool:
+    """Whether `state_space_decode` takes heads of these sizes."""
+    return state <= DECAY_SCAN_MAX_KEY_DIM and value_dim % 4 == 0 and value_dim <= _STATE_SPACE_MAX_P
+
+
+def state_space_decode(y, first: int, conv, conv_bias, conv_state, a_log, dt_bias, skip, norm, s_state, seg_row0, seg_slot,
+                       eps: float, out, *, heads: int, groups: int, state: int, value_dim: int, norm_groups: int, factor: float):
+    """A decoded row of every segment through a state-space layer (see csrc/state_space.hip), bfloat16: y float32 [T, .] or a
+    stack [S, T, .] of partial sums to be added in order, its columns from `first` on z | x | B | C | dt; conv [channels, taps]
+    and conv_bias [channels]; conv_state bfloat16 [slots, taps - 1, channels], moved on, or None with one tap; a_log, dt_bias,
+    skip float32 [heads], norm float32 [heads * P]; s_state float32 [slots, heads, N, P].  Writes what the output projection
+    reads, times `factor`, into the view out [T, heads * P]."""
+    H, G, N, P = heads, groups, state, value_dim
+    segments = _check_segments(s_state, seg_row0, seg_slot, H, N, P)
+    _gpu(y, conv, conv_bias, conv_state, out)
+    T, width = y.shape[-2:]
+    inner = H * P
+    channels = inner + 2 * G * N
+    _need(G > 0 and H % G == 0 and state_space_decode_supported(N, P) and inner % norm_groups == 0, "sizes outside this form's")
+    _need(T == segments, "one row a segment")
+    _need(y.dim() in (2, 3) and y.dtype == torch.float32 and y.is_contiguous() and 0 <= first and first + inner + channels + H <= width,
+          "y must be contiguous float32 with the columns z | x | B | C | dt")
+    _need(conv.dim() == 2 and conv.shape[0] == channels and conv.is_contiguous() and conv.dtype in _CODES
+          and 1 <= conv.shape[1] <= CONV_MAX_TAPS, f"conv must be contiguous [channels, 1..{CONV_MAX_TAPS} taps]")
+    taps = conv.shape[1]
+    _need(conv_bias.shape == (channels,) and conv_bias.is_contiguous() and conv_bias.dtype in _CODES, "conv_bias must be [channels]")
+    _need(taps == 1 or (conv_state is not None and tuple(conv_state.shape[1:]) == (taps - 1, channels)
+                        and conv_state.dtype == torch.bfloat16 and conv_state.is_contiguous()),
+          "conv_state must be bfloat16 [slots, taps - 1, channels]")
+    for name, t, n in (("a_log", a_log, H), ("dt_bias", dt_bias, H), ("skip", skip, H), ("norm", norm, inner)):
+        _f32_vector(t, n, name)
+    _rows(out, "out")
+    _need(out.shape == (T, inner) and out.dtype == torch.bfloat16, "out must be bfloat16 [T, heads * P]")
+    scratch = torch.empty((T, inner), dtype=torch.float32, device=y.device)
+    lib.call("arle_state_space_decode", y.data_ptr() + 4 * first, y.shape[0] if y.dim() == 3 else 1, T * width, width,
+             conv.data_ptr(), _code(conv), conv_bias.data_ptr(), _code(conv_bias), conv_state.data_ptr() if taps > 1 else 0, taps,
+             a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(), s_state.data_ptr(),
+             scratch.data_ptr(), norm.data_ptr(), float(eps), float(factor), int(norm_groups), out.data_ptr(), out.stride(0),
+             segments, H, G, N, P, _stream())
+    return out
+
+
+def state_space_chunks_supported(dtype, tokens: int, segments: int, heads: int, state: int, value_dim: int) -> bool:
+    """Whether the form over chunks on the matrix cores takes these sizes."""
+    work = _chunk_items(tokens, segments) * heads * state * value_dim * 4
+    return (dtype == torch.bfloat16 and state % 8 == 0 and value_dim % 8 == 0 and value_dim <= _STATE_SPACE_MAX_P
+            and work <= _DECAY_WORK_BYTES)
+
+
+def state_space_chunks(u, dt, a_log, dt_bias, skip, s_state, seg_row0, seg_slot, *, heads: int, groups: int, state: int,
+                       value_dim: int):
+    """`state_space_rows` over chunks of 64 rows on the matrix cores (see csrc/state_space.hip); u bfloat16 [T, x | B | C],
+    contiguous, as the convolution left it."""
+    H, G, N, P = heads, groups, state, value_dim
+    segments = _check_segments(s_state, seg_row0, seg_slot, H, N, P)
+    T = u.shape[0]
+    _gpu(u, dt)
+    _need(G > 0 and H % G == 0 and u.shape == (T, H * P + 2 * G * N) and u.is_contiguous()
+          and state_space_chunks_supported(u.dtype, T, segments, H, N, P), "sizes outside the chunks' form")
+    _rows(dt, "dt")
+    _need(dt.dtype == torch.float32 and dt.shape[0] == T and dt.shape[1] >= H, "dt must be float32 [T, >= heads]")
+    for name, t in (("a_log", a_log), ("dt_bias", dt_bias), ("skip", skip)):
+        _f32_vector(t, H, name)
+    items = _chunk_items(T, segments)
+    work = torch.empty((items, H, P, N), dtype=torch.float32, device=u.device)
+    ends = torch.empty((items, H), dtype=torch.float32, device=u.device)
+    out = torch.empty((T, H * P), dtype=torch.float32, device=u.device)
+    lib.call("arle_state_space_chunks", u.data_ptr(), u.stride(0), dt.data_ptr(), dt.stride(0), a_log.data_ptr(),
+             dt_bias.data_ptr(), skip.data_ptr(), seg_row0.data_ptr(), seg_slot.data_ptr(), segments, items, s_state.data_ptr(),
+             work.data_ptr(), ends.data_ptr(), out.data_ptr(), H, G, N, P, _stream())
     return out

@@ -9,7 +9,9 @@ Per token, with h the mixer's input, H heads, key size D, value size Dv:
 
 S starts at zero and lives in a 32-bit state slot `[H, D, Dv]` of the request.  One fused product makes q, k, v, the gate
 and the narrow middle and hands over its 32-bit sums; decays, recurrence and head norm are 32-bit in every mode (at a
-request's first rows o is a few terms, whose signs the norm magnifies).  The middle's width is the tensors' own.
+request's first rows o is a few terms, whose signs the norm magnifies).  The middle's width is the tensors' own.  A float32
+engine works row by row, in one order however a prompt is cut; a bfloat16 engine takes decoded rows in one kernel and
+longer portions in chunks on the matrix cores (see csrc/gated_linear.hip).
 """
 from __future__ import annotations
 
@@ -24,6 +26,8 @@ from .linear import Linear
 @register("mixer", "gated_linear")
 class GatedLinearMixer(Part):
     """params: hidden_size, heads, key_dim, value_dim, tau, eps, decay_rank (int, or None: whatever the tensors have)."""
+
+    CHUNKS_FROM = 64    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
 
     graph_safe = True  # rows, slots and lengths are read on the GPU; launches depend on shapes only
 
@@ -70,7 +74,17 @@ class GatedLinearMixer(Part):
 
     def forward(self, x, batch, cache):
         """x [T, W] -> float32 [T, W], or a float32 stack [S, T, W] to be added in order (see Linear)."""
-        y = self.proj(x, out_dtype=torch.float32)
-        out = ops.gated_linear_rows(y, self.a2, self.a2_bias, self.norm, cache.state, batch.seg_row0, batch.seg_slot, self.eps,
-                                    self.rt.act_dtype, tau=self.tau, heads=self.H, key_dim=self.D, value_dim=self.Dv)
+        rows, segments = x.shape[0], batch.seg_slot.numel()
+        y = self.proj(x, out_dtype=torch.float32, partials_ok=True)
+        form = ops.gated_linear_rows
+        if not self.rt.is_f32 and batch.max_qlen == 1 and rows == segments and ops.gated_linear_decode_supported(self.Dv, self.rank):
+            form = ops.gated_linear_decode
+        else:
+            if y.dim() == 3:
+                y = ops.sum_partials(y, torch.float32)
+            if (not self.rt.is_f32 and batch.max_qlen >= self.CHUNKS_FROM
+                    and ops.gated_linear_chunks_supported(rows, segments, self.H, self.D, self.Dv)):
+                form = ops.gated_linear_chunks
+        out = form(y, self.a2, self.a2_bias, self.norm, cache.state, batch.seg_row0, batch.seg_slot, self.eps, self.rt.act_dtype,
+                   tau=self.tau, heads=self.H, key_dim=self.D, value_dim=self.Dv)
         return self.o(out, out_dtype=torch.float32, partials_ok=True)   # into the 32-bit residual unrounded

@@ -117,11 +117,16 @@ class MixerSum(_TwoMixers):
     def forward(self, x, batch, cache):
         """x [T, W] -> float32 [T, W], or a float32 stack [S, T, W] to be added in order (see Linear)."""
         cache = cache or {}
-        y = self.proj(x)
+        sums = all(m.takes_sums(x, batch) for m in (self.left, self.right))     # decoded rows: no pass that adds the partial sums
+        y = self.proj(x, out_dtype=torch.float32, partials_ok=True) if sums else self.proj(x)
         make = torch.zeros if self.padded else torch.empty
         out = make((x.shape[0], sum(self.out_widths)), dtype=x.dtype, device=x.device)
         first, at = 0, 0
         for name, m, factor, width in zip(("left", "right"), (self.left, self.right), self.scales, self.out_widths):
-            m.heads(y[:, first:first + m.in_width], x, batch, cache.get(name), out[:, at:at + m.heads_width], factor)
+            view = out[:, at:at + m.heads_width]
+            if sums:
+                m.heads_of_sums(y, first, batch, cache.get(name), view, factor)
+            else:
+                m.heads(y[:, first:first + m.in_width], x, batch, cache.get(name), view, factor)
             first, at = self.in_at, at + width
         return self.o(out, out_dtype=torch.float32, partials_ok=True)   # it goes into the 32-bit residual unrounded

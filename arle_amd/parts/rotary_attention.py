@@ -126,17 +126,38 @@ class RotaryAttention(Part):
             raise ValueError("this attention keeps keys and values of its own")
         Q, K, _ = self.widths
         q, k, v = y[:, :Q], y[:, Q:Q + K], y[:, Q + K:self.in_width]
+        ops.rotary_qkv_store(q, k, v, **self._preparation(batch, cache))
+        self._attend(q, batch, cache, out, factor)
+
+    def _preparation(self, batch, cache) -> dict:
         cos = sin = None
         rotary_dim, interleaved = 0, False
         if self.position is not None:
             cos, sin, rotary_dim = self.position.fused_rotary()
             interleaved = self.position.kind == "rope_interleaved"
-        ops.rotary_qkv_store(q, k, v, num_q_heads=self.nq, num_kv_heads=self.nkv, key_dim=self.Dk, value_dim=self.Dv,
-                             eps=self.eps, q_weight=self.q_norm, k_weight=self.k_norm,
-                             unit_after=self.qk_norm == "unit_after", cos=cos, sin=sin, rotary_dim=rotary_dim or 0,
-                             interleaved=interleaved, positions=batch.positions, slot_of_token=batch.slot_of_token,
-                             block_table=cache.block_table, k_pages=cache.pages["k"], v_pages=cache.pages["v"],
-                             page_size=cache.page_size)
+        return dict(num_q_heads=self.nq, num_kv_heads=self.nkv, key_dim=self.Dk, value_dim=self.Dv, eps=self.eps,
+                    q_weight=self.q_norm, k_weight=self.k_norm, unit_after=self.qk_norm == "unit_after", cos=cos, sin=sin,
+                    rotary_dim=rotary_dim or 0, interleaved=interleaved, positions=batch.positions,
+                    slot_of_token=batch.slot_of_token, block_table=cache.block_table, k_pages=cache.pages["k"],
+                    v_pages=cache.pages["v"], page_size=cache.page_size)
+
+    def _attend(self, q, batch, cache, out, factor: float) -> None:
         softcap_attention(q, out, cache, batch, num_q_heads=self.nq, num_kv_heads=self.nkv, key_dim=self.Dk,
                           value_dim=self.Dv, scale=self.scale, softcap=self.softcap, r1=None, r2=None,
                           window=self.window, sink=self.sink, out_scale=factor)
+
+    def takes_sums(self, x, batch) -> bool:
+        """Whether this step is one of decoded rows that `heads_of_sums` takes."""
+        rotary_dim, interleaved = 0, False
+        if self.position is not None:
+            rotary_dim, interleaved = self.position.rotary_dim, self.position.kind == "rope_interleaved"
+        return (not self.rt.is_f32 and batch.max_qlen == 1 and x.shape[0] == batch.seg_slot.numel()
+                and ops.rotary_sums_supported(self.Dk, self.Dv, rotary_dim, interleaved))
+
+    def heads_of_sums(self, y, first, batch, cache, out, factor: float = 1.0):
+        """`heads` of decoded rows from the product's 32-bit sums (a tensor or a stack of partial ones), whose columns from
+        `first` on are q, k and v."""
+        if not cache.writes:
+            raise ValueError("this attention keeps keys and values of its own")
+        q = ops.rotary_sums_store(y, first, **self._preparation(batch, cache))
+        self._attend(q, batch, cache, out, factor)

@@ -11,7 +11,9 @@ Per token, with h the mixer's input, H heads of P values, G groups (head j belon
 
 S starts at zero and lives in a 32-bit state slot `[H, N, P]` of the request; the convolution's last taps - 1 inputs are
 state too.  Step sizes leave their projection as 32-bit sums; decays, recurrence, gate and norm are 32-bit in every mode;
-the other projections and the convolution run in the activation type.
+the other projections and the convolution run in the activation type.  A float32 engine works row by row, in one order however a
+prompt is cut; a bfloat16 engine takes decoded rows from the projection's sums to the gated norm in two kernels, and longer
+portions in chunks on the matrix cores (see csrc/state_space.hip).
 """
 from __future__ import annotations
 
@@ -28,6 +30,8 @@ from .short_conv import ShortConv
 class StateSpaceMixer(Part):
     """params: hidden_size, heads, value_dim, state, groups, conv_taps, norm_groups, eps, project_out (bool, default True;
     False: one of a joined pair of mixers, which owns the products in front and behind, and calls `heads`)."""
+
+    CHUNKS_FROM = 32    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
 
     graph_safe = True  # rows, slots and lengths are read on the GPU; launches depend on shapes only
 
@@ -100,7 +104,10 @@ class StateSpaceMixer(Part):
     def forward(self, x, batch, cache):
         """x [T, W] -> float32 [T, W], or a float32 stack [S, T, W] to be added in order (see Linear)."""
         out = torch.empty((x.shape[0], self.heads_width), dtype=x.dtype, device=x.device)
-        self.heads(self.proj(x), x, batch, cache, out)
+        if self.takes_sums(x, batch):
+            self.heads_of_sums(self.proj(x, out_dtype=torch.float32, partials_ok=True), 0, batch, cache, out)
+        else:
+            self.heads(self.proj(x), x, batch, cache, out)
         return self.o(out, out_dtype=torch.float32, partials_ok=True)   # into the 32-bit residual unrounded
 
     def heads(self, y, x, batch, cache, out, factor: float = 1.0):
@@ -109,7 +116,25 @@ class StateSpaceMixer(Part):
         inner, gn = self.inner, self.G * self.N
         dt = self.dt(x, out_dtype=torch.float32)
         u = self.conv(y[:, inner:inner + self.channels], batch, cache.get("conv"), silu=True)
-        o = ops.state_space_rows(u[:, :inner], u[:, inner:inner + gn], u[:, inner + gn:], dt, self.a_log, self.dt_bias,
-                                 self.skip, cache["S"].state, batch.seg_row0, batch.seg_slot, heads=self.H, groups=self.G,
-                                 state=self.N, value_dim=self.P)
+        rest = (dt, self.a_log, self.dt_bias, self.skip, cache["S"].state, batch.seg_row0, batch.seg_slot)
+        sizes = dict(heads=self.H, groups=self.G, state=self.N, value_dim=self.P)
+        if (not self.rt.is_f32 and batch.max_qlen >= self.CHUNKS_FROM
+                and ops.state_space_chunks_supported(u.dtype, x.shape[0], batch.seg_slot.numel(), self.H, self.N, self.P)):
+            o = ops.state_space_chunks(u, *rest, **sizes)
+        else:
+            o = ops.state_space_rows(u[:, :inner], u[:, inner:inner + gn], u[:, inner + gn:], *rest, **sizes)
         ops.gated_group_norm(o, y[:, :inner], self.norm, self.eps, groups=self.norm_groups, factor=factor, out=out)
+
+    def takes_sums(self, x, batch) -> bool:
+        """Whether this step is one of decoded rows that `heads_of_sums` takes."""
+        return (not self.rt.is_f32 and batch.max_qlen == 1 and x.shape[0] == batch.seg_slot.numel()
+                and ops.state_space_decode_supported(self.N, self.P))
+
+    def heads_of_sums(self, y, first, batch, cache, out, factor: float = 1.0):
+        """`heads` of decoded rows from the product's 32-bit sums (a tensor or a stack of partial ones), whose columns from
+        `first` on are this mixer's."""
+        conv = cache.get("conv")
+        ops.state_space_decode(y, first, self.conv.weight, self.conv.out_bias, conv.state if conv is not None else None, self.a_log,
+                               self.dt_bias, self.skip, self.norm, cache["S"].state, batch.seg_row0, batch.seg_slot, self.eps, out,
+                               heads=self.H, groups=self.G, state=self.N, value_dim=self.P, norm_groups=self.norm_groups,
+                               factor=factor)

@@ -11,8 +11,8 @@ import torch
 
 F = torch.float64
 
-# a test may set this to a function of a matrix product's result (to move every entry by a rounding, say)
-after_product = None
+# a test may set this to a function (x, w) -> product (one that moves every entry by a rounding, say)
+around_product = None
 
 
 def t64(x):
@@ -21,8 +21,7 @@ def t64(x):
 
 def mm(x, w):
     """x [.., K] times w [N, K] transposed: every projection goes through here."""
-    y = x @ w.T
-    return after_product(y) if after_product is not None else y
+    return around_product(x, w) if around_product is not None else x @ w.T
 
 
 def silu(z):
