@@ -28,6 +28,8 @@ struct AttnArgs {
   int p_shift;  // log2(P): page sizes are powers of two, so / and % by P are a shift and a mask
   float scale_log2;
   int window;  // 0: all earlier keys
+  const float* sink;   // [q heads] or null: exp(sink_h) joins the softmax's denominator, with no value behind it
+  float out_scale;     // a factor on the output, in 32 bits
   int splits;
   int ws_rows;   // token rows that the split-KV workspace holds for a segment
   int portion_splits;  // parts into which the LDS kernel cuts the keys of a row block (1: whole; it writes out)
@@ -59,6 +61,12 @@ __device__ __forceinline__ bf16x8 load_bf16x8(const uint16_t* p) {
 __device__ __forceinline__ bf16x8 zero_bf16x8() {
   uint4 z = {0u, 0u, 0u, 0u};
   return __builtin_bit_cast(bf16x8, z);
+}
+
+// The factor that turns a row's summed values into its output: m is what its exponentials (of base 2) are taken from, l their sum.
+__device__ __forceinline__ float row_factor(const float* sink, float out_scale, int head, float m, float l) {
+  if (sink) l += exp2f(sink[head] * 1.4426950408889634f - m);
+  return l > 0.f ? out_scale / l : 0.f;
 }
 
 __device__ __forceinline__ float group_max4(float v) {  // over the 4 lanes i, i+16, i+32, i+48

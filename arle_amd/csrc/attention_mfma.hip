@@ -302,6 +302,8 @@ static AttnArgs make_args(const void* q, long long q_stride, void* out, long lon
   a.p_shift = __builtin_ctz(static_cast<unsigned>(page_size));
   a.scale_log2 = scale * 1.4426950408889634f;
   a.window = window;
+  a.sink = nullptr;
+  a.out_scale = 1.0f;
   a.splits = splits;
   a.ws_rows = arle_attn_ws_rows(max_qlen, nq, nkv);
   a.portion_splits = 1;
@@ -334,7 +336,8 @@ static AttnArgs make_args(const void* q, long long q_stride, void* out, long lon
 // must hold [token rows][nq][portion_splits][D] and [..][2] floats, and a merge of their own runs after.
 // plan_token: 0, or a number that names the step (the same for every layer of it, another for every other step of
 // the process): the portions kernels then list their work once a step instead of once a call.
-// Requires D % 16 == 0, D <= 256, page_size a power of two >= 4.
+// sink: float32 [nq] or null; out_scale: a factor on the output (see AttnArgs).
+// Requires D % 16 == 0, D <= 256, page_size a power of two >= 4; rows of out 8-byte aligned.
 extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out, long long o_stride,
                                     const void* k_pages, const void* v_pages, const int* block_table,
                                     int table_stride, const int* seg_row0, const int* seg_slot,
@@ -342,7 +345,8 @@ extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out
                                     int max_kv_len, int token_rows,
                                     int nq, int nkv, int D, int page_size, float scale, int window,
                                     int splits, float* ws_o, float* ws_ml, int portion_splits, float* pws_o,
-                                    float* pws_ml, long long plan_token, void* stream) {
+                                    float* pws_ml, long long plan_token, const float* sink, float out_scale,
+                                    void* stream) {
   if (segments == 0 || token_rows == 0) return 0;
   if (D % 16 != 0 || D > 256 || D <= 0 || page_size < 4 || (page_size & (page_size - 1)) != 0 || nq % nkv != 0 ||
       splits < 1 || splits > 64 || portion_splits < 1 || portion_splits > kPortionPartsMax ||
@@ -351,6 +355,8 @@ extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out
   hipStream_t s = static_cast<hipStream_t>(stream);
   AttnArgs a = make_args(q, q_stride, out, o_stride, k_pages, v_pages, block_table, table_stride, seg_row0, seg_slot,
                          seg_start, max_qlen, nq, nkv, D, page_size, scale, window, splits, ws_o, ws_ml);
+  a.sink = sink;
+  a.out_scale = out_scale;
   a.portion_splits = portion_splits;
   a.pws_o = pws_o;
   a.pws_ml = pws_ml;
@@ -380,7 +386,7 @@ extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out
       side_rc = launch_attn<1>(b, dim3(1, nkv, static_cast<unsigned>(z)), side->stream);
       if (side_rc == 0 && splits > 1) {
         attn_merge_kernel<<<dim3(segments * b.ws_rows, nq), kMergeWaves * kWave, 0, side->stream>>>(
-            ws_o, ws_ml, b.out, o_stride, seg_row0, b.ws_rows, b.rows_max, nq, nkv, D, splits);
+            ws_o, ws_ml, b.out, o_stride, seg_row0, b.ws_rows, b.rows_max, nq, nkv, D, splits, a.sink, a.out_scale);
         side_rc = launch_status();
       }
     }
@@ -417,7 +423,7 @@ extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out
     rc = launch_attn<1>(a, dim3(1, nkv, static_cast<unsigned>(z)), s);
     if (rc != 0 || splits == 1) return rc;
     attn_merge_kernel<<<dim3(segments * a.ws_rows, nq), kMergeWaves * kWave, 0, s>>>(
-        ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, a.rows_max, nq, nkv, D, splits);
+        ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, a.rows_max, nq, nkv, D, splits, a.sink, a.out_scale);
     return launch_status();
   }
   if (max_rows > 16 && splits > 1) return static_cast<int>(hipErrorInvalidValue);  // two row tiles: no split
@@ -427,7 +433,7 @@ extern "C" int arle_attn_paged_mfma(const void* q, long long q_stride, void* out
   rc = nt == 1 ? launch_attn<1>(a, grid, s) : launch_attn<2>(a, grid, s);
   if (rc != 0 || splits == 1) return rc;
   attn_merge_kernel<<<dim3(segments * a.ws_rows, nq), kMergeWaves * kWave, 0, s>>>(
-      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits);
+      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits, a.sink, a.out_scale);
   return launch_status();
 }
 
@@ -516,7 +522,7 @@ extern "C" int arle_attn_decode_prep(const void* parts, int parts_bf16, int n_pa
   const int rc = launch_status();
   if (rc != 0 || splits == 1) return rc;
   attn_merge_kernel<<<dim3(segments * a.ws_rows, nq), kMergeWaves * kWave, 0, s>>>(
-      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits);
+      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits, a.sink, a.out_scale);
   return launch_status();
 }
 
@@ -599,6 +605,6 @@ extern "C" int arle_attn_decode_static(const void* q, long long q_stride, void* 
   int rc = launch_attn<1>(a, dim3(1, nkv, static_cast<unsigned>(z)), s);
   if (rc != 0 || splits == 1) return rc;
   attn_merge_kernel<<<dim3(segments * a.ws_rows, nq), kMergeWaves * kWave, 0, s>>>(
-      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits);
+      ws_o, ws_ml, a.out, o_stride, seg_row0, a.ws_rows, 0, nq, nkv, D, splits, a.sink, a.out_scale);
   return launch_status();
 }

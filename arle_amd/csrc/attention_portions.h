@@ -510,7 +510,7 @@ __global__ __launch_bounds__(kPfWaves* kWave, 1) __attribute__((amdgpu_waves_per
       }
       continue;
     }
-    const float inv_l = l[n] > 0.f ? 1.0f / l[n] : 0.f;
+    const float inv_l = row_factor(a.sink, a.out_scale, my_head[n], m[n], l[n]);
     uint16_t* op = a.out + static_cast<int64_t>(row0 + my_tok[n]) * a.o_stride + my_head[n] * D;
 #pragma unroll
     for (int dt = 0; dt < DTL; ++dt) {
@@ -576,7 +576,7 @@ __global__ __launch_bounds__(kPfWaves* kWave) void attn_merge_portions_kernel(co
       o.z += os[p].z * w;
       o.w += os[p].w * w;
     }
-    const float inv = denom > 0.f ? 1.0f / denom : 0.f;
+    const float inv = row_factor(a.sink, a.out_scale, head, mx, denom);
     if (d0 < D) {
       uint2 w;
       w.x = static_cast<uint32_t>(f32_to_bf16_bits(o.x * inv)) | (static_cast<uint32_t>(f32_to_bf16_bits(o.y * inv)) << 16);

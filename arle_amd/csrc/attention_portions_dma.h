@@ -500,7 +500,7 @@ __global__ __launch_bounds__(GROUPS* kDmWaves* kWave, GROUPS == 1 ? 2 : 1) void 
         a.pws_ml[slot * 2 + 1] = l;
       }
     } else {
-      const float inv_l = l > 0.f ? 1.0f / l : 0.f;
+      const float inv_l = row_factor(a.sink, a.out_scale, my_head, m, l);
       uint16_t* op = a.out + static_cast<int64_t>(row0 + my_tok) * a.o_stride + my_head * D;
 #pragma unroll
       for (int dt = 0; dt < D / 32; ++dt)

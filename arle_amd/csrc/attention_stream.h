@@ -552,7 +552,7 @@ __global__ __launch_bounds__(INWG ? kInWgWavesMax * kWave : kWave) void attn_mfm
     if (!row_ok[n]) continue;
     const int64_t tok_row = row0 + my_tok[n];
     if (INWG || a.splits == 1) {
-      const float inv_l = l[n] > 0.f ? 1.0f / l[n] : 0.f;
+      const float inv_l = row_factor(a.sink, a.out_scale, my_head[n], m[n], l[n]);
       uint16_t* op = a.out + tok_row * a.o_stride + my_head[n] * D;
 #pragma unroll
       for (int dt = 0; dt < DTL; ++dt) {
@@ -594,7 +594,7 @@ constexpr int kMergeMaxD = 256;
 __global__ __launch_bounds__(kMergeWaves* kWave) void attn_merge_kernel(
     const float* __restrict__ ws_o, const float* __restrict__ ws_ml, uint16_t* __restrict__ out,
     int64_t o_stride, const int* __restrict__ seg_row0, int ws_rows, int rows_max, int nq, int nkv, int D,
-    int splits) {
+    int splits, const float* __restrict__ sink, float out_scale) {
   __shared__ float part[kMergeWaves][kMergeMaxD];
   const int head = blockIdx.y;
   const int seg = blockIdx.x / ws_rows, tok = blockIdx.x % ws_rows;
@@ -612,7 +612,7 @@ __global__ __launch_bounds__(kMergeWaves* kWave) void attn_merge_kernel(
   const float mx = wave_max(ms);
   const float wgt = ms > -INFINITY ? exp2f(ms - mx) : 0.f;  // an empty split weighs nothing
   const float denom = wave_sum(ls * wgt);
-  const float inv = denom > 0.f ? 1.0f / denom : 0.f;
+  const float inv = row_factor(sink, out_scale, head, mx, denom);
   // each lane owns d = 4*lane .. 4*lane+3 (D <= 256)
   const int d0 = 4 * lane;
   float4 o = {0.f, 0.f, 0.f, 0.f};

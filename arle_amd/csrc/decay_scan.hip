@@ -169,7 +169,7 @@ __global__ __launch_bounds__(kDsThreads) void decay_gates_kernel(const float* __
 // y [T, width] float32 times silu(z), each of `groups` equal runs of entries divided by its own root mean square, times a
 // weight and a factor.  A workgroup a (row, group).
 template <typename T>
-__global__ __launch_bounds__(kDsThreads) void gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ z,
+__global__ __launch_bounds__(kDsThreads) void gated_norm_kernel(const float* __restrict__ y, const T* __restrict__ z,
                                                                       long long z_stride, const float* __restrict__ w, float eps,
                                                                       float factor, T* __restrict__ out, long long o_stride,
                                                                       int width, int size) {
@@ -252,8 +252,8 @@ extern "C" int arle_gated_group_norm(const float* y, const void* z, long long z_
   const size_t lds = static_cast<size_t>(size) * sizeof(float);     // at most 64 KB
   static bool raised = false;
   if (!raised && lds > 48 * 1024) {
-    const void* kernels[] = {reinterpret_cast<const void*>(&gated_group_norm_kernel<float>),
-                             reinterpret_cast<const void*>(&gated_group_norm_kernel<bf16>)};
+    const void* kernels[] = {reinterpret_cast<const void*>(&gated_norm_kernel<float>),
+                             reinterpret_cast<const void*>(&gated_norm_kernel<bf16>)};
     for (const void* f : kernels) {
       const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024);
       if (e != hipSuccess) return static_cast<int>(e);
@@ -262,10 +262,10 @@ extern "C" int arle_gated_group_norm(const float* y, const void* z, long long z_
   }
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == kF32)
-    gated_group_norm_kernel<float><<<grid, kDsThreads, lds, s>>>(y, static_cast<const float*>(z), z_stride, w, eps, factor,
+    gated_norm_kernel<float><<<grid, kDsThreads, lds, s>>>(y, static_cast<const float*>(z), z_stride, w, eps, factor,
                                                                  static_cast<float*>(out), o_stride, width, size);
   else
-    gated_group_norm_kernel<bf16><<<grid, kDsThreads, lds, s>>>(y, static_cast<const bf16*>(z), z_stride, w, eps, factor,
+    gated_norm_kernel<bf16><<<grid, kDsThreads, lds, s>>>(y, static_cast<const bf16*>(z), z_stride, w, eps, factor,
                                                                 static_cast<bf16*>(out), o_stride, width, size);
   return launch_status();
 }

@@ -48,7 +48,7 @@ SIGNATURES = {
     "arle_attn_prefill_groups": ("attention_mfma", [_i]),
     "arle_attn_side_branch": ("attention_mfma", [_i]),
     "arle_attn_paged_mfma": ("attention_mfma", [_p, _ll, _p, _ll, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i,
-                                                _i, _i, _i, _f, _i, _i, _p, _p, _i, _p, _p, _ll, _p]),
+                                                _i, _i, _i, _f, _i, _i, _p, _p, _i, _p, _p, _ll, _p, _f, _p]),
     "arle_argmax_chunks": ("sampling", [_i, _i]),
     "arle_argmax_rows": ("sampling", [_p, _i, _i, _p, _p, _p]),
     "arle_sample_scratch_bytes": ("sampling", [_i, _i]),

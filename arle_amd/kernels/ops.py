@@ -380,7 +380,7 @@ def attn_paged_mfma(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, s
                     max_qlen: int, max_kv_len: int, num_q_heads: int, num_kv_heads: int, head_dim: int,
                     page_size: int, scale: float, window: int = 0, splits: int | None = None,
                     min_qlen: int = 1, short_segments: int | None = None, portion_splits: int | None = None,
-                    plan_token: int = 0, max_portion_kv_len: int | None = None):
+                    plan_token: int = 0, max_portion_kv_len: int | None = None, sink=None, out_scale: float = 1.0):
     """Causal attention of a packed step on the matrix cores (bfloat16).
 
     Segments: rows seg_row0[s]..seg_row0[s+1] belong to block-table row seg_slot[s] and start at
@@ -392,14 +392,18 @@ def attn_paged_mfma(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, s
     same segments the portions kernels list their work once, for the first layer, and not once a layer.
     `max_portion_kv_len`: the longest context among the segments of more than one token (default: max_kv_len); what
     the portions kernels plan by, so that a fresh portion beside requests that decode deep into their contexts is
-    not cut into parts for the decoders' sake.
+    not cut into parts for the decoders' sake.  `sink` float32 [q heads]: exp(sink_h) joins the softmax's denominator;
+    `out_scale`: a factor on the output, in 32 bits.  out may be a view whose rows lie further apart.
     """
-    _gpu(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, seg_start)
+    _gpu(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, seg_start, sink)
+    _need(sink is None or (sink.shape == (num_q_heads,) and sink.dtype == torch.float32 and sink.is_contiguous()),
+          "sink must be contiguous float32 [heads]")
     tokens = q.shape[0]
     _rows(q, "q")
     _need(q.dtype == torch.bfloat16 and out.dtype == torch.bfloat16, "the MFMA attention takes bfloat16")
-    _need(q.shape == (tokens, num_q_heads * head_dim) and out.shape == q.shape and out.is_contiguous(),
-          "q must be [T, nq*D] and out contiguous [T, nq*D]")
+    _rows(out, "out")
+    _need(q.shape == (tokens, num_q_heads * head_dim) and out.shape == q.shape and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0,
+          "q and out must be [T, nq*D], rows of out 8-byte aligned")
     _need(attn_mfma_supported(q.dtype, head_dim, page_size),
           f"the MFMA attention needs head_dim % 16 == 0, head_dim <= {MFMA_MAX_HEAD_DIM} and a power-of-two page_size >= 4 "
           f"(got head_dim {head_dim}, page_size {page_size})")
@@ -441,7 +445,8 @@ def attn_paged_mfma(q, out, k_pages, v_pages, block_table, seg_row0, seg_slot, s
              seg_row0.data_ptr(), seg_slot.data_ptr(), seg_start.data_ptr(), segments, int(max_qlen),
              int(min_qlen), int(max_portion_kv_len or max_kv_len), tokens,
              num_q_heads, num_kv_heads, head_dim, page_size, float(scale), int(window), int(splits),
-             _ptr(ws_o), _ptr(ws_ml), int(portion_splits), _ptr(pws_o), _ptr(pws_ml), int(plan_token), _stream())
+             _ptr(ws_o), _ptr(ws_ml), int(portion_splits), _ptr(pws_o), _ptr(pws_ml), int(plan_token),
+             _ptr(sink), float(out_scale), _stream())
     return out
 
 

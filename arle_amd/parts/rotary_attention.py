@@ -28,6 +28,7 @@ from .softcap_attention import softcap_attention
 
 QK_NORMS = (None, "weighted_before", "unit_after")
 SINKS = (None, "zero", "learned")
+PAGE_ANY = 16       # a page size that every kernel takes (what a decode step's launches depend on is asked without one)
 
 
 @register("mixer", "rotary_attention")
@@ -142,9 +143,34 @@ class RotaryAttention(Part):
                     v_pages=cache.pages["v"], page_size=cache.page_size)
 
     def _attend(self, q, batch, cache, out, factor: float) -> None:
+        if (self._plain_scores(cache.page_size) and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0 and out.stride(0) % 4 == 0
+                and out.data_ptr() % 8 == 0):
+            # no cap and heads of one size: the kernels of the plain softmax
+            ops.attn_paged_mfma(q, out, cache.pages["k"], cache.pages["v"], cache.block_table, batch.seg_row0, batch.seg_slot,
+                                batch.seg_start, max_qlen=batch.max_qlen, min_qlen=batch.min_qlen,
+                                max_kv_len=self._keys_seen(batch.max_position + 1), num_q_heads=self.nq, num_kv_heads=self.nkv,
+                                head_dim=self.Dk, page_size=cache.page_size, scale=self.scale, window=self.window,
+                                splits=getattr(batch, "kv_splits", None),
+                                short_segments=getattr(batch, "single_segments", 0) or None,
+                                plan_token=getattr(batch, "plan_token", 0), sink=self.sink, out_scale=factor,
+                                max_portion_kv_len=getattr(batch, "max_portion_kv", 0) or None)
+            return
         softcap_attention(q, out, cache, batch, num_q_heads=self.nq, num_kv_heads=self.nkv, key_dim=self.Dk,
                           value_dim=self.Dv, scale=self.scale, softcap=self.softcap, r1=None, r2=None,
                           window=self.window, sink=self.sink, out_scale=factor)
+
+    def _plain_scores(self, page_size: int) -> bool:
+        return (not self.rt.is_f32 and self.softcap == 0.0 and self.Dk == self.Dv
+                and ops.attn_mfma_supported(torch.bfloat16, self.Dk, page_size))
+
+    def _keys_seen(self, keys: int) -> int:
+        return min(keys, self.window + 64) if self.window else keys
+
+    def decode_launch_class(self, rows, max_context):
+        # the split-KV factor of the kernels of the plain softmax follows the context
+        if not self._plain_scores(PAGE_ANY):
+            return None
+        return ops.decode_splits(rows, self.nkv, self._keys_seen(max_context))
 
     def takes_sums(self, x, batch) -> bool:
         """Whether this step is one of decoded rows that `heads_of_sums` takes."""

@@ -8,6 +8,7 @@
     python bench.py --workload tazitar [--shape 4b|8b] [--layers L]  (the Tazitar design beside Qwen3 at equal sizes)
     python bench.py --workload retudra [--shape 4b|8b] [--layers L]  (the Retudra design beside Sovutar and Qwen3 at equal sizes)
     python bench.py --workload nafezen [--shape 4b|8b] [--layers L]  (the Nafezen design beside Retudra and Qwen3 at equal sizes)
+    python bench.py --workload pozirax [--shape 4b|8b] [--layers L]  (the Pozirax design beside Nafezen and Qwen3 at equal sizes)
 
 A step is one decode step of `batch` requests, each holding a `prompt`-token random prompt
 (prefilled by the engine itself before the clock starts) and growing by one token per step.
@@ -1061,6 +1062,90 @@ def nafezen_bench(args) -> int:
                         {"retudra": lambda tokens, batch, context: retudra_work(ret, q, tokens, batch, context)})
 
 
+# ---- the Pozirax design beside Nafezen and Qwen3 at equal sizes ------------------------------------------
+# The widths and head counts of Qwen3-4B / 8B; layers alternate between the pair (a windowed attention beside a state-space
+# layer of twice the width in heads of 64 over 128 state rows, eight groups) and the gated linear attention (its states as
+# large as those of Nafezen's retention); sixteen gated experts, four choices a token, and a shared one.  `layers` layer runs:
+# two layers run twice.
+def pozirax_config(shape: str, layers: int) -> dict:
+    q, span, ff = SOVUTAR_SHAPES[shape]
+    W, H, D = q["hidden_size"], q["num_attention_heads"], q["head_dim"]
+    left = {"heads": H, "kv_heads": q["num_key_value_heads"], "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": span},
+            "rot": {"base": 1000000.0, "dims": D}}
+    right = {"heads": 2 * W // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    kinds = [("parallel", {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.6}),
+             ("gla", {"heads": H, "dim": D, "vdim": D, "tau": 16.0, "decay_rank": 16})]
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": 16, "top": 4}, "shared": {"ff": ff}}
+    looped = layers >= 4
+    out = [{"type": kinds[i % 2][0], "mixer": json.loads(json.dumps(kinds[i % 2][1])), "mlp": json.loads(json.dumps(moe))}
+           for i in range(layers - 2 if looped else layers)]
+    raw = {"architecture": "Pozirax", "vocab": q["vocab_size"], "width": W, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+           "logit_softcap": 30.0, "layers": out}
+    if looped:
+        raw["loop"] = {"start": 0, "stop": 2, "times": 2}
+    return raw
+
+
+def pozirax_work(raw: dict, tokens: int, batch: int, context: int) -> dict:
+    """Ideal work of the design's kernels, per step: kernel family -> (bytes, flops)."""
+    W = raw["width"]
+    loop = raw.get("loop") or {"start": 0, "stop": 0, "times": 0}
+    runs = raw["layers"] + raw["layers"][loop["start"]:loop["stop"]] * max(loop["times"] - 1, 0)
+    of = lambda kind: [l["mixer"] for l in runs if l["type"] == kind]
+    pairs, glas, L = of("parallel"), of("gla"), len(runs)
+    mlp = raw["layers"][0]["mlp"]
+    E, top, F = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"]
+    decode = tokens == batch
+    active = min(E, batch * top) if decode else E
+    # a layer's norm: the residual in and out, its normed copy, and what the layer before left; a loop's entry as well
+    work = {"group_norm": (tokens * W * ((L + 1) * (4 + 4 + 2) + L * (top + 2) * 4 + (loop["times"] + 1) * (4 + 2)), 0),
+            "moe_route_kernel": (L * (tokens + E) * W * 2, 0),
+            "moe_expert": (L * (active * 3 * W * F * 2 + tokens * top * (W * 2 + F * 4 + W * 4)), L * tokens * top * 2 * 3 * W * F)}
+    if pairs:
+        n, a, s = len(pairs), pairs[0]["left"], pairs[0]["right"]
+        H, G, D, Dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+        window = a["mask"]["size"]
+        keys = min(context, window) if decode else sum(min(i + 1, window) for i in range(tokens)) / tokens
+        cached = batch * (min(context, window) if decode else tokens)
+        work["attn_softcap"] = (n * (cached * G * (D + Dv) * 2 + tokens * H * (D + Dv) * 2), n * tokens * keys * H * 2 * (D + Dv))
+        work["rotary_qkv_store"] = (n * tokens * ((H + G) * D + G * Dv) * (4 + 2 if decode else 2 + 2), 0)
+        h, P, N = s["heads"], s["vdim"], s["state"]
+        inner, channels, state = h * P, h * P + 2 * s["groups"] * N, h * P * N
+        work["causal_conv"] = (n * tokens * channels * 2 * 2, 0)
+        work["conv_state_update"] = (n * batch * channels * (s["conv"] - 1) * 2 * 2, 0)
+        work["state_space_decode"] = (n * (batch * state * 8 + tokens * (inner + channels) * 4 + tokens * inner * 4), n * tokens * state * 4)
+        work["state_space_finish"] = (n * tokens * (inner * 6 + channels * 4), 0)
+        work["state_space_chunk_sum"] = (n * tokens * channels * 2, n * tokens * state * 2)
+        work["state_space_chunk_carry"] = (n * batch * state * 8, 0)
+        work["state_space_chunk_out"] = (n * tokens * (channels * 2 + inner * 4), n * tokens * state * 2)
+        work["gated_norm"] = (n * tokens * inner * (4 + 2 + 2), 0)
+    if glas:
+        n, m = len(glas), glas[0]
+        H, D, Dv = m["heads"], m["dim"], m["vdim"]
+        state = H * D * Dv
+        rows = H * (2 * D + 2 * Dv) * 4 + H * Dv * 2      # q, k, v and the gate in 32 bits, the output in 16
+        work["gated_linear_decode"] = (n * (batch * state * 8 + tokens * rows), n * tokens * state * 4)
+        work["decay_gates"] = (n * tokens * H * D * 4, 0)
+        work["gated_linear_chunk_sum"] = (n * tokens * H * (D + Dv) * 4, n * tokens * state * 2)
+        work["gated_linear_chunk_carry"] = (n * batch * state * 8, 0)
+        work["gated_linear_chunk_out"] = (n * tokens * rows, n * tokens * state * 2)
+    return work
+
+
+def pozirax_bench(args) -> int:
+    """Prefill and decode throughput of the Pozirax design, of Nafezen (the closest design: parallel layers with a linear
+    recurrence and a mixture of experts) and of Qwen3 at the same widths and number of layer runs."""
+    from arle_amd.config import NafezenConfig, PoziraxConfig, Qwen3Config
+
+    layers = args.layers if args.layers != FULL_LAYERS else 8
+    q = dict(SOVUTAR_SHAPES[args.shape][0], num_hidden_layers=layers)
+    raw, naf = pozirax_config(args.shape, layers), nafezen_config(args.shape, layers)
+    models = {"pozirax": ("Pozirax", PoziraxConfig.from_dict(raw)), "nafezen": ("Nafezen", NafezenConfig.from_dict(naf)),
+              "qwen3": ("Qwen3ForCausalLM", Qwen3Config.from_dict(q))}
+    return design_bench(args, "pozirax", models, q, layers, lambda tokens, batch, context: pozirax_work(raw, tokens, batch, context),
+                        {"nafezen": lambda tokens, batch, context: nafezen_work(naf, tokens, batch, context)})
+
+
 def tazitar_bench(args) -> int:
     """Prefill and decode throughput of the Tazitar design and of Qwen3 at the same widths and depth."""
     from arle_amd.config import Qwen3Config, TazitarConfig
@@ -1221,10 +1306,10 @@ def main() -> int:
                          "and write the table that ARLE_AMD_PRODUCT_TABLE / ops.load_product_table reads; WIDTHS: 4b, 8b, "
                          "32b or hidden,q_width,kv_width,intermediate[,vocabulary]")
     ap.add_argument("--out", default=None, help="--tune-products: the table's file (default: product_table_<widths>.json)")
-    ap.add_argument("--workload", default="qwen3-4b", choices=["qwen3-4b", "qwen3-8b-mixed", "qwen3-32b-decode", "gufasun", "sovutar", "tazitar", "retudra", "nafezen"],
+    ap.add_argument("--workload", default="qwen3-4b", choices=["qwen3-4b", "qwen3-8b-mixed", "qwen3-32b-decode", "gufasun", "sovutar", "tazitar", "retudra", "nafezen", "pozirax"],
                     help="qwen3-4b is the default run; the next two are further workloads at larger shapes; gufasun: "
                          "the Gufasun design beside Qwen3 at equal widths and depth (--shape, --layers, --batch, --prompt-len)")
-    ap.add_argument("--shape", default="4b", choices=["4b", "8b"], help="--workload gufasun / sovutar / tazitar / retudra / nafezen: whose widths")
+    ap.add_argument("--shape", default="4b", choices=["4b", "8b"], help="--workload gufasun / sovutar / tazitar / retudra / nafezen / pozirax: whose widths")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path (asked for --gpus {args.gpus})")
@@ -1254,6 +1339,8 @@ def main() -> int:
         return retudra_bench(args)
     if args.workload == "nafezen":
         return nafezen_bench(args)
+    if args.workload == "pozirax":
+        return pozirax_bench(args)
     if args.workload == "qwen3-4b" and args.batch is None:
         args.batch = 8
     if args.workload != "qwen3-4b":

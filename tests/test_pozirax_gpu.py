@@ -166,6 +166,12 @@ ATTENTIONS = [
     (attention(6, 6, 48, 32, 16, 0.2, rot(100.0, 48)), 16, 70),
     (attention(2, 2, 24, 16, 64, 0.2, rot(1000.0, 2)), 16, 140),
     (attention(3, 3, 128, 128, 65, 0.1, rot(1e6, 128)), 64, 140),
+    # heads of one size: in bfloat16 the kernels of the plain softmax
+    (attention(4, 2, 16, 16, 9, 0.35, rot(500.0, 12)), 4, 40),
+    (attention(6, 2, 48, 48, 40, 0.2, rot(1e6, 48)), 16, 150),
+    (attention(8, 1, 64, 64, 17, 0.15, rot(1e4, 64)), 16, 90),
+    (attention(2, 1, 256, 256, 33, 0.08, rot(1e4, 32)), 16, 70),
+    (attention(5, 5, 32, 32, 1, 0.2), 8, 30),
 ]
 
 
@@ -233,6 +239,67 @@ def test_the_sink_takes_its_share_and_scores_below_it_leave_nothing(dtype):
     for c in ((1000,), (1,), (4,)):
         got = run_mixer(part, x, c, dtype=dtype)
         assert float((got.double() - want).abs().max()) < 1e-3 * float(whole.abs().max())
+
+
+SINK_OPS = [
+    # (q heads, kv heads, head size, page, window, segments: (rows now, position of the first), portions' keys in parts)
+    (4, 2, 64, 16, 0, [(300, 0), (1, 200), (5, 63)], 1),
+    (8, 2, 128, 64, 100, [(300, 40), (1, 700), (40, 0), (1, 99), (1, 100)], 1),
+    (6, 3, 48, 16, 17, [(97, 0), (2, 31), (1, 0), (1, 500)], 1),
+    (8, 8, 128, 64, 0, [(200, 300), (150, 0)], 4),
+    (16, 2, 64, 32, 65, [(64, 500)], 3),
+    (2, 1, 256, 16, 33, [(50, 0), (1, 80)], 1),
+    (4, 4, 128, 16, 1, [(140, 3), (1, 5)], 1),
+]
+
+
+@pytest.mark.parametrize("single", [False, True])
+@pytest.mark.parametrize("case", range(len(SINK_OPS)))
+def test_the_plain_softmax_with_a_sink_a_factor_and_a_window_equals_float64(case, single):
+    """Segments of several requests on pages in a shuffled order, sinks of several sizes, rows of the output far apart; decoded
+    rows with their keys split several ways."""
+    nq, nkv, D, page, window, segments, parts = SINK_OPS[case]
+    if single:
+        segments = [(1, start + n - 1) for n, start in segments]
+    S, T = len(segments), sum(n for n, _ in segments)
+    g = torch.Generator().manual_seed(case)
+    per = -(-max(n + start for n, start in segments) // page)
+    order = torch.randperm(S * per + 2, generator=g).to(torch.int32)
+    table = torch.full((S, per), -1, dtype=torch.int32)
+    k_pages = torch.full((S * per + 2, nkv, page, D), float("nan"))
+    v_pages = torch.full((S * per + 2, nkv, D, page), float("nan"))
+    q, sink = rnd((T, nq, D), 3 + case), rnd((nq,), 5, 2.0)
+    sink[0] = 0.0
+    want = torch.zeros(T, nq, D, dtype=torch.float64)
+    row0, at, scale, factor = [0], 0, 1.5 / D ** 0.5, -0.7
+    for s, (n, start) in enumerate(segments):
+        k, v = rnd((start + n, nkv, D), 100 + 10 * case + s), rnd((start + n, nkv, D), 500 + 10 * case + s)
+        first = max(0, start - window + 1) if window else 0
+        for p in range(first // page, -(-(start + n) // page)):
+            pid = int(order[s * per + p])
+            table[s, p] = pid
+            m = min(page, start + n - p * page)
+            k_pages[pid, :, :m] = k[p * page:p * page + m].transpose(0, 1)
+            v_pages[pid, :, :, :m] = v[p * page:p * page + m].permute(1, 2, 0)
+        for t in range(n):
+            pos = start + t
+            lo = max(0, pos - window + 1) if window else 0
+            for h in range(nq):
+                z = (k[lo:pos + 1, h // (nq // nkv)].double() @ q[at + t, h].double()) * scale
+                p = torch.softmax(torch.cat([z, sink[h:h + 1].double()]), dim=0)[:-1]
+                want[at + t, h] = factor * (p @ v[lo:pos + 1, h // (nq // nkv)].double())
+        at += n
+        row0.append(at)
+    lengths = [n for n, _ in segments]
+    for splits in (1, 2, 8) if max(lengths) == 1 else (None,):
+        out = torch.full((T, nq * D + 24), 9.0, dtype=BF16, device=DEV)
+        ops.attn_paged_mfma(q.reshape(T, nq * D).to(DEV, BF16), out[:, 8:8 + nq * D], k_pages.to(DEV, BF16), v_pages.to(DEV, BF16),
+                            table.to(DEV), i32(row0), i32(list(range(S))), i32([start for _, start in segments]),
+                            max_qlen=max(lengths), min_qlen=min(lengths), max_kv_len=max(n + start for n, start in segments),
+                            num_q_heads=nq, num_kv_heads=nkv, head_dim=D, page_size=page, scale=scale, window=window, splits=splits,
+                            portion_splits=None if single else parts, sink=sink.to(DEV), out_scale=factor)
+        close(out[:, 8:8 + nq * D].reshape(T, nq, D), want, BF16, f"splits {splits}", tol=1.2e-2)
+        assert bool((out[:, :8] == 9).all()) and bool((out[:, 8 + nq * D:] == 9).all())
 
 
 def test_decoded_rows_are_prepared_from_the_sums_with_the_same_bits():
