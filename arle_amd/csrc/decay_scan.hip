@@ -121,48 +121,72 @@ __global__ __launch_bounds__(kDsThreads) void decay_scan_kernel(const ScanArgs a
   }
 }
 
-// A thread takes one channel and the up to 64 rows of a chunk; the rows of m lie in LDS, a slice of the middle at a time.
+// A thread takes one channel and the up to 64 rows of a chunk.  R > 0: a middle of up to R, whose weights a thread keeps in
+// registers; R == 0: any, in slices, with the rows' sums in registers.
 constexpr int kGateSlice = 64;
 
-template <typename TW>
+// The logarithm of a decay.  In the running sums an absolute error of 1e-7 is what a float can hold anyway.
+template <bool SUMS>
+__device__ __forceinline__ float log_decay(float z, float inv_tau) {
+  if (SUMS) return -(fmaxf(-z, 0.f) + __logf(1.0f + __expf(-fabsf(z)))) * inv_tau;
+  return -softplus_f(-z) * inv_tau;
+}
+
+template <typename TW, int R, bool SUMS>
 __global__ __launch_bounds__(kDsThreads) void decay_gates_kernel(const float* __restrict__ m, long long m_stride,
                                                                  const TW* __restrict__ w, const float* __restrict__ bias,
-                                                                 float inv_tau, const int* __restrict__ seg_row0,
-                                                                 int segments, int chunk_sums, float* __restrict__ out,
-                                                                 int tokens, int rank, int channels) {
-  __shared__ float ms[kChunkRows][kGateSlice];
+                                                                 float inv_tau, const int* __restrict__ seg_row0, int segments,
+                                                                 float* __restrict__ out, int tokens, int rank, int channels) {
+  constexpr int W = R > 0 ? R : kGateSlice;
+  __shared__ __attribute__((aligned(16))) float ms[kChunkRows][W];
   ChunkAt at;
-  if (chunk_sums) {
+  if (SUMS) {
     at = find_chunk(seg_row0, segments, blockIdx.x);
   } else {
     at = ChunkAt{0, static_cast<int>(blockIdx.x) * kChunkRows, min(kChunkRows, tokens - static_cast<int>(blockIdx.x) * kChunkRows)};
   }
   if (at.rows <= 0) return;
   const int c = blockIdx.y * kDsThreads + threadIdx.x, cc = min(c, channels - 1);
-  float z[kChunkRows];
-#pragma unroll
-  for (int t = 0; t < kChunkRows; ++t) z[t] = 0.f;
-  for (int r0 = 0; r0 < rank; r0 += kGateSlice) {
-    const int n = min(kGateSlice, rank - r0);
-    __syncthreads();                               // the slice before has been read
-    for (int i = threadIdx.x; i < at.rows * n; i += kDsThreads) ms[i / n][i % n] = m[(at.row0 + i / n) * m_stride + r0 + i % n];
-    __syncthreads();
-    const TW* wr = w + static_cast<int64_t>(cc) * rank + r0;
-    for (int r = 0; r < n; ++r) {
-      const float wv = to_float(wr[r]);
-#pragma unroll
-      for (int t = 0; t < kChunkRows; ++t) z[t] = fmaf(wv, ms[t][r], z[t]);   // (rows past the chunk's: dropped below)
-    }
-  }
-  if (c >= channels) return;
-  const float b = bias[c];
+  const float b = bias[cc];
   float sum = 0.f;
+  auto finish = [&](int t, float z) {
+    const float g = log_decay<SUMS>(z + b, inv_tau);
+    sum += g;
+    if (c < channels) out[static_cast<int64_t>(at.row0 + t) * channels + c] = SUMS ? sum : expf(g);
+  };
+  if constexpr (R > 0) {
+    for (int i = threadIdx.x; i < at.rows * R; i += kDsThreads)
+      ms[i / R][i % R] = i % R < rank ? m[(at.row0 + i / R) * m_stride + i % R] : 0.f;
+    float wr[R];
 #pragma unroll
-  for (int t = 0; t < kChunkRows; ++t) {
-    if (t >= at.rows) continue;
-    const float log_decay = -softplus_f(-(z[t] + b)) * inv_tau;
-    sum += log_decay;
-    out[static_cast<int64_t>(at.row0 + t) * channels + c] = chunk_sums ? sum : expf(log_decay);
+    for (int r = 0; r < R; ++r) wr[r] = r < rank ? to_float(w[static_cast<int64_t>(cc) * rank + min(r, rank - 1)]) : 0.f;
+    __syncthreads();
+#pragma unroll 4
+    for (int t = 0; t < at.rows; ++t) {
+      float z = 0.f;
+#pragma unroll
+      for (int r = 0; r < R; ++r) z = fmaf(wr[r], ms[t][r], z);
+      finish(t, z);
+    }
+  } else {
+    float z[kChunkRows];
+#pragma unroll
+    for (int t = 0; t < kChunkRows; ++t) z[t] = 0.f;
+    for (int r0 = 0; r0 < rank; r0 += kGateSlice) {
+      const int n = min(kGateSlice, rank - r0);
+      __syncthreads();                               // the slice before has been read
+      for (int i = threadIdx.x; i < at.rows * n; i += kDsThreads) ms[i / n][i % n] = m[(at.row0 + i / n) * m_stride + r0 + i % n];
+      __syncthreads();
+      const TW* wr = w + static_cast<int64_t>(cc) * rank + r0;
+      for (int r = 0; r < n; ++r) {
+        const float wv = to_float(wr[r]);
+#pragma unroll
+        for (int t = 0; t < kChunkRows; ++t) z[t] = fmaf(wv, ms[t][r], z[t]);   // (rows past the chunk's: dropped below)
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < kChunkRows; ++t)
+      if (t < at.rows) finish(t, z[t]);
   }
 }
 
@@ -170,9 +194,9 @@ __global__ __launch_bounds__(kDsThreads) void decay_gates_kernel(const float* __
 // weight and a factor.  A workgroup a (row, group).
 template <typename T>
 __global__ __launch_bounds__(kDsThreads) void gated_norm_kernel(const float* __restrict__ y, const T* __restrict__ z,
-                                                                      long long z_stride, const float* __restrict__ w, float eps,
-                                                                      float factor, T* __restrict__ out, long long o_stride,
-                                                                      int width, int size) {
+                                                                long long z_stride, const float* __restrict__ w, float eps,
+                                                                float factor, T* __restrict__ out, long long o_stride, int width,
+                                                                int size) {
   extern __shared__ float xs[];
   __shared__ float red[kDsThreads / kWave];
   const int64_t t = blockIdx.x;
@@ -186,6 +210,42 @@ __global__ __launch_bounds__(kDsThreads) void gated_norm_kernel(const float* __r
   const float inv = factor / sqrtf(block_sum<kDsThreads / kWave>(ss, red) / static_cast<float>(size) + eps);
   for (int i = threadIdx.x; i < size; i += kDsThreads)
     out[t * o_stride + first + i] = from_float<T>(xs[i] * inv * w[first + i]);
+}
+
+// A wave a (row, group), four entries a lane and access (sizes that are multiples of 4 up to 256 VPT, aligned rows).
+template <typename T, int VPT>
+__global__ __launch_bounds__(kDsThreads) void gated_norm_vec_kernel(const float* __restrict__ y, const T* __restrict__ z,
+                                                                    long long z_stride, const float* __restrict__ w, float eps,
+                                                                    float factor, T* __restrict__ out, long long o_stride,
+                                                                    int width, int size, int64_t items) {
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * (kDsThreads / kWave) + threadIdx.x / kWave;
+  if (item >= items) return;
+  const int groups = width / size, lane = threadIdx.x % kWave;
+  const int64_t t = item / groups;
+  const int first = static_cast<int>(item % groups) * size;
+  float4 x[VPT], g[VPT], wv[VPT];
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = first + min(4 * (lane + j * kWave), size - 4);
+    x[j] = ld4<float>(y + t * width + i);
+    g[j] = ld4<T>(z + t * z_stride + i);
+    wv[j] = ld4<float>(w + i);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    x[j] = float4{x[j].x * gate_act(g[j].x, kActSilu), x[j].y * gate_act(g[j].y, kActSilu), x[j].z * gate_act(g[j].z, kActSilu),
+                  x[j].w * gate_act(g[j].w, kActSilu)};
+    if (4 * (lane + j * kWave) < size) ss += (x[j].x * x[j].x + x[j].y * x[j].y) + (x[j].z * x[j].z + x[j].w * x[j].w);
+  }
+  const float inv = factor / sqrtf(wave_sum(ss) / static_cast<float>(size) + eps);
+#pragma unroll
+  for (int j = 0; j < VPT; ++j) {
+    const int i = 4 * (lane + j * kWave);
+    if (i < size)
+      st4<T>(out + t * o_stride + first + i, float4{x[j].x * inv * wv[j].x, x[j].y * inv * wv[j].y, x[j].z * inv * wv[j].z,
+                                                    x[j].w * inv * wv[j].w});
+  }
 }
 
 }  // namespace arle
@@ -231,12 +291,23 @@ extern "C" int arle_decay_gates(const float* m, long long m_stride, const void* 
     return static_cast<int>(hipErrorInvalidValue);
   const dim3 grid(blocks, (channels + kDsThreads - 1) / kDsThreads);
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (w_dtype == kF32)
-    decay_gates_kernel<float><<<grid, kDsThreads, 0, s>>>(m, m_stride, static_cast<const float*>(w), bias, inv_tau, seg_row0,
-                                                          segments, chunk_sums, out, tokens, rank, channels);
-  else
-    decay_gates_kernel<bf16><<<grid, kDsThreads, 0, s>>>(m, m_stride, static_cast<const bf16*>(w), bias, inv_tau, seg_row0,
-                                                         segments, chunk_sums, out, tokens, rank, channels);
+#define ARLE_DG(TW, R, SUMS)                                                                                               \
+  decay_gates_kernel<TW, R, SUMS><<<grid, kDsThreads, 0, s>>>(m, m_stride, static_cast<const TW*>(w), bias, inv_tau, seg_row0, \
+                                                              segments, out, tokens, rank, channels)
+#define ARLE_DG_R(TW, SUMS)                    \
+  do {                                         \
+    if (rank <= 16) ARLE_DG(TW, 16, SUMS);     \
+    else if (rank <= 64) ARLE_DG(TW, 64, SUMS);\
+    else ARLE_DG(TW, 0, SUMS);                 \
+  } while (0)
+#define ARLE_DG_S(TW)                                            \
+  do {                                                           \
+    if (chunk_sums) ARLE_DG_R(TW, true); else ARLE_DG_R(TW, false); \
+  } while (0)
+  if (w_dtype == kF32) ARLE_DG_S(float); else ARLE_DG_S(bf16);
+#undef ARLE_DG_S
+#undef ARLE_DG_R
+#undef ARLE_DG
   return launch_status();
 }
 
@@ -249,6 +320,27 @@ extern "C" int arle_gated_group_norm(const float* y, const void* z, long long z_
     return static_cast<int>(hipErrorInvalidValue);
   const int size = width / groups;
   const dim3 grid(tokens, groups);
+  const auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  if (size % 4 == 0 && size <= 2048 && width % 4 == 0 && z_stride % 4 == 0 && o_stride % 4 == 0 && al(y) && al(w) &&
+      reinterpret_cast<uintptr_t>(z) % (dtype == kF32 ? 16 : 8) == 0 && reinterpret_cast<uintptr_t>(out) % (dtype == kF32 ? 16 : 8) == 0) {
+    const int64_t items = static_cast<int64_t>(tokens) * groups;
+    const unsigned blocks = static_cast<unsigned>((items + kDsThreads / kWave - 1) / (kDsThreads / kWave));
+    hipStream_t s = static_cast<hipStream_t>(stream);
+#define ARLE_GNV(T, VPT)                                                                                                   \
+  gated_norm_vec_kernel<T, VPT><<<blocks, kDsThreads, 0, s>>>(y, static_cast<const T*>(z), z_stride, w, eps, factor,       \
+                                                              static_cast<T*>(out), o_stride, width, size, items)
+#define ARLE_GNV_T(T)                        \
+  do {                                       \
+    if (size <= 256) ARLE_GNV(T, 1);         \
+    else if (size <= 512) ARLE_GNV(T, 2);    \
+    else if (size <= 1024) ARLE_GNV(T, 4);   \
+    else ARLE_GNV(T, 8);                     \
+  } while (0)
+    if (dtype == kF32) ARLE_GNV_T(float); else ARLE_GNV_T(bf16);
+#undef ARLE_GNV_T
+#undef ARLE_GNV
+    return launch_status();
+  }
   const size_t lds = static_cast<size_t>(size) * sizeof(float);     // at most 64 KB
   static bool raised = false;
   if (!raised && lds > 48 * 1024) {

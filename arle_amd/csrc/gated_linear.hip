@@ -259,7 +259,7 @@ __global__ __launch_bounds__(kGlThreads) void gated_linear_chunk_carry_kernel(co
 
 // The outputs of a chunk: wave w makes rows 16 w .. + 15 in all columns, norms them and applies the gate.
 template <int NV>
-__global__ __launch_bounds__(kGlThreads) void gated_linear_chunk_out_kernel(const GlChunkArgs a, const float* __restrict__ norm,
+__global__ __launch_bounds__(kGlThreads, NV <= 8 ? 2 : 1) void gated_linear_chunk_out_kernel(const GlChunkArgs a, const float* __restrict__ norm,
                                                                             float eps, void* __restrict__ out, int out_dtype) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const ChunkAt at = find_chunk(a.seg_row0, a.segments, blockIdx.x);
@@ -283,12 +283,6 @@ __global__ __launch_bounds__(kGlThreads) void gated_linear_chunk_out_kernel(cons
   for (int j = 0; j < 4; ++j) p[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int j = 0; j < NV; ++j) o[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float4 v_next[NV];                               // the chunk's values, 64 rows of EP entries over the workgroup
-#pragma unroll
-  for (int x = 0; x < NV; ++x) {
-    const int i = x * kGlThreads + tid, r = min(i / (EP / 4), at.rows - 1), e = min(4 * (i % (EP / 4)), Dv - 4);
-    v_next[x] = ld4<float>(a.y + (at.row0 + r) * a.row_stride + 2 * qw + h * Dv + e);
-  }
   for (int d0 = 0; d0 < D; d0 += kGlSlice) {
     // fetched into registers first: the state's slice, k's slice with its sums, this lane's pieces of q and of its sums
     float4 s_next[NV], k_next[4], kb[4], ke[4], q4[4], b4[4];
@@ -371,6 +365,12 @@ __global__ __launch_bounds__(kGlThreads) void gated_linear_chunk_out_kernel(cons
           }
       }
     }
+  }
+  float4 v_next[NV];                               // the chunk's values, 64 rows of EP entries over the workgroup
+#pragma unroll
+  for (int x = 0; x < NV; ++x) {
+    const int i = x * kGlThreads + tid, r = min(i / (EP / 4), at.rows - 1), e = min(4 * (i % (EP / 4)), Dv - 4);
+    v_next[x] = ld4<float>(a.y + (at.row0 + r) * a.row_stride + 2 * qw + h * Dv + e);
   }
   __syncthreads();                                 // the last slices have been read by every wave
 #pragma unroll

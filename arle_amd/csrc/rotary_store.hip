@@ -138,6 +138,31 @@ __device__ __forceinline__ uint4 summed8(const QkvSums& a, int64_t t, int col) {
   return uint4{pack_bf16x2(s[0], s[1]), pack_bf16x2(s[2], s[3]), pack_bf16x2(s[4], s[5]), pack_bf16x2(s[6], s[7])};
 }
 
+// Values of a step of many rows: 64 rows of a kv head go through LDS, and each entry's 64 are written by one wave, side by
+// side where the rows' positions follow one another (the pages hold an entry's tokens next to each other).
+constexpr int kTurnRows = 64;
+
+__global__ __launch_bounds__(256) void value_store_kernel(const bf16* __restrict__ v, long long v_stride,
+                                                          const int* __restrict__ positions, const int* __restrict__ slot_of_token,
+                                                          const int* __restrict__ block_table, int table_stride,
+                                                          bf16* __restrict__ v_pages, int tokens, int nkv, int Dv, int page_size) {
+  extern __shared__ uint16_t tile[];      // [64][Dv + 2]
+  const int t0 = blockIdx.x * kTurnRows, g = blockIdx.y, units = Dv / 8, row = Dv + 2;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  for (int i = threadIdx.x; i < kTurnRows * units; i += 256) {
+    const int r = i / units, u = i % units;
+    const uint4 raw = *reinterpret_cast<const uint4*>(v + static_cast<int64_t>(min(t0 + r, tokens - 1)) * v_stride + g * Dv + 8 * u);
+    uint32_t* dst = reinterpret_cast<uint32_t*>(tile + r * row + 8 * u);
+    dst[0] = raw.x; dst[1] = raw.y; dst[2] = raw.z; dst[3] = raw.w;
+  }
+  const int t = min(t0 + lane, tokens - 1), pos = positions[t];
+  const int page = block_table[static_cast<int64_t>(slot_of_token[t]) * table_stride + pos / page_size];
+  uint16_t* out = reinterpret_cast<uint16_t*>(v_pages) + (static_cast<int64_t>(page) * nkv + g) * Dv * page_size + pos % page_size;
+  __syncthreads();
+  if (t0 + lane >= tokens) return;
+  for (int d = wave; d < Dv; d += 4) out[static_cast<int64_t>(d) * page_size] = tile[lane * row + d];
+}
+
 // LPH: lanes of a head (a power of two, 8 LPH >= Dk).  A row's lanes: (nq + nkv) LPH for q and k, then Dv / 8 for
 // every head of v.
 template <int LPH, bool SUMS>
@@ -197,15 +222,42 @@ __global__ __launch_bounds__(256) void rotary_qkv_store_x8_kernel(
     return ss;
   };
   if (weight) {
+    float wv[8];
+    if (w_dtype == kF32) {
+      const float4* w4 = reinterpret_cast<const float4*>(static_cast<const float*>(weight) + (live ? 8 * u : 0));
+      const float4 lo = w4[0], hi = w4[1];
+      wv[0] = lo.x; wv[1] = lo.y; wv[2] = lo.z; wv[3] = lo.w;
+      wv[4] = hi.x; wv[5] = hi.y; wv[6] = hi.z; wv[7] = hi.w;
+    } else {
+      const uint4 raw = *reinterpret_cast<const uint4*>(static_cast<const bf16*>(weight) + (live ? 8 * u : 0));
+      const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        wv[2 * i] = __uint_as_float(w[i] << 16);
+        wv[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+      }
+    }
     const float f = 1.0f / sqrtf(head_sum_sq() / static_cast<float>(Dk) + eps);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) x[i] = x[i] * f * load_as_float(weight, w_dtype, live ? 8 * u + i : 0);
+    for (int i = 0; i < 8; ++i) x[i] = x[i] * f * wv[i];
   }
   if (R > 0) {
     const int half = R / 2;
     const float* c_row = cos_t + static_cast<int64_t>(pos) * half;
     const float* s_row = sin_t + static_cast<int64_t>(pos) * half;
-    if (interleaved) {
+    if (interleaved && half % 4 == 0) {      // four pairs a lane, whose angles are one access each
+      const int e = min(4 * u, half - 4);
+      const float4 c4 = ld4<float>(c_row + e), s4 = ld4<float>(s_row + e);
+      const float c[4] = {c4.x, c4.y, c4.z, c4.w}, s[4] = {s4.x, s4.y, s4.z, s4.w};
+      if (4 * u < half) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float a = x[2 * i], b = x[2 * i + 1];
+          x[2 * i] = a * c[i] - b * s[i];
+          x[2 * i + 1] = b * c[i] + a * s[i];
+        }
+      }
+    } else if (interleaved) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int e = 4 * u + i;   // the pair's number
@@ -224,9 +276,16 @@ __global__ __launch_bounds__(256) void rotary_qkv_store_x8_kernel(
       for (int i = 0; i < 8; ++i) other[i] = __shfl(x[i], partner, kWave);
       if (turns) {
         const int e0 = 8 * (first ? u : u - hu);
+        float cs[8], sn[8];
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+          const float4 c4 = ld4<float>(c_row + e0 + 4 * k), s4 = ld4<float>(s_row + e0 + 4 * k);
+          cs[4 * k] = c4.x; cs[4 * k + 1] = c4.y; cs[4 * k + 2] = c4.z; cs[4 * k + 3] = c4.w;
+          sn[4 * k] = s4.x; sn[4 * k + 1] = s4.y; sn[4 * k + 2] = s4.z; sn[4 * k + 3] = s4.w;
+        }
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-          const float c = c_row[e0 + i], s = s_row[e0 + i];
+          const float c = cs[i], s = sn[i];
           x[i] = first ? x[i] * c - other[i] * s : x[i] * c + other[i] * s;
         }
       }
@@ -260,12 +319,26 @@ extern "C" int arle_rotary_qkv_store(void* q, long long q_stride, const void* k,
   hipStream_t s = static_cast<hipStream_t>(stream);
   const auto aligned = [](const void* p, long long stride) { return reinterpret_cast<uintptr_t>(p) % 16 == 0 && stride % 8 == 0; };
   if (dtype != kF32 && Dk % 8 == 0 && Dk <= 512 && Dv % 8 == 0 && (interleaved || rotary_dim % 16 == 0) &&
-      aligned(q, q_stride) && aligned(k, k_stride) && aligned(v, v_stride) && aligned(k_pages, 8)) {
+      aligned(cos_t, 8) && aligned(sin_t, 8) && aligned(q_weight, 8) && aligned(k_weight, 8) && aligned(q, q_stride) && aligned(k, k_stride) && aligned(v, v_stride) && aligned(k_pages, 8)) {
     int lph = 1;
     while (8 * lph < Dk) lph *= 2;
     // a head's lanes lie in one wave (lph divides 64); the values' lanes start at the next multiple of 64
-    const int lanes = ((nq + nkv) * lph + 63) / 64 * 64 + nkv * (Dv / 8);
+    const bool turned = tokens >= kTurnRows && Dv <= 512 && nkv <= 65535;     // the values in a launch of their own
+    const int lanes = ((nq + nkv) * lph + 63) / 64 * 64 + (turned ? 0 : nkv * (Dv / 8));
     if ((lanes + 255) / 256 <= 65535) {
+      if (turned) {
+        const size_t lds = static_cast<size_t>(kTurnRows) * (Dv + 2) * sizeof(uint16_t);     // at most 64 KB
+        static bool raised = false;
+        if (!raised && lds > 48 * 1024) {
+          const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&value_store_kernel),
+                                                   hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);
+          if (e != hipSuccess) return static_cast<int>(e);
+          raised = true;
+        }
+        value_store_kernel<<<dim3((tokens + kTurnRows - 1) / kTurnRows, nkv), 256, lds, s>>>(
+            static_cast<const bf16*>(v), v_stride, positions, slot_of_token, block_table, table_stride, static_cast<bf16*>(v_pages),
+            tokens, nkv, Dv, page_size);
+      }
       const dim3 grid(tokens, (lanes + 255) / 256);
 #define ARLE_ROT_X8(LPH)                                                                                             \
   rotary_qkv_store_x8_kernel<LPH, false><<<grid, 256, 0, s>>>(                                                       \
@@ -315,7 +388,8 @@ extern "C" int arle_rotary_sums_store(const float* sums, int parts, long long pa
   if (tokens == 0) return 0;
   const auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   if (parts < 1 || Dk < 8 || Dk > 512 || Dk % 8 || Dv < 8 || Dv % 8 || rotary_dim < 0 || rotary_dim > Dk || rotary_dim % 2 ||
-      (!interleaved && rotary_dim % 16) || part_stride % 4 || row_stride % 4 || !al(sums) || !al(q_out) || !al(k_pages))
+      (!interleaved && rotary_dim % 16) || part_stride % 4 || row_stride % 4 || !al(sums) || !al(q_out) || !al(k_pages) ||
+      !al(cos_t) || !al(sin_t) || !al(q_weight) || !al(k_weight))
     return static_cast<int>(hipErrorInvalidValue);
   int lph = 1;
   while (8 * lph < Dk) lph *= 2;

@@ -15,6 +15,7 @@
 namespace arle {
 
 constexpr int kConvMaxTaps = 16;
+constexpr int kConvManyRows = 128;   // rows of a step from which on a lane takes several
 constexpr int kConvAdd = 1, kConvSilu = 2;
 
 __device__ __forceinline__ float conv_out(float y, int flags) { return (flags & kConvSilu) ? y / (1.0f + expf(-y)) : y; }
@@ -101,6 +102,80 @@ __global__ void causal_conv_vec_kernel(const T* __restrict__ u, long long u_stri
                                          conv_out(acc[3], add_input)});
 }
 
+// The same for steps of many rows: a lane takes kConvRows rows of its four channels, whose inputs it slides over (each is
+// fetched once, not once a tap), where they and the rows they look back on belong to one request; else row by row.
+constexpr int kConvRows = 8;
+
+template <typename T, int TAPS>
+__global__ void causal_conv_rows_kernel(const T* __restrict__ u, long long u_stride, const T* __restrict__ bias,
+                                        const T* __restrict__ out_bias, const T* __restrict__ w, const T* __restrict__ state,
+                                        const int* __restrict__ slot_of_token, T* __restrict__ out, long long out_stride,
+                                        int tokens, int channels, int add_input) {
+  const int t0 = blockIdx.x * kConvRows, rows = min(kConvRows, tokens - t0);
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+  if (c >= channels) return;
+  const float4 b = bias ? ld4<T>(bias + c) : float4{0.f, 0.f, 0.f, 0.f};
+  const float4 ob = out_bias ? ld4<T>(out_bias + c) : float4{0.f, 0.f, 0.f, 0.f};
+  float wt[4][TAPS];   // four channels' taps are 4 * TAPS consecutive elements
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    const float4 v = ld4<T>(w + static_cast<int64_t>(c) * TAPS + 4 * j);
+    const float e[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) wt[(4 * j + i) / TAPS][(4 * j + i) % TAPS] = e[i];
+  }
+  auto row_out = [&](int t, const float4 (&in)[TAPS]) {      // in[back]: the input `back` rows before row t
+    float acc[4] = {ob.x, ob.y, ob.z, ob.w};
+    const float now[4] = {in[0].x, in[0].y, in[0].z, in[0].w};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = fmaf(wt[i][TAPS - 1], now[i], ((add_input & kConvAdd) ? now[i] : 0.f) + acc[i]);
+#pragma unroll
+    for (int back = 1; back < TAPS; ++back) {
+      const float v[4] = {in[back].x, in[back].y, in[back].z, in[back].w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] = fmaf(wt[i][TAPS - 1 - back], v[i], acc[i]);
+    }
+    st4<T>(out + t * out_stride + c, float4{conv_out(acc[0], add_input), conv_out(acc[1], add_input), conv_out(acc[2], add_input),
+                                           conv_out(acc[3], add_input)});
+  };
+  const int slot = slot_of_token[t0];
+  bool one = t0 >= TAPS - 1;
+  for (int r = one ? 1 - TAPS : 0; r < rows; ++r) one = one && slot_of_token[t0 + r] == slot;
+  if (one) {
+    float4 raw[kConvRows + TAPS - 1];
+#pragma unroll
+    for (int r = 0; r < kConvRows + TAPS - 1; ++r) {
+      const float4 v = ld4<T>(u + static_cast<int64_t>(min(t0 + r - (TAPS - 1), tokens - 1)) * u_stride + c);
+      raw[r] = float4{v.x + b.x, v.y + b.y, v.z + b.z, v.w + b.w};
+    }
+#pragma unroll
+    for (int r = 0; r < kConvRows; ++r) {
+      float4 in[TAPS];
+#pragma unroll
+      for (int back = 0; back < TAPS; ++back) in[back] = raw[r + TAPS - 1 - back];
+      if (r < rows) row_out(t0 + r, in);
+    }
+    return;
+  }
+  for (int r = 0; r < rows; ++r) {
+    const int t = t0 + r, mine_slot = slot_of_token[t];
+    int mine = 0;
+    while (mine < TAPS - 1 && t - mine - 1 >= 0 && slot_of_token[t - mine - 1] == mine_slot) ++mine;
+    float4 in[TAPS];
+#pragma unroll
+    for (int back = 0; back < TAPS; ++back) {
+      if (back <= mine) {
+        const float4 v = ld4<T>(u + (t - back) * u_stride + c);
+        in[back] = float4{v.x + b.x, v.y + b.y, v.z + b.z, v.w + b.w};
+      } else {
+        const int64_t row = static_cast<int64_t>(mine_slot) * (TAPS - 1) + (TAPS - 1 - (back - mine));
+        in[back] = ld4<T>(state + row * channels + c);
+      }
+    }
+    row_out(t, in);
+  }
+}
+
 // One thread a (segment, channel): the new state is the last taps-1 of (old state, this step's inputs).
 __global__ void conv_state_update_kernel(const void* __restrict__ u, long long u_stride, int u_dtype,
                                          const void* __restrict__ bias, int bias_dtype, void* __restrict__ state,
@@ -144,6 +219,21 @@ extern "C" int arle_causal_conv(const void* u, long long u_stride, int u_dtype, 
   if (w && taps >= 2 && taps <= 4 && channels % 4 == 0 && u_stride % 4 == 0 && out_stride % 4 == 0 && at16(u) && at16(out) &&
       at16(state) && at16(w) && at16(bias) && at16(out_bias) && u_dtype == out_dtype && w_dtype == out_dtype && state_dtype == out_dtype &&
       (!bias || bias_dtype == out_dtype) && (!out_bias || ob_dtype == out_dtype)) {
+    if (tokens >= kConvManyRows) {
+      dim3 rgrid((tokens + kConvRows - 1) / kConvRows, (channels / 4 + 255) / 256);
+#define ARLE_CONV_ROWS(T, TAPS)                                                                                     \
+  causal_conv_rows_kernel<T, TAPS><<<rgrid, 256, 0, s>>>(static_cast<const T*>(u), u_stride, static_cast<const T*>(bias), \
+                                                         static_cast<const T*>(out_bias), static_cast<const T*>(w),  \
+                                                         static_cast<const T*>(state), slot_of_token,               \
+                                                         static_cast<T*>(out), out_stride, tokens, channels, add_input)
+      if (out_dtype == kF32) {
+        if (taps == 2) ARLE_CONV_ROWS(float, 2); else if (taps == 3) ARLE_CONV_ROWS(float, 3); else ARLE_CONV_ROWS(float, 4);
+      } else {
+        if (taps == 2) ARLE_CONV_ROWS(bf16, 2); else if (taps == 3) ARLE_CONV_ROWS(bf16, 3); else ARLE_CONV_ROWS(bf16, 4);
+      }
+#undef ARLE_CONV_ROWS
+      return launch_status();
+    }
     dim3 vgrid(tokens, (channels / 4 + 255) / 256);
 #define ARLE_CONV(T, TAPS)                                                                                          \
   causal_conv_vec_kernel<T, TAPS><<<vgrid, 256, 0, s>>>(static_cast<const T*>(u), u_stride, static_cast<const T*>(bias), \

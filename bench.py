@@ -1107,8 +1107,10 @@ def pozirax_work(raw: dict, tokens: int, batch: int, context: int) -> dict:
         window = a["mask"]["size"]
         keys = min(context, window) if decode else sum(min(i + 1, window) for i in range(tokens)) / tokens
         cached = batch * (min(context, window) if decode else tokens)
-        work["attn_softcap"] = (n * (cached * G * (D + Dv) * 2 + tokens * H * (D + Dv) * 2), n * tokens * keys * H * 2 * (D + Dv))
-        work["rotary_qkv_store"] = (n * tokens * ((H + G) * D + G * Dv) * (4 + 2 if decode else 2 + 2), 0)
+        work["attn_mfma" if decode else "attn_prefill"] = (n * (cached * G * (D + Dv) * 2 + tokens * H * (D + Dv) * 2),
+                                                            n * tokens * keys * H * 2 * (D + Dv))
+        work["rotary_qkv_store"] = (n * tokens * ((H + G) * D + (G * Dv if decode else 0)) * (4 + 2 if decode else 2 + 2), 0)
+        work["value_store"] = (n * tokens * G * Dv * 4, 0)
         h, P, N = s["heads"], s["vdim"], s["state"]
         inner, channels, state = h * P, h * P + 2 * s["groups"] * N, h * P * N
         work["causal_conv"] = (n * tokens * channels * 2 * 2, 0)

@@ -551,7 +551,7 @@ def test_the_forms_of_gated_linear_attention_agree_with_float64_from_a_state_on(
             got = ops.gated_linear_decode(stack, *args, **sizes)
             assert torch.equal(ops.gated_linear_decode(d(y), args[0], args[1], args[2], d(state).clone(), *args[4:], **sizes), got)
         close(got, want, out_dtype, f"{form} {out_dtype}", tol=1e-2 if out_dtype == BF16 else 2e-4)
-        close(held, after, F32, "the states", tol=1e-5)
+        close(held, after, F32, "the states", tol=3e-5)
         untouched = [s for s in range(state.shape[0]) if s not in slots]
         assert torch.equal(held.cpu()[untouched], state[untouched]), "other slots keep theirs"
 
