@@ -27,7 +27,7 @@ from .linear import Linear
 class GatedLinearMixer(Part):
     """params: hidden_size, heads, key_dim, value_dim, tau, eps, decay_rank (int, or None: whatever the tensors have)."""
 
-    CHUNKS_FROM = 64    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
+    CHUNKS_FROM = 128    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
 
     graph_safe = True  # rows, slots and lengths are read on the GPU; launches depend on shapes only
 

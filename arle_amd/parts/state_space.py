@@ -31,7 +31,7 @@ class StateSpaceMixer(Part):
     """params: hidden_size, heads, value_dim, state, groups, conv_taps, norm_groups, eps, project_out (bool, default True;
     False: one of a joined pair of mixers, which owns the products in front and behind, and calls `heads`)."""
 
-    CHUNKS_FROM = 32    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
+    CHUNKS_FROM = 72    # rows of the longest portion from which on the form over chunks is ahead of the one row by row
 
     graph_safe = True  # rows, slots and lengths are read on the GPU; launches depend on shapes only
 

@@ -1107,7 +1107,7 @@ def pozirax_work(raw: dict, tokens: int, batch: int, context: int) -> dict:
         window = a["mask"]["size"]
         keys = min(context, window) if decode else sum(min(i + 1, window) for i in range(tokens)) / tokens
         cached = batch * (min(context, window) if decode else tokens)
-        work["attn_mfma" if decode else "attn_prefill"] = (n * (cached * G * (D + Dv) * 2 + tokens * H * (D + Dv) * 2),
+        work["attn_mfma" if decode else "attn_prefill_dma"] = (n * (cached * G * (D + Dv) * 2 + tokens * H * (D + Dv) * 2),
                                                             n * tokens * keys * H * 2 * (D + Dv))
         work["rotary_qkv_store"] = (n * tokens * ((H + G) * D + (G * Dv if decode else 0)) * (4 + 2 if decode else 2 + 2), 0)
         work["value_store"] = (n * tokens * G * Dv * 4, 0)
