@@ -22,7 +22,8 @@ __device__ __forceinline__ float conv_out(float y, int flags) { return (flags & 
 
 __global__ void causal_conv_kernel(const void* __restrict__ u, long long u_stride, int u_dtype,
                                    const void* __restrict__ bias, int bias_dtype, const void* __restrict__ out_bias,
-                                   int ob_dtype, const void* __restrict__ w, int w_dtype, const void* __restrict__ state, int state_dtype,
+                                   int ob_dtype, const void* __restrict__ w, int w_dtype,
+                                   const void* __restrict__ state, int state_dtype,
                                    const int* __restrict__ slot_of_token, void* __restrict__ out,
                                    long long out_stride, int out_dtype, int channels, int taps, int add_input) {
   const int t = blockIdx.x;
@@ -209,7 +210,8 @@ using namespace arle;
 // u [T, channels] rows u_stride apart; out likewise; w [channels, taps] or null (then out = u + bias);
 // state [slots, taps-1, channels]; slot_of_token int32 [T].
 extern "C" int arle_causal_conv(const void* u, long long u_stride, int u_dtype, const void* bias, int bias_dtype,
-                                const void* out_bias, int ob_dtype, const void* w, int w_dtype, const void* state, int state_dtype,
+                                const void* out_bias, int ob_dtype, const void* w, int w_dtype,
+                                const void* state, int state_dtype,
                                 const int* slot_of_token, void* out, long long out_stride, int out_dtype, int tokens,
                                 int channels, int taps, int add_input, void* stream) {
   if (tokens == 0 || channels == 0) return 0;

@@ -168,7 +168,7 @@ ATTENTIONS = [
     (attention(3, 3, 128, 128, 65, 0.1, rot(1e6, 128)), 64, 140),
     # heads of one size: in bfloat16 the kernels of the plain softmax
     (attention(4, 2, 16, 16, 9, 0.35, rot(500.0, 12)), 4, 40),
-    (attention(6, 2, 48, 48, 40, 0.2, rot(1e6, 48)), 16, 150),
+    (attention(6, 2, 48, 48, 41, 0.2, rot(3e5, 48)), 16, 150),
     (attention(8, 1, 64, 64, 17, 0.15, rot(1e4, 64)), 16, 90),
     (attention(2, 1, 256, 256, 33, 0.08, rot(1e4, 32)), 16, 70),
     (attention(5, 5, 32, 32, 1, 0.2), 8, 30),
@@ -596,7 +596,7 @@ def test_a_pair_of_mixers_counts_each_by_its_factor(dtype, case):
 ROUTERS = [
     # (experts, top, width, ff, shared)
     (6, 2, 72, 40, 56), (5, 3, 40, 24, 24), (4, 1, 42, 30, None), (7, 7, 96, 48, 64), (9, 3, 80, 40, 72), (2, 2, 64, 16, 8),
-    (70, 6, 128, 64, 128), (1, 1, 48, 32, 10), (8, 1, 256, 64, 96),
+    (70, 6, 128, 64, 128), (1, 1, 48, 32, 10), (8, 1, 160, 56, 72),
 ]
 
 
